@@ -4,10 +4,14 @@
 // heads; queries arrive already folded into latent space (qa = W_uk^T q), so
 //   score(h, t, j) = (qa[h,t] . c_j + rot(qr[t,h]) . kr_j) * scale
 //   out[h, t]      = sum_j softmax_j(score)[j] * c_j      (W_uv is applied after)
-// with an optional learned sink per head that only joins the denominator.
+// with an optional learned sink per head that only joins the denominator, and
+// an optional sliding window (the query at position p sees p - j < window).
 //
-// latent_append_kernel: RMS-norm of the latent part, interleaved rotary on the
-//   key part (pairs 2i, 2i+1 of the first `dims` entries), store at the slot.
+// latent_inputs_kernel: everything between the fused projection and attention
+//   that is no matrix product: RMS-norm of the latent part, interleaved rotary
+//   on the key part (pairs 2i, 2i+1 of the first `dims` entries), store at the
+//   slot; optionally the RMS norm of a query latent in the same rows, and the
+//   side columns of a parallel layer.
 // latent_attn_kernel: one workgroup per (query token, group of 4 heads,
 //   key split). Key tiles are staged once in LDS (f32, odd row stride) for the
 //   group's heads; each wave owns one head: a lane scores one key of the tile,
@@ -22,38 +26,59 @@
 #define LAT_WAVES 4
 #define LAT_MAXR 8      // R <= 64 * LAT_MAXR
 
+struct LatInParams {
+  const void* z; long ldz;               // [T, R + Dr]
+  const float* nw; float eps;
+  const int* pos; const float* cs; int max_pos;
+  void* cache; long cache_rows; const int* slots;
+  int R, Dr, dims;
+  const void* dq; long lddq; const float* qw; int Rq; void* cq;   // query latent [T, Rq], or Rq == 0
+};
+
 template <typename T>
-__global__ __launch_bounds__(128) void latent_append_kernel(
-    const T* __restrict__ z, long ldz, const float* __restrict__ nw, float eps,
-    const int* __restrict__ pos, const float* __restrict__ cs, int max_pos, T* __restrict__ cache,
-    long cache_rows, const int* __restrict__ slots, int R, int Dr, int dims) {
-  __shared__ float scratch[2];
-  const int t = blockIdx.x;
-  const int slot = slots[t];
-  if (slot < 0 || slot >= cache_rows) return;      // padding row (uniform for the block)
-  const T* zr = z + (size_t)t * ldz;
-  float ss = 0.f;
-  for (int i = threadIdx.x; i < R; i += blockDim.x) {
+__global__ __launch_bounds__(128) void latent_inputs_kernel(LatInParams p, SideCols side) {
+  __shared__ float part[2][2];
+  const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const T* zr = (const T*)p.z + (size_t)t * p.ldz;
+  const T* qr = p.Rq ? (const T*)p.dq + (size_t)t * p.lddq : nullptr;
+  float ss = 0.f, sq = 0.f;
+  for (int i = threadIdx.x; i < p.R; i += 128) {
     const float v = Act<T>::ld(zr + i);
     ss += v * v;
   }
-  ss = block_sum(ss, scratch);
-  const float inv = 1.f / sqrtf(ss / (float)R + eps);
-  T* row = cache + (size_t)slot * (R + Dr);
-  for (int i = threadIdx.x; i < R; i += blockDim.x)
-    Act<T>::st(row + i, Act<T>::ld(zr + i) * inv * nw[i]);
-  const int p = min(max(pos[t], 0), max_pos - 1);
-  const float* csr = cs + (size_t)p * dims;          // [dims/2][2]
-  for (int i = threadIdx.x; i < Dr; i += blockDim.x) {
+  for (int i = threadIdx.x; i < p.Rq; i += 128) {
+    const float v = Act<T>::ld(qr + i);
+    sq += v * v;
+  }
+  ss = wave_sum(ss);
+  sq = wave_sum(sq);
+  if (lane == 0) { part[0][wave] = ss; part[1][wave] = sq; }
+  __syncthreads();
+  if (p.Rq) {
+    const float inv = 1.f / sqrtf((part[1][0] + part[1][1]) / (float)p.Rq + p.eps);
+    T* cq = (T*)p.cq + (size_t)t * p.Rq;
+    for (int i = threadIdx.x; i < p.Rq; i += 128)
+      Act<T>::st(cq + i, Act<T>::ld(qr + i) * inv * p.qw[i]);
+  }
+  side_relu2<T>(side, t);
+  const int slot = p.slots[t];
+  if (slot < 0 || slot >= p.cache_rows) return;    // padding row
+  const float inv = 1.f / sqrtf((part[0][0] + part[0][1]) / (float)p.R + p.eps);
+  T* row = (T*)p.cache + (size_t)slot * (p.R + p.Dr);
+  for (int i = threadIdx.x; i < p.R; i += 128)
+    Act<T>::st(row + i, Act<T>::ld(zr + i) * inv * p.nw[i]);
+  const int pp = min(max(p.pos[t], 0), p.max_pos - 1);
+  const float* csr = p.cs + (size_t)pp * p.dims;     // [dims/2][2]
+  for (int i = threadIdx.x; i < p.Dr; i += 128) {
     float o;
-    if (i < dims) {
+    if (i < p.dims) {
       const float c = csr[(i >> 1) * 2], s = csr[(i >> 1) * 2 + 1];
-      const float u = Act<T>::ld(zr + R + (i & ~1)), v = Act<T>::ld(zr + R + (i | 1));
+      const float u = Act<T>::ld(zr + p.R + (i & ~1)), v = Act<T>::ld(zr + p.R + (i | 1));
       o = (i & 1) ? v * c + u * s : u * c - v * s;
     } else {
-      o = Act<T>::ld(zr + R + i);
+      o = Act<T>::ld(zr + p.R + i);
     }
-    Act<T>::st(row + R + i, o);
+    Act<T>::st(row + p.R + i, o);
   }
 }
 
@@ -68,6 +93,7 @@ struct LatAttnParams {
   void* out;                             // [H, T, R]
   int num_splits, KT;
   float* ws;                             // [splits, T, H, R + 2] when num_splits > 1
+  int window;                            // > 0: keys p - window + 1 .. p only
 };
 
 template <typename T>
@@ -86,15 +112,16 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_attn_kernel(LatAttnParams 
   float* wsr = p.num_splits > 1
       ? p.ws + (((size_t)split * p.T + t) * p.H + h) * (p.R + 2) : nullptr;
 
-  int nk = 0, b = 0;
+  int nk = 0, lo = 0, b = 0;
   if (t < p.cu_q[p.B]) {
     while (b + 1 < p.B && t >= p.cu_q[b + 1]) ++b;
     nk = min(p.pos[t] + 1, p.ctx[b]);
+    if (p.window > 0) lo = min(max(0, p.pos[t] + 1 - p.window), nk);
   }
-  int k0 = 0, k1 = nk;
+  int k0 = lo, k1 = nk;
   if (p.num_splits > 1) {
-    const int per = ((nk + p.num_splits - 1) / p.num_splits + KT - 1) / KT * KT;
-    k0 = min(nk, split * per);
+    const int per = ((nk - lo + p.num_splits - 1) / p.num_splits + KT - 1) / KT * KT;
+    k0 = min(nk, lo + split * per);
     k1 = min(nk, k0 + per);
   }
   // the wave's query in LDS, pre-scaled; its rotary part rotated here
@@ -228,15 +255,16 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_attn2_kernel(LatAttnParams
   T* out = (T*)p.out + ((size_t)h * p.T + t) * p.R;
   float* wsr = p.num_splits > 1
       ? p.ws + (((size_t)split * p.T + t) * p.H + h) * (p.R + 2) : nullptr;
-  int nk = 0, b = 0;
+  int nk = 0, lo = 0, b = 0;
   if (t < p.cu_q[p.B]) {
     while (b + 1 < p.B && t >= p.cu_q[b + 1]) ++b;
     nk = min(p.pos[t] + 1, p.ctx[b]);
+    if (p.window > 0) lo = min(max(0, p.pos[t] + 1 - p.window), nk);
   }
-  int k0 = 0, k1 = nk;
+  int k0 = lo, k1 = nk;
   if (p.num_splits > 1) {
-    const int per = ((nk + p.num_splits - 1) / p.num_splits + KT - 1) / KT * KT;
-    k0 = min(nk, split * per);
+    const int per = ((nk - lo + p.num_splits - 1) / p.num_splits + KT - 1) / KT * KT;
+    k0 = min(nk, lo + split * per);
     k1 = min(nk, k0 + per);
   }
   {
@@ -454,20 +482,21 @@ __global__ __launch_bounds__(64) void latent_combine_kernel(
   }
 }
 
-extern "C" int loqa_latent_append(const void* z, int dt, long ldz, const void* nw, float eps,
+extern "C" int loqa_latent_inputs(const void* z, int dt, long ldz, const void* nw, float eps,
                                   const void* pos, const void* cs, int max_pos, void* cache, int blk,
                                   int nblocks, const void* slots, int T, int R, int Dr, int dims,
-                                  hipStream_t st) {
+                                  const void* dq, long lddq, const void* qw, int Rq, void* cq,
+                                  const void* s_src, long s_src_ld, void* s_dst, long s_dst_ld,
+                                  int s_n, int s_lo, int s_hi, int s_vec, hipStream_t st) {
   if (T <= 0) return 0;
-  const long rows = (long)blk * nblocks;
-  if (dt == 0)
-    hipLaunchKernelGGL(latent_append_kernel<bf16_t>, dim3(T), dim3(128), 0, st, (const bf16_t*)z,
-                       ldz, (const float*)nw, eps, (const int*)pos, (const float*)cs, max_pos,
-                       (bf16_t*)cache, rows, (const int*)slots, R, Dr, dims);
-  else
-    hipLaunchKernelGGL(latent_append_kernel<float>, dim3(T), dim3(128), 0, st, (const float*)z, ldz,
-                       (const float*)nw, eps, (const int*)pos, (const float*)cs, max_pos,
-                       (float*)cache, rows, (const int*)slots, R, Dr, dims);
+  if (R <= 0 || Dr < 0 || dims < 0 || dims > Dr || Rq < 0 || (Rq && (!dq || !qw || !cq)))
+    return (int)hipErrorInvalidValue;
+  const LatInParams p{z, ldz, (const float*)nw, eps, (const int*)pos, (const float*)cs, max_pos,
+                      cache, (long)blk * nblocks, (const int*)slots, R, Dr, dims, dq, lddq,
+                      (const float*)qw, Rq, cq};
+  const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
+  if (dt == 0) hipLaunchKernelGGL(latent_inputs_kernel<bf16_t>, dim3(T), dim3(128), 0, st, p, side);
+  else hipLaunchKernelGGL(latent_inputs_kernel<float>, dim3(T), dim3(128), 0, st, p, side);
   return (int)hipGetLastError();
 }
 
@@ -475,7 +504,7 @@ extern "C" int loqa_latent_attention(
     const void* qa, long qa_st, long qa_sh, const void* qr, long qr_st, long qr_sh, int dt,
     const void* cache, int blk, int nblocks, const void* cu_q, const void* ctx, const void* bt,
     int max_blocks, const void* pos, const void* cs, int max_pos, const void* sink, float scale,
-    int B, int H, int T, int R, int Dr, int dims, void* out, int num_splits, void* ws,
+    int B, int H, int T, int R, int Dr, int dims, void* out, int num_splits, void* ws, int window,
     hipStream_t st) {
   if (T <= 0 || H <= 0) return 0;
   if (R > 64 * LAT_MAXR || R <= 0 || B <= 0) return (int)hipErrorInvalidValue;
@@ -488,6 +517,7 @@ extern "C" int loqa_latent_attention(
   p.cs = (const float*)cs; p.max_pos = max_pos; p.sink = (const float*)sink; p.scale = scale;
   p.B = B; p.H = H; p.T = T; p.R = R; p.Dr = Dr; p.dims = dims; p.out = out;
   p.num_splits = num_splits < 1 ? 1 : num_splits; p.ws = (float*)ws;
+  p.window = window;
   const int W = R + Dr, Ws = W | 1;
   if (W % 2 == 0 && R % 2 == 0 && R <= 128 * LAT_MAXP) {
     const size_t esz = dt == 0 ? 2 : 4;

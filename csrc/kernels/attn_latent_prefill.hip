@@ -10,11 +10,13 @@
 //   B operand and V^T read from LDS with transposed reads.
 // Differences from the Llama kernel: DK != DV (rotary part only in the keys),
 // zero-padded head sizes (DK, DV are the next instantiated sizes), the causal
-// bound comes from each row's absolute position, and a learned per-head sink
-// joins the softmax denominator at the end.
+// bound comes from each row's absolute position (with a sliding window the keys
+// before it are neither gathered nor visited), a learned per-head sink joins the
+// softmax denominator at the end, and the output gate sigmoid(gate) is applied
+// in the epilogue, which writes unpadded heads into rows of any stride.
 //
-// Helpers: latent_gather_kernel copies each sequence's latent rows from its
-// pages into contiguous [sum L, R] / [sum L, Dr] buffers; latent_kfill_kernel
+// Helpers: latent_gather_kernel copies the last cu_k[b + 1] - cu_k[b] latent rows
+// of each sequence from its pages into contiguous [sum L, R] / [sum L, Dr] buffers; latent_kfill_kernel
 // writes the shared rotary key part into every head's key row;
 // rope_pairs_kernel rotates the queries' rotary part in place.
 #include "seqmix.h"
@@ -29,10 +31,13 @@ struct LatPrefillParams {
   const bf16_t* q; long q_st;       // [T, H, DK]
   const bf16_t* k;                  // [sum L, H, DK]
   const bf16_t* v;                  // [sum L, H, DV]
-  bf16_t* o;                        // [T, H, DV]
+  bf16_t* o; long o_ld;             // [T, H * Dv], row stride o_ld
   const int* cu_q; const int* cu_k; const int* pos;
+  const int* ctx;                   // [B] keys in the cache; the buffer holds the last of them
   const float* sink; float scale_log2;
-  int H;
+  int H, Dv, window;
+  const bf16_t* gate; long gate_ld; // [T, H * Dv] or null
+  int runs;                         // output and gate rows can be accessed in runs of four
 };
 
 template <int DK, int DV>
@@ -52,10 +57,17 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
   if (row_lo >= qlen) return;
   const int row_hi = min(qlen - 1, row_lo + LP_WAVES * 32 - 1);
   const int k0 = p.cu_k[b], klen = p.cu_k[b + 1] - k0;
+  const int koff = p.ctx[b] - klen;                       // position of the buffer's first key
   const int qi = row_lo + wave * 32 + (lane & 31);
   const bool valid = qi < qlen;
-  const int qpos = p.pos[q0 + (valid ? qi : row_hi)];
-  const int kend = min(klen, p.pos[q0 + row_hi] + 1);     // positions grow along a sequence
+  // positions relative to the buffer's first key
+  const int qpos = p.pos[q0 + (valid ? qi : row_hi)] - koff;
+  const int kend = min(klen, p.pos[q0 + row_hi] - koff + 1);   // positions grow along a sequence
+  const int first = p.window > 0 ? max(0, p.pos[q0 + row_lo] - koff - p.window + 1) : 0;
+  const int kt0 = first / LP_TILE * LP_TILE;
+  // what this wave's rows see at all
+  const int wpos_lo = p.pos[q0 + min(row_lo + wave * 32, row_hi)] - koff;
+  const int wpos_hi = p.pos[q0 + min(row_lo + wave * 32 + 31, row_hi)] - koff;
 
   bf16x8 qf[NS];
   {
@@ -95,8 +107,8 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
                              : make_uint4(0, 0, 0, 0);
     }
   };
-  fetch(0);
-  for (int kt = 0; kt < kend; kt += LP_TILE) {
+  fetch(kt0);
+  for (int kt = kt0; kt < kend; kt += LP_TILE) {
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < NKC; ++j) {
@@ -110,6 +122,8 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
     }
     __syncthreads();
     if (kt + LP_TILE < kend) fetch(kt + LP_TILE);
+    // a wave whose rows see nothing of this tile only keeps the barriers
+    if (kt > wpos_hi || (p.window > 0 && kt + LP_TILE <= wpos_lo - p.window + 1)) continue;
 
     float16v st[2];
 #pragma unroll
@@ -131,7 +145,7 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
         for (int j = 0; j < 16; ++j) {
           const int key = kt + 32 * t + (j & 3) + 8 * (j >> 2) + 4 * h;
           float sv = st[t][j] * p.scale_log2;
-          if (key >= kend || key > qpos) sv = -INFINITY;
+          if (key >= kend || key > qpos || (p.window > 0 && qpos - key >= p.window)) sv = -INFINITY;
           st[t][j] = sv;
           mx = fmaxf(mx, sv);
         }
@@ -188,28 +202,46 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
     den = l_run * f + exp2f(sk - M);
   }
   const float inv = den > 0.f ? f / den : 0.f;
-  bf16_t* orow = p.o + ((size_t)(q0 + qi) * p.H + head) * DV;
+  bf16_t* orow = p.o + (size_t)(q0 + qi) * p.o_ld + (size_t)head * p.Dv;
+  const bf16_t* grow = p.gate ? p.gate + (size_t)(q0 + qi) * p.gate_ld + (size_t)head * p.Dv : nullptr;
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
 #pragma unroll
     for (int g4 = 0; g4 < 4; ++g4) {
       const int d0 = 32 * dt + 8 * g4 + 4 * h;
-      uint2 w;
-      w.x = pack_bf16x2(acc[dt][4 * g4] * inv, acc[dt][4 * g4 + 1] * inv);
-      w.y = pack_bf16x2(acc[dt][4 * g4 + 2] * inv, acc[dt][4 * g4 + 3] * inv);
-      *reinterpret_cast<uint2*>(orow + d0) = w;
+      if (d0 >= p.Dv) continue;
+      float o4[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o4[i] = acc[dt][4 * g4 + i] * inv;
+      if (p.runs) {
+        if (grow) {
+          float gv[4];
+          ld_run<bf16_t, 4>(grow + d0, gv);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) o4[i] *= sigmoid_fast(gv[i]);
+        }
+        st_run<bf16_t, 4>(orow + d0, o4);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (d0 + i < p.Dv)
+            orow[d0 + i] = f2bf(grow ? o4[i] * sigmoid_fast(bf2f(grow[d0 + i])) : o4[i]);
+      }
     }
 }
 
-// Latent rows of every sequence, gathered from its pages in position order.
+// The last latent rows of every sequence (as many as its share of cu_k), gathered
+// from its pages in position order.
 __global__ __launch_bounds__(256) void latent_gather_kernel(
     const bf16_t* __restrict__ cache, int blk, const int* __restrict__ bt, int max_blocks,
-    const int* __restrict__ cu_k, int R, int Dr, bf16_t* __restrict__ cl, bf16_t* __restrict__ kr) {
+    const int* __restrict__ cu_k, const int* __restrict__ ctx, int R, int Dr,
+    bf16_t* __restrict__ cl, bf16_t* __restrict__ kr) {
   const int b = blockIdx.y;
-  const int k0 = cu_k[b], L = cu_k[b + 1] - k0;
+  const int k0 = cu_k[b], L = cu_k[b + 1] - k0, off = ctx[b] - L;
   const int W = R + Dr;
   for (int j = blockIdx.x * 4 + (threadIdx.x >> 6); j < L; j += gridDim.x * 4) {
-    const bf16_t* src = cache + ((size_t)bt[(size_t)b * max_blocks + j / blk] * blk + j % blk) * W;
+    const int jp = off + j;
+    const bf16_t* src = cache + ((size_t)bt[(size_t)b * max_blocks + jp / blk] * blk + jp % blk) * W;
     for (int c = threadIdx.x & 63; c < W; c += 64) {
       if (c < R) cl[(size_t)(k0 + j) * R + c] = src[c];
       else kr[(size_t)(k0 + j) * Dr + (c - R)] = src[c];
@@ -248,12 +280,12 @@ __global__ __launch_bounds__(256) void rope_pairs_kernel(bf16_t* __restrict__ x,
 }
 
 extern "C" int loqa_latent_gather(const void* cache, int blk, const void* bt, int max_blocks,
-                                  const void* cu_k, int B, int max_len, int R, int Dr, void* cl,
-                                  void* kr, hipStream_t st) {
+                                  const void* cu_k, const void* ctx, int B, int max_len, int R,
+                                  int Dr, void* cl, void* kr, hipStream_t st) {
   if (B <= 0 || max_len <= 0) return 0;
   const dim3 grid(min(1024, (max_len + 3) / 4), B);
   hipLaunchKernelGGL(latent_gather_kernel, grid, dim3(256), 0, st, (const bf16_t*)cache, blk,
-                     (const int*)bt, max_blocks, (const int*)cu_k, R, Dr, (bf16_t*)cl, (bf16_t*)kr);
+                     (const int*)bt, max_blocks, (const int*)cu_k, (const int*)ctx, R, Dr, (bf16_t*)cl, (bf16_t*)kr);
   return (int)hipGetLastError();
 }
 
@@ -273,16 +305,23 @@ extern "C" int loqa_rope_pairs(void* x, long st_t, long st_h, int T, int H, int 
   return (int)hipGetLastError();
 }
 
-// DK in {64, 128, 192, 256}, DV in {64, 128}: callers pad head sizes up.
+// DK in {64, 128, 192, 256}, DV in {64, 128}: callers pad head sizes up; the
+// output keeps the model's value size Dv <= DV.
 extern "C" int loqa_latent_prefill(const void* q, long q_st, const void* k, const void* v, void* o,
-                                   const void* cu_q, const void* cu_k, const void* pos,
-                                   const void* sink, float scale, int B, int H, int max_q, int DK,
-                                   int DV, hipStream_t st) {
+                                   long o_ld, const void* cu_q, const void* cu_k, const void* ctx,
+                                   const void* pos, const void* sink, float scale, int window,
+                                   const void* gate, long gate_ld, int B, int H, int max_q, int DK,
+                                   int DV, int Dv, hipStream_t st) {
   if (B <= 0 || H <= 0 || max_q <= 0) return 0;
+  if (Dv <= 0 || Dv > DV || o_ld < (long)H * Dv || !ctx) return (int)hipErrorInvalidValue;
   LatPrefillParams p;
   p.q = (const bf16_t*)q; p.q_st = q_st; p.k = (const bf16_t*)k; p.v = (const bf16_t*)v;
-  p.o = (bf16_t*)o; p.cu_q = (const int*)cu_q; p.cu_k = (const int*)cu_k; p.pos = (const int*)pos;
+  p.o = (bf16_t*)o; p.o_ld = o_ld; p.cu_q = (const int*)cu_q; p.cu_k = (const int*)cu_k;
+  p.pos = (const int*)pos; p.ctx = (const int*)ctx; p.Dv = Dv; p.window = window;
   p.sink = (const float*)sink; p.scale_log2 = scale * 1.4426950408889634f; p.H = H;
+  p.gate = (const bf16_t*)gate; p.gate_ld = gate_ld;
+  p.runs = Dv % 4 == 0 && o_ld % 4 == 0 && ((size_t)o & 7) == 0 &&
+           (!gate || (gate_ld % 4 == 0 && ((size_t)gate & 7) == 0));
   const dim3 grid((max_q + LP_WAVES * 32 - 1) / (LP_WAVES * 32), H, B);
 #define GO(A, C)                                                                              \
   if (DK == A && DV == C) {                                                                   \

@@ -1,10 +1,13 @@
-// Softmax attention over paged K / V with a sliding window, kept first tokens
-// and score soft-capping, and the launch that prepares its q / k rows.
+// Softmax attention over paged K / V with a sliding window, kept first tokens,
+// score soft-capping and a linear distance bias, and the launch that prepares
+// its q / k rows.
 //
-//   score(i, j) = q_i . k_j * scale;   with cap > 0: cap * tanh(score / cap)
+//   score(i, j) = q_i . k_j * scale;   with cap > 0: cap * tanh(score / cap);
+//                 with slopes: minus slope_h * (i - j)
 //   key j is visible to the query at position p if j <= p and
 //        (window == 0  or  p - j < window  or  j < keep_first)
 //   out_i = softmax_j(score) V,  times sigmoid(gate_i) per entry if a gate is given
+//   (with a sink the denominator also holds exp(sink_h))
 //
 // K pages are [blocks][BLK][G * D], V pages [blocks][BLK][G * Dv]; query head h
 // reads key/value head h / (H / G). Rows find their sequence through cu_q and
@@ -17,7 +20,10 @@
 // position's angles, each head is divided by its root mean square (no weight),
 // q is multiplied by the position's temperature; q out, k into its page, and
 // the value row (its own projection columns, or the k columns as projected)
-// into its page. Statistics, angles and temperature are f32.
+// into its page. Statistics, angles and temperature are f32. Options: a norm
+// over the whole projection, or per head, both with weights and before the
+// rotation; values blended with another layer's value rows of the same tokens;
+// side columns of a parallel layer (seqmix.h).
 //
 // window_attn_keys_kernel (any dtype, any head size up to 512; decode steps,
 // short feeds and the exact f32 mode): a workgroup per (token, key/value head)
@@ -38,7 +44,8 @@
 // contexts the windows are also dealt out to several workgroups per row, whose
 // partial triples a small combine launch merges.
 //
-// window_attn_mfma_kernel (bf16, D and Dv in {64, 128}; prompt portions): a
+// window_attn_mfma_kernel (bf16, D up to 256 and Dv up to 128 in multiples of 8,
+// padded with zeros in LDS to the next built size; prompt portions): a
 // workgroup per (64, 128 or 256 query rows of one sequence, query head); each
 // wave owns 32 rows. The block-table entries of the key range go to LDS once.
 // K and V tiles of 64 keys are gathered from the pages into LDS for all waves
@@ -56,6 +63,8 @@ struct WinAttnParams {
   int B, T, H, G, D, Dv; void* o;
   int ns; float* part;               // key splits over workgroups and their partial results
   const float* sink;                 // [H] or null: exp(sink[h]) joins head h's softmax denominator
+  const float* slopes;               // [H] or null: slopes[h] * (i - j) comes off head h's score
+  long o_ld;                         // row stride of o (head h at column h * Dv)
 };
 
 // K / V pages (and the block table) are read through pointers in the global
@@ -117,23 +126,27 @@ __device__ __forceinline__ int wa_seq_of_row(const int* __restrict__ cu_q, int B
 }
 
 // ------------------------------------------------------------------ q / k rows
+enum { QKN_HEAD = 0, QKN_WHOLE = 1, QKN_HEAD_W = 2 };
+
 template <typename T>
 __global__ __launch_bounds__(256) void qk_prep_append_kernel(
     const T* __restrict__ u, long ldu, int H, int G, int D, int Dv, int v_off,
     const float* __restrict__ cs, int max_pos, int dims, float eps, float coef, int every,
     const int* __restrict__ pos, T* __restrict__ kc, T* __restrict__ vc, long cache_rows,
     const int* __restrict__ kvslots, T* __restrict__ q, const float* __restrict__ qn,
-    const float* __restrict__ kn) {
+    const float* __restrict__ kn, int norm, const T* __restrict__ vf, long vf_ld, float lam,
+    SideCols side) {
   __shared__ float wsum[2][4];
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int p = pos[t];
   const long slot = kvslots[t];
   const bool store = slot >= 0 && slot < cache_rows;
   const T* ur = u + (size_t)t * ldu;
-  // the other norm: q and k RMS-normed over their whole projection, with
-  // weights, before the rotation (then no per-head division)
+  // norm: QKN_HEAD divides each head by its root mean square after the rotation;
+  // QKN_WHOLE is an RMS norm over the whole q and the whole k projection and
+  // QKN_HEAD_W one per head with weights shared by the heads, both before it
   float invq = 1.f, invk = 1.f;
-  if (qn) {
+  if (norm == QKN_WHOLE) {
     float sq = 0.f, sk = 0.f;
     for (int c = threadIdx.x; c < (H + G) * D; c += blockDim.x) {
       const float v = Act<T>::ld(ur + c);
@@ -159,18 +172,33 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(
       const int e = 2 * (lane + 64 * i);
       a[i] = b[i] = 0.f;
       if (e < D) {
+        const bool two = e + 1 < D;
         a[i] = Act<T>::ld(src + e);
-        b[i] = Act<T>::ld(src + e + 1);
+        if (two) b[i] = Act<T>::ld(src + e + 1);
         if (!isq && v_off < 0 && store) {         // the values are the keys as projected
           T* vr = vc + (size_t)slot * G * Dv + (size_t)(job - H) * Dv + e;
           Act<T>::st(vr, a[i]);
-          Act<T>::st(vr + 1, b[i]);
+          if (two) Act<T>::st(vr + 1, b[i]);
         }
-        if (qn) {
+        ss += a[i] * a[i] + b[i] * b[i];
+      }
+    }
+    float inv = 1.f;
+    if (norm == QKN_HEAD_W) inv = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
+    ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int e = 2 * (lane + 64 * i);
+      if (e < D) {
+        if (norm == QKN_WHOLE) {
           const float* wn = isq ? qn + (size_t)job * D + e : kn + (size_t)(job - H) * D + e;
           const float iv = isq ? invq : invk;
           a[i] *= iv * wn[0];
-          b[i] *= iv * wn[1];
+          if (e + 1 < D) b[i] *= iv * wn[1];
+        } else if (norm == QKN_HEAD_W) {
+          const float* wn = (isq ? qn : kn) + e;
+          a[i] *= inv * wn[0];
+          if (e + 1 < D) b[i] *= inv * wn[1];
         }
         if (e < dims) {
           const float c = csr[e], s = csr[e + 1];
@@ -181,8 +209,7 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(
         ss += a[i] * a[i] + b[i] * b[i];
       }
     }
-    ss = wave_sum(ss);
-    float inv = qn ? 1.f : 1.f / sqrtf(ss / (float)D + eps);
+    inv = norm == QKN_HEAD ? 1.f / sqrtf(wave_sum(ss) / (float)D + eps) : 1.f;
     if (isq) inv *= temp;
     T* dst = isq ? q + (size_t)t * H * D + (size_t)job * D
                  : (store ? kc + (size_t)slot * G * D + (size_t)(job - H) * D : nullptr);
@@ -192,15 +219,22 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(
         const int e = 2 * (lane + 64 * i);
         if (e < D) {
           Act<T>::st(dst + e, a[i] * inv);
-          Act<T>::st(dst + e + 1, b[i] * inv);
+          if (e + 1 < D) Act<T>::st(dst + e + 1, b[i] * inv);
         }
       }
     }
   }
   if (v_off >= 0 && store) {
     T* vr = vc + (size_t)slot * G * Dv;
-    for (int c = threadIdx.x; c < G * Dv; c += blockDim.x) vr[c] = ur[v_off + c];
+    if (vf) {                                      // (1 - lam) v + lam v_first
+      const T* fr = vf + (size_t)t * vf_ld;
+      for (int c = threadIdx.x; c < G * Dv; c += blockDim.x)
+        Act<T>::st(vr + c, (1.f - lam) * Act<T>::ld(ur + v_off + c) + lam * Act<T>::ld(fr + c));
+    } else {
+      for (int c = threadIdx.x; c < G * Dv; c += blockDim.x) vr[c] = ur[v_off + c];
+    }
   }
+  side_relu2<T>(side, t);
 }
 
 // ------------------------------------------------------------ few rows, many keys
@@ -267,6 +301,10 @@ __global__ __launch_bounds__(64 * NW) void window_attn_keys_kernel(WinAttnParams
 #pragma unroll
     for (int i = 0; i < VN; ++i) qreg[r][i] = krows ? qs[r * D + kch + i] : 0.f;
   constexpr int VU = NV > 2 ? 4 : 8;                 // value rows in flight per lane (column form)
+  float slope[REP];
+#pragma unroll
+  for (int r = 0; r < REP; ++r)
+    slope[r] = p.slopes ? p.slopes[g * rep + min(r0 + r, rep - 1)] : 0.f;
   for (int wk = sp * NW + wave; wk < nwin; wk += p.ns * NW) {
     const int k0 = (wk < n1 ? wk : w_lo + (wk - n1)) << 6;
     const int j = k0 + jl;
@@ -316,6 +354,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_keys_kernel(WinAttnParams
     for (int r = 0; r < REP; ++r) {
       float sv = s[r] * p.scale;
       if (p.cap > 0.f) sv = p.cap * tanhf(sv / p.cap);
+      sv -= slope[r] * (float)(pq - j);
       if (!seen) sv = -INFINITY;
       const float mn = fmaxf(m[r], wave_max(sv));      // a window holds at least one visible key
       const float e = seen ? expf(sv - mn) : 0.f;
@@ -422,7 +461,7 @@ __global__ __launch_bounds__(64 * NW) void window_attn_keys_kernel(WinAttnParams
     float out = den > 0.f ? num / den : 0.f;
     if (p.gate)
       out *= sigmoid_f(Act<T>::ld((const T*)p.gate + (size_t)t * p.gate_ld + (size_t)h * Dv + e));
-    Act<T>::st((T*)p.o + (size_t)t * p.H * Dv + (size_t)h * Dv + e, out);
+    Act<T>::st((T*)p.o + (size_t)t * p.o_ld + (size_t)h * Dv + e, out);
   }
 }
 
@@ -445,7 +484,7 @@ __global__ __launch_bounds__(128) void window_attn_combine_kernel(WinAttnParams 
     float out = den > 0.f ? num / den : 0.f;
     if (p.gate)
       out *= sigmoid_f(Act<T>::ld((const T*)p.gate + (size_t)t * p.gate_ld + (size_t)h * Dv + e));
-    Act<T>::st((T*)p.o + (size_t)t * p.H * Dv + (size_t)h * Dv + e, out);
+    Act<T>::st((T*)p.o + (size_t)t * p.o_ld + (size_t)h * Dv + e, out);
   }
 }
 
@@ -467,7 +506,9 @@ __device__ __forceinline__ float tanh_fast(float z) {
   return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.885390081777927f * z));
 }
 
-template <int DK, int DV, int WM_WAVES>
+// DK, DV: the sizes in LDS and registers. PAD: the model's sizes p.D <= DK and
+// p.Dv <= DV are smaller (multiples of 8); the rest is zero.
+template <int DK, int DV, int WM_WAVES, bool PAD>
 __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttnParams p) {
   __shared__ __attribute__((aligned(16))) WinMfmaSmem<DK, DV> sm;
   __shared__ int pages[WM_MAXPG];
@@ -476,6 +517,7 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = lane >> 5;
   const int head = blockIdx.y, b = blockIdx.z;
   const int g = head / (p.H / p.G);
+  const int D = PAD ? p.D : DK, Dv = PAD ? p.Dv : DV;
   const int q0 = p.cu_q[b], qlen = p.cu_q[b + 1] - q0;
   // long row blocks (the most keys) start first
   const int nblk = (int)gridDim.x;
@@ -500,11 +542,12 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
 
   bf16x8 qf[NS];
   {
-    const bf16_t* qrow = (const bf16_t*)p.q + (size_t)(q0 + (valid ? qi : row_hi)) * p.H * DK +
-                         (size_t)head * DK;
+    const bf16_t* qrow = (const bf16_t*)p.q + (size_t)(q0 + (valid ? qi : row_hi)) * p.H * D +
+                         (size_t)head * D;
 #pragma unroll
     for (int s = 0; s < NS; ++s) {
-      uint4 v = valid ? *reinterpret_cast<const uint4*>(qrow + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
+      uint4 v = valid && (!PAD || 16 * s + 8 * h < D)
+                    ? *reinterpret_cast<const uint4*>(qrow + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
       qf[s] = *reinterpret_cast<bf16x8*>(&v);
     }
   }
@@ -515,9 +558,9 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     for (int j = 0; j < 16; ++j) acc[i][j] = 0.f;
   float m_run = -1e30f, l_run = 0.f;
   constexpr int CHK = DK / 8, CHV = DV / 8;
-  const size_t kst = (size_t)p.G * DK, vst = (size_t)p.G * DV;
-  const WA_GLOBAL bf16_t* kbase = (const WA_GLOBAL bf16_t*)p.kc + (size_t)g * DK;
-  const WA_GLOBAL bf16_t* vbase = (const WA_GLOBAL bf16_t*)p.vc + (size_t)g * DV;
+  const size_t kst = (size_t)p.G * D, vst = (size_t)p.G * Dv;
+  const WA_GLOBAL bf16_t* kbase = (const WA_GLOBAL bf16_t*)p.kc + (size_t)g * D;
+  const WA_GLOBAL bf16_t* vbase = (const WA_GLOBAL bf16_t*)p.vc + (size_t)g * Dv;
   const WA_GLOBAL int* bt = (const WA_GLOBAL int*)p.bt + (size_t)b * p.max_blocks;
   // the pages of this workgroup's key range, looked up once
   const int npg = (kend + p.blk - 1) / p.blk;
@@ -527,6 +570,7 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     __syncthreads();
   }
   const float scale_log2 = p.scale * 1.4426950408889634f;
+  const float slope_log2 = p.slopes ? p.slopes[head] * 1.4426950408889634f : 0.f;
   const float cap_log2 = p.cap * 1.4426950408889634f, inv_cap = p.cap > 0.f ? p.scale / p.cap : 0.f;
 
   // K / V tiles go through registers: the next tile's 16-byte chunks are
@@ -544,14 +588,14 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
 #pragma unroll
     for (int j = 0; j < NKC; ++j) {
       const int c = threadIdx.x + WM_THREADS * j, kr = c / CHK, cc = (c - kr * CHK) * 8;
-      pk[j] = kt + kr < kend
+      pk[j] = kt + kr < kend && (!PAD || cc < D)
                   ? *reinterpret_cast<const WA_GLOBAL wa_u32x4*>(kbase + page_row(kt + kr) * kst + cc)
                   : wa_u32x4{0, 0, 0, 0};
     }
 #pragma unroll
     for (int j = 0; j < NVC; ++j) {
       const int c = threadIdx.x + WM_THREADS * j, kr = c / CHV, cc = (c - kr * CHV) * 8;
-      pv[j] = kt + kr < kend
+      pv[j] = kt + kr < kend && (!PAD || cc < Dv)
                   ? *reinterpret_cast<const WA_GLOBAL wa_u32x4*>(vbase + page_row(kt + kr) * vst + cc)
                   : wa_u32x4{0, 0, 0, 0};
     }
@@ -593,6 +637,8 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     bf16x8 pf[2][2];
     {
       float mx = -INFINITY;
+      // the distance bias of key kt + c for this lane's query: nb + slope * c
+      const float nb = slope_log2 * (float)(kt + 4 * h - qpos);
       // a tile that every row of this wave sees whole needs no per-score tests
       const bool whole = kt + WM_TILE - 1 <= wpos_lo && kt + WM_TILE <= kend &&
                          (p.window <= 0 || wpos_hi - kt < p.window || kt + WM_TILE <= p.keep_first);
@@ -601,8 +647,9 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
         for (int t = 0; t < 2; ++t)
 #pragma unroll
           for (int j = 0; j < 16; ++j) {
-            const float sv = p.cap > 0.f ? cap_log2 * tanh_fast(st[t][j] * inv_cap)
-                                         : st[t][j] * scale_log2;
+            const float sv = (p.cap > 0.f ? cap_log2 * tanh_fast(st[t][j] * inv_cap)
+                                          : st[t][j] * scale_log2) +
+                             (nb + slope_log2 * (float)(32 * t + (j & 3) + 8 * (j >> 2)));
             st[t][j] = sv;
             mx = fmaxf(mx, sv);
           }
@@ -612,7 +659,9 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
 #pragma unroll
           for (int j = 0; j < 16; ++j) {
             const int key = kt + 32 * t + (j & 3) + 8 * (j >> 2) + 4 * h;
-            float sv = p.cap > 0.f ? cap_log2 * tanh_fast(st[t][j] * inv_cap) : st[t][j] * scale_log2;
+            float sv = (p.cap > 0.f ? cap_log2 * tanh_fast(st[t][j] * inv_cap)
+                                    : st[t][j] * scale_log2) +
+                       (nb + slope_log2 * (float)(32 * t + (j & 3) + 8 * (j >> 2)));
             if (key >= kend || key > qpos ||
                 (p.window > 0 && qpos - key >= p.window && key >= p.keep_first))
               sv = -INFINITY;
@@ -674,14 +723,15 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     const float a = __builtin_amdgcn_exp2f(m_run - mx2);
     inv = a / (l_run * a + __builtin_amdgcn_exp2f(sl - mx2));
   }
-  bf16_t* orow = (bf16_t*)p.o + ((size_t)(q0 + qi) * p.H + head) * DV;
-  const bf16_t* grow = p.gate ? (const bf16_t*)p.gate + (size_t)(q0 + qi) * p.gate_ld + (size_t)head * DV
+  bf16_t* orow = (bf16_t*)p.o + (size_t)(q0 + qi) * p.o_ld + (size_t)head * Dv;
+  const bf16_t* grow = p.gate ? (const bf16_t*)p.gate + (size_t)(q0 + qi) * p.gate_ld + (size_t)head * Dv
                               : nullptr;
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
 #pragma unroll
     for (int g8 = 0; g8 < 4; ++g8) {
       const int d0 = 32 * dt + 8 * g8 + 4 * h;
+      if (PAD && d0 >= Dv) continue;
       float o4[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) o4[i] = acc[dt][4 * g8 + i] * inv;
@@ -710,14 +760,26 @@ int window_attention_mfma(const WinAttnParams& p, int max_q, hipStream_t st) {
 #define GO(A, C)                                                                              \
   if (p.D == A && p.Dv == C) {                                                                \
     if (waves == 8)                                                                           \
-      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 8>), grid, dim3(512), 0, st, p);      \
+      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 8, false>), grid, dim3(512), 0, st, p); \
     else if (waves == 4)                                                                      \
-      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 4>), grid, dim3(256), 0, st, p);      \
+      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 4, false>), grid, dim3(256), 0, st, p); \
     else                                                                                      \
-      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 2>), grid, dim3(128), 0, st, p);      \
+      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 2, false>), grid, dim3(128), 0, st, p); \
     return (int)hipGetLastError();                                                            \
   }
   GO(64, 64) GO(128, 64) GO(64, 128) GO(128, 128)
+#undef GO
+  // other sizes: the next built size, in two block widths
+  const dim3 grid_p = waves == 8 ? grid : dim3((max_q + 63) / 64, p.H, p.B);
+#define GO(A, C)                                                                              \
+  if (p.D <= A && p.Dv <= C) {                                                                \
+    if (waves == 8)                                                                           \
+      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 8, true>), grid_p, dim3(512), 0, st, p); \
+    else                                                                                      \
+      hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 2, true>), grid_p, dim3(128), 0, st, p); \
+    return (int)hipGetLastError();                                                            \
+  }
+  GO(64, 64) GO(64, 128) GO(128, 64) GO(128, 128) GO(256, 64) GO(256, 128)
 #undef GO
   return (int)hipErrorInvalidValue;
 }
@@ -727,17 +789,22 @@ extern "C" int loqa_qk_prep_append(const void* u, int dt, long ldu, int H, int G
                                    int v_off, const void* cs, int max_pos, int dims, float eps,
                                    float coef, int every, const void* pos, void* kc, void* vc,
                                    int blk, int nblocks, const void* kvslots, void* q, int T,
-                                   const void* qn, const void* kn, hipStream_t st) {
+                                   const void* qn, const void* kn, int norm, const void* vf,
+                                   long vf_ld, float lam, const void* s_src, long s_src_ld,
+                                   void* s_dst, long s_dst_ld, int s_n, int s_lo, int s_hi,
+                                   int s_vec, hipStream_t st) {
   if (T <= 0) return 0;
-  if (D <= 0 || D > 512 || D % 2 || dims < 0 || dims > D || dims % 2 || every < 1 ||
-      (dims > 0 && (!cs || max_pos <= 0)) || H <= 0 || G <= 0 || (!qn) != (!kn))
+  if (D <= 0 || D > 512 || dims < 0 || dims > D || dims % 2 || every < 1 ||
+      (dims > 0 && (!cs || max_pos <= 0)) || H <= 0 || G <= 0 || norm < QKN_HEAD ||
+      norm > QKN_HEAD_W || (norm != QKN_HEAD && (!qn || !kn)) || (vf && v_off < 0))
     return (int)hipErrorInvalidValue;
+  const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
   const long rows = (long)blk * nblocks;
 #define GO(TT)                                                                                  \
   hipLaunchKernelGGL(qk_prep_append_kernel<TT>, dim3(T), dim3(256), 0, st, (const TT*)u, ldu, H, \
                      G, D, Dv, v_off, (const float*)cs, max_pos, dims, eps, coef, every,        \
                      (const int*)pos, (TT*)kc, (TT*)vc, rows, (const int*)kvslots, (TT*)q,      \
-                     (const float*)qn, (const float*)kn)
+                     (const float*)qn, (const float*)kn, norm, (const TT*)vf, vf_ld, lam, side)
   if (dt == 0) GO(bf16_t); else GO(float);
 #undef GO
   return (int)hipGetLastError();
@@ -748,10 +815,11 @@ extern "C" int loqa_window_attention(const void* q, int dt, const void* kc, cons
                                      int max_blocks, const void* pos, const void* gate, long gate_ld,
                                      float scale, float cap, int window, int keep_first, int B,
                                      int T, int H, int G, int D, int Dv, int max_q, int mfma,
-                                     void* o, int ns, void* part, const void* sink,
-                                     hipStream_t st) {
+                                     void* o, long o_ld, int ns, void* part, const void* sink,
+                                     const void* slopes, hipStream_t st) {
   if (T <= 0) return 0;
-  if (B <= 0 || H <= 0 || G <= 0 || H % G || D <= 0 || D > 512 || Dv <= 0 || Dv > 512 || blk <= 0)
+  if (B <= 0 || H <= 0 || G <= 0 || H % G || D <= 0 || D > 512 || Dv <= 0 || Dv > 512 || blk <= 0 ||
+      o_ld < (long)H * Dv)
     return (int)hipErrorInvalidValue;
   WinAttnParams p;
   p.q = q; p.kc = kc; p.vc = vc; p.blk = blk; p.cache_rows = (long)blk * nblocks;
@@ -760,9 +828,11 @@ extern "C" int loqa_window_attention(const void* q, int dt, const void* kc, cons
   p.scale = scale; p.cap = cap; p.window = window; p.keep_first = keep_first;
   p.B = B; p.T = T; p.H = H; p.G = G; p.D = D; p.Dv = Dv; p.o = o;
   p.ns = 1; p.part = nullptr; p.sink = (const float*)sink;
-  // the matrix-core form reads the gate in 8-byte runs
-  const bool gate_ok = !gate || (gate_ld % 4 == 0 && ((size_t)gate & 7) == 0);
-  if (mfma && dt == 0 && (D == 64 || D == 128) && (Dv == 64 || Dv == 128) && gate_ok)
+  p.slopes = (const float*)slopes; p.o_ld = o_ld;
+  // the matrix-core form reads the gate and writes the output in 8-byte runs
+  const bool runs_ok = (!gate || (gate_ld % 4 == 0 && ((size_t)gate & 7) == 0)) && o_ld % 4 == 0 &&
+                       ((size_t)o & 7) == 0;
+  if (mfma && dt == 0 && D % 8 == 0 && D <= 256 && Dv % 8 == 0 && Dv <= 128 && runs_ok)
     return window_attention_mfma(p, max_q, st);
   const int rep = H / G;
   // value layout: whole rows in 16-byte runs when Dv / (elements per run) is a

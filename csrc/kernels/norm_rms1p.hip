@@ -12,7 +12,8 @@
 //                             run side by side on norms of the same x
 //   rms_norm_cols_kernel:     y = u[:, :n] / sqrt(mean(.^2) + eps) * w, a plain-weight
 //                             norm over a column slice of a fused projection
-//   sigmoid_gate_kernel:      o[t, h, :Dv] *= sigmoid(gate[t, h Dv]) (heads may be padded)
+//   sigmoid_gate_kernel:      out[t, h Dv] = o[t, h, :Dv] * sigmoid(gate[t, h Dv]); o by
+//                             strides (padded heads, head-major), out may be o itself
 //   softcap_kernel:           x <- cap tanh(x / cap)
 //
 // One workgroup per row. A row of up to 4096 entries (a multiple of 4) stays
@@ -191,14 +192,16 @@ __global__ __launch_bounds__(R1_THREADS) void rms_norm_cols_kernel(
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void sigmoid_gate_kernel(T* __restrict__ o,
+__global__ __launch_bounds__(256) void sigmoid_gate_kernel(const T* o, long o_st, long o_sh,
                                                            const T* __restrict__ gate, long ldg,
-                                                           int H, int Dvo, int Dv) {
+                                                           T* out, long out_st, long out_sh, int H,
+                                                           int Dv) {
   const size_t t = blockIdx.x;
   for (int i = blockIdx.y * blockDim.x + threadIdx.x; i < H * Dv; i += gridDim.y * blockDim.x) {
     const int h = i / Dv, e = i % Dv;
-    T* p = o + (t * H + h) * Dvo + e;
-    Act<T>::st(p, Act<T>::ld(p) * sigmoid_for<T>(Act<T>::ld(gate + t * ldg + i)));
+    const float v = Act<T>::ld(o + t * o_st + h * o_sh + e);
+    Act<T>::st(out + t * out_st + h * out_sh + e,
+               v * sigmoid_for<T>(Act<T>::ld(gate + t * ldg + i)));
   }
 }
 
@@ -275,17 +278,18 @@ extern "C" int loqa_rms_norm_cols(const void* u, int u_dt, long ldu, int n, cons
   return (int)hipGetLastError();
 }
 
-extern "C" int loqa_sigmoid_gate(void* o, int dt, const void* gate, long ldg, int T, int H, int Dvo,
-                                 int Dv, hipStream_t st) {
+extern "C" int loqa_sigmoid_gate(const void* o, long o_st, long o_sh, int dt, const void* gate,
+                                 long ldg, void* out, long out_st, long out_sh, int T, int H, int Dv,
+                                 hipStream_t st) {
   if (T <= 0) return 0;
-  if (H <= 0 || Dv <= 0 || Dvo < Dv) return (int)hipErrorInvalidValue;
+  if (H <= 0 || Dv <= 0) return (int)hipErrorInvalidValue;
   const dim3 grid(T, T >= 512 ? 1 : (H * Dv + 255) / 256);
   if (dt == 0)
-    hipLaunchKernelGGL(sigmoid_gate_kernel<bf16_t>, grid, dim3(256), 0, st, (bf16_t*)o,
-                       (const bf16_t*)gate, ldg, H, Dvo, Dv);
+    hipLaunchKernelGGL(sigmoid_gate_kernel<bf16_t>, grid, dim3(256), 0, st, (const bf16_t*)o, o_st,
+                       o_sh, (const bf16_t*)gate, ldg, (bf16_t*)out, out_st, out_sh, H, Dv);
   else
-    hipLaunchKernelGGL(sigmoid_gate_kernel<float>, grid, dim3(256), 0, st, (float*)o,
-                       (const float*)gate, ldg, H, Dvo, Dv);
+    hipLaunchKernelGGL(sigmoid_gate_kernel<float>, grid, dim3(256), 0, st, (const float*)o, o_st,
+                       o_sh, (const float*)gate, ldg, (float*)out, out_st, out_sh, H, Dv);
   return (int)hipGetLastError();
 }
 

@@ -35,4 +35,65 @@ template <typename T> __device__ __forceinline__ float sigmoid_for(float z) {
   return sizeof(T) == 2 ? sigmoid_fast(z) : sigmoid_f(z);
 }
 
+// Runs of N neighbouring entries (N = 4: one 16- or 8-byte access, N = 1: one
+// entry) as f32.
+template <typename T, int N> __device__ __forceinline__ void ld_run(const T* p, float* f) {
+  if constexpr (N == 1) {
+    f[0] = Act<T>::ld(p);
+  } else if constexpr (sizeof(T) == 4) {
+    const float4 v = *reinterpret_cast<const float4*>(p);
+    f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
+  } else {
+    const uint2 r = *reinterpret_cast<const uint2*>(p);
+    f[0] = __uint_as_float(r.x << 16); f[1] = __uint_as_float(r.x & 0xffff0000u);
+    f[2] = __uint_as_float(r.y << 16); f[3] = __uint_as_float(r.y & 0xffff0000u);
+  }
+}
+template <typename T, int N> __device__ __forceinline__ void st_run(T* p, const float* f) {
+  if constexpr (N == 1) {
+    Act<T>::st(p, f[0]);
+  } else if constexpr (sizeof(T) == 4) {
+    *reinterpret_cast<float4*>(p) = make_float4(f[0], f[1], f[2], f[3]);
+  } else {
+    uint2 r;
+    r.x = pack_bf16x2(f[0], f[1]);
+    r.y = pack_bf16x2(f[2], f[3]);
+    *reinterpret_cast<uint2*>(p) = r;
+  }
+}
+
+// Side columns of a parallel layer's fused projection: the ungated feed-forward
+// reads the same input as the mixer, so its up projection is a column slice of
+// the same matrix product. src [T, src_ld] (the slice's first column) ->
+// dst[t, 0 .. n) = relu(src)^2, and zeros in the columns zero_lo .. 0 (negative
+// offsets: padding before the slice) and n .. zero_hi. One workgroup per token
+// calls it with its row; vec: rows and bases are aligned for runs of four.
+struct SideCols {
+  const void* src; long src_ld;
+  void* dst; long dst_ld;
+  int n, zero_lo, zero_hi, vec;
+};
+template <typename T>
+__device__ __forceinline__ void side_relu2(const SideCols& s, size_t t) {
+  if (!s.dst) return;
+  const T* a = (const T*)s.src + t * s.src_ld;
+  T* o = (T*)s.dst + t * s.dst_ld;
+  if (s.vec) {
+    for (int c = 4 * threadIdx.x; c < s.n; c += 4 * blockDim.x) {
+      float f[4];
+      ld_run<T, 4>(a + c, f);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) { f[i] = fmaxf(f[i], 0.f); f[i] *= f[i]; }
+      st_run<T, 4>(o + c, f);
+    }
+  } else {
+    for (int c = threadIdx.x; c < s.n; c += blockDim.x) {
+      const float f = fmaxf(Act<T>::ld(a + c), 0.f);
+      Act<T>::st(o + c, f * f);
+    }
+  }
+  for (int c = s.zero_lo + (int)threadIdx.x; c < 0; c += blockDim.x) Act<T>::st(o + c, 0.f);
+  for (int c = s.n + (int)threadIdx.x; c < s.zero_hi; c += blockDim.x) Act<T>::st(o + c, 0.f);
+}
+
 static inline int ceil_div(long a, long b) { return (int)((a + b - 1) / b); }

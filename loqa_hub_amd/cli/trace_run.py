@@ -35,8 +35,7 @@ def build_engine(model_dir: str, dtype: str, max_tokens: int, device=None, block
     cfg = lm_config_of_checkpoint(model_dir, os.path.basename(os.path.normpath(model_dir)))
     if dt == torch.float32 and not family_of(cfg).hybrid:
         raise SystemExit(3)          # that family is served in bfloat16 only
-    if device is None:
-        device = "cuda:0" if torch.cuda.is_available() else "cpu"
+    device = device or "cuda:0"      # the CPU reference ops only when asked for by name
     if dt == torch.float32:
         # true 32-bit matrix products
         torch.backends.cuda.matmul.allow_tf32 = False

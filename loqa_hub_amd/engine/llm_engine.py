@@ -260,6 +260,12 @@ class LLMEngine:
             np.cumsum(ctx[:B_pad], out=cu_k[1:])
             host["cu_k"] = cu_k
             host["total_k"] = int(cu_k[-1])
+            # prompt passes of windowed latent attention gather the last keys only
+            for w in (getattr(self.model, "key_windows", ())
+                      if max_q >= getattr(self.model, "prompt_min_q", 0) else ()):
+                cu_w = np.zeros(B_pad + 1, np.int32)
+                np.cumsum(np.minimum(ctx[:B_pad], np.diff(cu[:B_pad + 1]) + (w - 1)), out=cu_w[1:])
+                host[f"cu_k_{w}"], host[f"total_k_{w}"] = cu_w, int(cu_w[-1])
         return max_q, max_ctx, host
 
     def _to_device(self, host: dict, dst: dict | None = None) -> dict:
@@ -328,7 +334,10 @@ class LLMEngine:
                         cu_q=dev["cu_q"], ctx_lens=dev["ctx_lens"], block_tables=dev["block_tables"],
                         logit_idx=dev["logit_idx"], max_q=max_q, max_ctx=max_ctx, decode=decode,
                         state_slots=dev.get("state_slots"), cu_k=dev.get("cu_k"),
-                        total_k=dev.get("total_k", 0))
+                        total_k=dev.get("total_k", 0),
+                        window_k={w: (dev[f"cu_k_{w}"], dev[f"total_k_{w}"])
+                                  for w in getattr(self.model, "key_windows", ())
+                                  if f"cu_k_{w}" in dev})
 
     CTX_BUCKET = 256
 

@@ -242,6 +242,7 @@ class LatentAttnConfig:
     kv_from: int | None = None      # reuse that layer's latent cache
     q_rank: int = 0                 # > 0: queries go through an RMS-normed latent of this size
     gate: bool = False              # heads' outputs times sigmoid(W_g h), per entry
+    window: int = 0                 # key j visible if p - j < window; 0: every earlier key
 
 
 @dataclass(frozen=True)
@@ -438,9 +439,13 @@ class SoftmaxAttnConfig:
     keep_first: int = 0             # ... or j < keep_first
     # "head": q and k divided by their root mean square per head after rotation,
     # no weight; "whole": RMS norm over the whole q (and k) projection with a
-    # weight vector of that size, before rotation
+    # weight vector of that size, before rotation; "head_weight": RMS norm per
+    # head with a weight of the head's size shared by the heads, before rotation
     qk_norm: str = "head"
     zero_sink: bool = False         # the softmax denominator holds one more term exp(0)
+    sink: bool = False              # ... one more term exp(sink_h), learned per head
+    alibi: bool = False             # slope_h (i - j) comes off the score (geometric slopes)
+    v_mix: bool = False             # values blended with the first such layer's values
 
 
 @dataclass(frozen=True)
@@ -688,3 +693,75 @@ def vilulix_config_from_json(d: dict, name: str = "vilulix") -> VilulixConfig:
             loop = None
     return VilulixConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]),
                          float(d.get("logit_softcap") or 0.0), tuple(layers), loop)
+
+
+# --------------------------------------------------------------------------
+# Gopopel: a decoder of parallel layers with ONE Dynamic-Tanh norm each, h =
+# norm(x); x <- x + mixer(h) + ff(h), and a scaled embedding. Mixers: sliding-
+# window softmax attention (per-head q / k norms with weights, a linear distance
+# bias, a learned sink, values blended with the first such layer's) and sliding-
+# window latent attention with a query latent and an output gate. Ungated
+# squared-relu feed-forwards. Every size and constant comes from config.json or
+# a tensor's shape.
+@dataclass(frozen=True)
+class GopopelConfig:
+    name: str
+    vocab_size: int
+    d_model: int
+    norm_eps: float
+    embed_scale: float
+    layers: tuple
+
+    @property
+    def n_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def first_v_mix(self) -> int:
+        """The layer whose values the later value-mixing layers blend in (-1: none)."""
+        return next((i for i, lc in enumerate(self.layers)
+                     if lc.kind == "attention" and lc.mixer.v_mix), -1)
+
+
+def gopopel_config_from_json(d: dict, name: str = "gopopel") -> GopopelConfig:
+    layers = []
+    for i, L in enumerate(d["layers"]):
+        m, kind = L["mixer"], L["type"]
+        window = int((m.get("mask") or {}).get("size") or 0)
+        if window < 0:
+            raise ValueError(f"layer {i}: mask size must be positive")
+        if kind == "attention":
+            mixer = SoftmaxAttnConfig(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]),
+                                      int(m.get("vdim", m["dim"])), float(m["scale"]),
+                                      window=window, qk_norm="head_weight", sink=True, alibi=True,
+                                      v_mix=bool(m.get("v_mix")))
+            if mixer.heads % mixer.kv_heads:
+                raise ValueError(f"layer {i}: {mixer.heads} heads do not split over "
+                                 f"{mixer.kv_heads} key/value heads")
+        elif kind == "latent_attention":
+            r, rot_dim = m["rot"], int(m["rot_dim"])
+            rot = RotaryConfig(int(r["dims"]), float(r["base"]))
+            if rot.dims % 2 or not 0 <= rot.dims <= rot_dim:
+                raise ValueError(f"layer {i}: rot.dims {rot.dims} does not fit {rot_dim} entries")
+            mixer = LatentAttnConfig(int(m["heads"]), int(m["dim"]), rot_dim, int(m["vdim"]),
+                                     int(m["kv_rank"]), float(m["scale"]), rot,
+                                     q_rank=int(m["q_rank"]), gate=True, window=window)
+            if mixer.q_rank < 1 or mixer.kv_rank < 1:
+                raise ValueError(f"layer {i}: latent sizes must be positive")
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        f = L.get("mlp")
+        if not f:
+            mlp = None
+        elif f["kind"] == "dense":
+            mlp = FeedForwardConfig("dense", int(f["ff"]), act="relu2")
+        else:
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+        layers.append(HybridLayerConfig(kind, mixer, mlp))
+    mix = [(i, lc.mixer) for i, lc in enumerate(layers) if lc.kind == "attention" and lc.mixer.v_mix]
+    for i, m in mix:
+        if m.kv_heads * m.vdim != mix[0][1].kv_heads * mix[0][1].vdim:
+            raise ValueError(f"layer {i}: its values are not as wide as those of layer "
+                             f"{mix[0][0]}, which they are mixed with")
+    return GopopelConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]),
+                         float((d.get("embedding") or {}).get("scale", 1.0)), tuple(layers))

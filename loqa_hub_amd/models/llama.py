@@ -51,6 +51,9 @@ class StepMeta:
     # and the buffer's row count (latent attention's prompt path)
     cu_k: torch.Tensor | None = None
     total_k: int = 0
+    # the same for the keys that a sliding window of that size leaves visible to
+    # some row of the step: {window: (cu_k, total_k)}
+    window_k: dict | None = None
 
 
 class TPGroup:

@@ -40,11 +40,11 @@ from .configs import PipizenConfig
 
 def latent_prompt_layout(L: dict, m, dtype, device) -> None:
     """Padded per-head copies for the matrix-core prompt kernel (bf16): the
-    query projection ``wq`` with DKp rows per head, W_uk / W_uv producing [H,
-    DKp] keys and [H, DVp] values from a latent row, and W_o with DVp columns
-    per head. Sizes that the kernel is built for are used as they are. ``L``
-    holds ``wq`` [H (D + Dr), n], ``wuk`` [H, D, R], ``wuv_t`` [H, R, Dv] and
-    ``wo``; shared by every family with latent attention layers."""
+    query projection ``wq`` with DKp rows per head and W_uk / W_uv producing [H,
+    DKp] keys and [H, DVp] values from a latent row. Sizes that the kernel is
+    built for are used as they are. ``L`` holds ``wq`` [H (D + Dr), n], ``wuk``
+    [H, D, R] and ``wuv_t`` [H, R, Dv]; shared by every family with latent
+    attention layers."""
     H, D, Dr, Dv, R = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
     sizes = seqmix.prefill_head_sizes(D + Dr, Dv) if dtype == torch.bfloat16 else None
     if sizes is None or torch.device(device).type != "cuda":
@@ -61,49 +61,46 @@ def latent_prompt_layout(L: dict, m, dtype, device) -> None:
     L["wq"], L["qw"] = pad_rows(L["wq"], D + Dr, DKp), DKp
     L["wuk_p"] = pad_rows(L["wuk"].reshape(H * D, R), D, DKp)
     L["wuv_p"] = pad_rows(L["wuv_t"].transpose(1, 2).reshape(H * Dv, R), Dv, DVp)
-    L["wo_p"] = L["wo"] if DVp == Dv else \
-        pad_rows(L["wo"].t().contiguous(), Dv, DVp).t().contiguous()
     L["prompt_sizes"] = (DKp, DVp)
 
 
-def latent_mix(L: dict, m, q: torch.Tensor, z: torch.Tensor | None, pages: torch.Tensor, meta,
-               eps: float, prompt_min_q: int, gate: torch.Tensor | None = None) -> torch.Tensor:
-    """Latent attention of one step after its projections, for every family
+def latent_heads(L: dict, m, q: torch.Tensor, pages: torch.Tensor, meta, prompt_min_q: int,
+                 gate: torch.Tensor | None = None, out: torch.Tensor | None = None) -> torch.Tensor:
+    """Latent attention of one step between its projections, for every family
     that has such layers. q [T, H * qw]: the projected queries (per head D
-    unrotated then Dr rotary entries, possibly padded to ``L["qw"]``); z [T, R +
-    Dr]: the projected latent and shared rotary key part, appended to ``pages``
-    here (None: the pages belong to another layer and are complete). ``gate``
-    [T, H Dv] multiplies the heads' outputs by sigmoid(gate) before the output
-    projection. Returns the mixer's output [T, width]."""
-    H, D, Dr, Dv, R = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank
+    unrotated then Dr rotary entries, possibly padded to ``L["qw"]``); ``pages``
+    hold the step's own latent rows already (``seqmix.latent_inputs``). ``gate``
+    [T, H Dv] multiplies the heads' outputs by sigmoid(gate). The heads' outputs
+    [T, H Dv] go to ``out`` (may be a column slice; made here when None)."""
+    H, D, Dr, Dv, R, window = m.heads, m.dim, m.rot_dim, m.vdim, m.kv_rank, m.window
     T = q.shape[0]
-    if z is not None:
-        seqmix.latent_append(z, L["dkv_norm"], eps, meta.positions, L["cos_sin"], pages,
-                             meta.slots, R, m.rot.dims)
     q = q.view(T, H, L["qw"])
     if "prompt_sizes" in L and meta.max_q >= prompt_min_q and meta.cu_k is not None:
-        # prompt pass: per-head keys / values from the gathered latents, then
-        # flash attention on the matrix cores
+        # prompt pass: per-head keys / values from the gathered latents (the
+        # whole contexts, or what the rows' windows reach), then flash attention
+        # on the matrix cores
         DKp, DVp = L["prompt_sizes"]
-        cl, kr = seqmix.latent_gather(pages, meta.block_tables, meta.cu_k, meta.total_k,
-                                      meta.max_ctx, R)
+        cu_k, total_k = meta.window_k[window] if window > 0 else (meta.cu_k, meta.total_k)
+        reach = min(meta.max_ctx, meta.max_q + window - 1) if window > 0 else meta.max_ctx
+        cl, kr = seqmix.latent_gather(pages, meta.block_tables, cu_k, meta.ctx_lens, total_k,
+                                      reach, R)
         k = ops.linear(cl, L["wuk_p"]).view(-1, H, DKp)
         seqmix.latent_kfill_(k, kr, D)
         v = ops.linear(cl, L["wuv_p"]).view(-1, H, DVp)
         seqmix.rope_pairs_(q, D, m.rot.dims, meta.positions, L["cos_sin"])
-        o = seqmix.latent_prefill(q, k, v, meta.cu_q, meta.cu_k, meta.positions, L["sink"],
-                                  m.scale, meta.max_q)
-        if gate is not None:
-            seqmix.sigmoid_gate_(o.view(T, H, DVp), gate, H, Dv)
-        return ops.linear(o, L["wo_p"])
+        return seqmix.latent_prefill(q, k, v, meta.cu_q, cu_k, meta.ctx_lens, meta.positions,
+                                     L["sink"], m.scale, meta.max_q, Dv, window, gate, out)
     qa = torch.bmm(q[:, :, :D].transpose(0, 1), L["wuk"])            # [H, T, R]
     lat = seqmix.latent_attention(qa, q[:, :, D:D + Dr], pages, meta.cu_q, meta.ctx_lens,
                                   meta.block_tables, meta.positions, L["cos_sin"], L["sink"],
-                                  m.scale, R, m.rot.dims, meta.max_ctx)
-    o = torch.bmm(lat, L["wuv_t"]).transpose(0, 1).reshape(T, H * Dv)     # [T, H Dv]
+                                  m.scale, R, m.rot.dims, meta.max_ctx, window=window)
+    o = torch.bmm(lat, L["wuv_t"]).transpose(0, 1)                   # [T, H, Dv], head-major
     if gate is not None:
-        seqmix.sigmoid_gate_(o.view(T, H, Dv), gate, H, Dv)
-    return ops.linear(o, L["wo"])
+        return seqmix.sigmoid_gate(o, gate, H, Dv, out)
+    if out is None:
+        return o.reshape(T, H * Dv)
+    out.view(T, H, Dv).copy_(o)
+    return out
 
 
 class PipizenWeights:
@@ -320,13 +317,12 @@ class PipizenModel:
         block_tables, state_slots, logit_idx); ``cache``: a HybridCache."""
         w, cfg, dt = self.w, self.cfg, self.w.dtype
         x = self.embed(meta.tokens).contiguous()
-        T = x.shape[0]
         h = seqmix.dyt_norm(x, w.layers[0]["norm1"], dt) if w.layers else None
         n = len(w.layers)
         for i, (lc, L) in enumerate(zip(cfg.layers, w.layers)):
             m = lc.mixer
             if lc.kind == "latent_attention":
-                y = self._latent(i, m, L, h, meta, cache, T)
+                y = self._latent(i, m, L, h, meta, cache)
             else:
                 y = self._lightning(i, m, L, h, meta, cache)
             nxt_layer = w.layers[i + 1]["norm1"] if i + 1 < n else None
@@ -340,11 +336,14 @@ class PipizenModel:
         hf = seqmix.dyt_norm(x, w.final_norm, torch.float32, row_idx=meta.logit_idx)
         return ops.linear(hf, w.head)
 
-    def _latent(self, i, m, L, h, meta, cache, T) -> torch.Tensor:
-        src = i if m.kv_from is None else m.kv_from
-        z = ops.linear(h, L["wdkv"]) if m.kv_from is None else None
-        return latent_mix(L, m, ops.linear(h, L["wq"]), z, cache.latent[src], meta,
-                          self.cfg.norm_eps, self.prompt_min_q)
+    def _latent(self, i, m, L, h, meta, cache) -> torch.Tensor:
+        pages = cache.latent[i if m.kv_from is None else m.kv_from]
+        if m.kv_from is None:        # else the pages belong to another layer and are complete
+            seqmix.latent_inputs(ops.linear(h, L["wdkv"]), L["dkv_norm"], self.cfg.norm_eps,
+                                 meta.positions, L["cos_sin"], pages, meta.slots, m.kv_rank,
+                                 m.rot.dims)
+        return ops.linear(latent_heads(L, m, ops.linear(h, L["wq"]), pages, meta,
+                                       self.prompt_min_q), L["wo"])
 
     def _lightning(self, i, m, L, h, meta, cache) -> torch.Tensor:
         H, D, Dv = m.heads, m.dim, m.vdim

@@ -3,10 +3,12 @@ config.json: the Llama family (Hugging Face naming) and the designs with their
 own naming, told apart by ``"architecture"``: the hybrid Pipizen (latent /
 lightning mixers), Sodonex (chunked sigmoid attention with row state) and
 Movinex (windowed softmax attention, Mamba-2 layers, a repeated stretch of
-layers) and Vilulix (parallel layers; matrix memory, latent attention, windowed
-attention beside a gated delta rule). A family knows how to
-read its config, load or seed its weights and build its step function; the
-engine, the scheduler and the command line go through this table only.
+layers), Vilulix (parallel layers; matrix memory, latent attention, windowed
+attention beside a gated delta rule) and Gopopel (parallel layers on one norm;
+windowed attention with a distance bias and value mixing, windowed latent
+attention). A family knows how to read its config, load or seed its weights and
+build its step function; the engine, the scheduler and the command line go
+through this table only.
 """
 from __future__ import annotations
 
@@ -15,10 +17,10 @@ from typing import Callable
 
 import torch
 
-from .configs import (LlamaConfig, MovinexConfig, PipizenConfig, SodonexConfig, VilulixConfig,
-                      checkpoint_config, llama_config_from_hf, movinex_config_from_json,
-                      pipizen_config_from_json, sodonex_config_from_json,
-                      vilulix_config_from_json)
+from .configs import (GopopelConfig, LlamaConfig, MovinexConfig, PipizenConfig, SodonexConfig,
+                      VilulixConfig, checkpoint_config, gopopel_config_from_json,
+                      llama_config_from_hf, movinex_config_from_json, pipizen_config_from_json,
+                      sodonex_config_from_json, vilulix_config_from_json)
 
 
 @dataclass(frozen=True)
@@ -46,6 +48,10 @@ def _is_vilulix(d: dict) -> bool:
     return str(d.get("architecture", "")).lower() == "vilulix"
 
 
+def _is_gopopel(d: dict) -> bool:
+    return str(d.get("architecture", "")).lower() == "gopopel"
+
+
 def _is_llama(d: dict) -> bool:
     arch = " ".join(d.get("architectures") or []) + " " + str(d.get("model_type", ""))
     return "num_attention_heads" in d and ("llama" in arch.lower() or "hidden_size" in d)
@@ -56,6 +62,7 @@ FAMILIES = (
     Family("sodonex", SodonexConfig, _is_sodonex, sodonex_config_from_json, True),
     Family("movinex", MovinexConfig, _is_movinex, movinex_config_from_json, True),
     Family("vilulix", VilulixConfig, _is_vilulix, vilulix_config_from_json, True),
+    Family("gopopel", GopopelConfig, _is_gopopel, gopopel_config_from_json, True),
     Family("llama", LlamaConfig, _is_llama, llama_config_from_hf, False),
 )
 
@@ -100,6 +107,8 @@ def load_lm_weights(cfg, path: str, device, *, dtype=torch.bfloat16, tp=None,
         return loader.load_movinex(cfg, path, device, dtype, max_positions)
     if fam.name == "vilulix":
         return loader.load_vilulix(cfg, path, device, dtype, max_positions)
+    if fam.name == "gopopel":
+        return loader.load_gopopel(cfg, path, device, dtype, max_positions)
     return loader.load_pipizen(cfg, path, device, dtype, max_positions)
 
 
@@ -118,6 +127,9 @@ def random_lm_weights(cfg, device, *, seed: int = 0, dtype=torch.bfloat16, tp=No
     if fam.name == "vilulix":
         from .vilulix import VilulixWeights
         return VilulixWeights.random(cfg, device, seed, dtype, max_positions)
+    if fam.name == "gopopel":
+        from .gopopel import GopopelWeights
+        return GopopelWeights.random(cfg, device, seed, dtype, max_positions)
     from .pipizen import PipizenWeights
     return PipizenWeights.random(cfg, device, seed, dtype, max_positions)
 
@@ -135,5 +147,8 @@ def build_model(weights):
     from .vilulix import VilulixModel, VilulixWeights
     if isinstance(weights, VilulixWeights):
         return VilulixModel(weights)
+    from .gopopel import GopopelModel, GopopelWeights
+    if isinstance(weights, GopopelWeights):
+        return GopopelModel(weights)
     from .pipizen import PipizenModel
     return PipizenModel(weights)

@@ -46,7 +46,7 @@ import torch
 from .. import ops
 from ..ops import seqmix
 from .configs import VilulixConfig
-from .pipizen import latent_mix, latent_prompt_layout
+from .pipizen import latent_heads, latent_prompt_layout
 
 
 def _pairs_from_halves(dims: int, size: int) -> torch.Tensor:
@@ -440,11 +440,13 @@ class VilulixModel:
         H, Dv, R, Dr = m.heads, m.vdim, m.kv_rank, m.rot_dim
         eps = self.cfg.norm_eps
         u = ops.linear(h, L["w_in"])                       # dq | dkv | gate
-        cq = seqmix.rms_norm_cols(u, m.q_rank, L["dq_norm"], eps, self.w.dtype)
-        z = u[:, L["z_off"]:L["z_off"] + R + Dr]
+        cq = seqmix.latent_inputs(u[:, L["z_off"]:L["z_off"] + R + Dr], L["dkv_norm"], eps,
+                                  meta.positions, L["cos_sin"], cache.latent[r], meta.slots, R,
+                                  m.rot.dims, u[:, :m.q_rank], L["dq_norm"])
         gate = u[:, L["g_off"]:L["g_off"] + H * Dv]
-        return latent_mix(L, m, ops.linear(cq, L["wq"]), z, cache.latent[r], meta, eps,
-                          self.prompt_min_q, gate)
+        o = latent_heads(L, m, ops.linear(cq, L["wq"]), cache.latent[r], meta, self.prompt_min_q,
+                         gate)
+        return ops.linear(o, L["wo"])
 
     def _parallel(self, r, m, L, h, meta, cache, side=None) -> list:
         u = ops.linear(h, L["w_in"])                       # left q | k | v, right q | k | v | g

@@ -206,16 +206,20 @@ _RUNTIME_SIGS = {
 
 
 _vp, _i, _f, _l = c_void_p, c_int, c_float, c_ll
+_SIDE = (_vp, _l, _vp, _l, _i, _i, _i, _i)      # SideCols (csrc/kernels/seqmix.h)
 _SEQMIX_SIGS = {
     "loqa_dyt_norm": [_vp, _i, _vp, _vp, _vp, _f, _vp, _i, _i, _i, _vp],
     "loqa_dyt_add_norm": [_vp, _vp, _i, _vp, _vp, _f, _vp, _vp, _f, _vp, _i, _i, _i, _vp],
-    "loqa_latent_append": [_vp, _i, _l, _vp, _f, _vp, _vp, _i, _vp, _i, _i, _vp, _i, _i, _i, _i, _vp],
+    "loqa_residual_dyt": [_vp, _vp, _vp, _i, _vp, _vp, _f, _vp, _i, _i, _i, _vp],
+    "loqa_latent_inputs": [_vp, _i, _l, _vp, _f, _vp, _vp, _i, _vp, _i, _i, _vp, _i, _i, _i, _i,
+                           _vp, _l, _vp, _i, _vp, *_SIDE, _vp],
     "loqa_latent_attention": [_vp, _l, _l, _vp, _l, _l, _i, _vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp,
-                              _i, _vp, _f, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp],
-    "loqa_latent_gather": [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _vp, _vp, _vp],
+                              _i, _vp, _f, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _i, _vp],
+    "loqa_latent_gather": [_vp, _i, _vp, _i, _vp, _vp, _i, _i, _i, _i, _vp, _vp, _vp],
     "loqa_latent_kfill": [_vp, _vp, _i, _i, _i, _i, _i, _vp],
     "loqa_rope_pairs": [_vp, _l, _l, _i, _i, _i, _i, _vp, _vp, _i, _vp],
-    "loqa_latent_prefill": [_vp, _l, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _f, _i, _i, _i, _i, _i, _vp],
+    "loqa_latent_prefill": [_vp, _l, _vp, _vp, _vp, _l, _vp, _vp, _vp, _vp, _vp, _f, _i, _vp, _l,
+                            _i, _i, _i, _i, _i, _i, _vp],
     "loqa_lightning_prep": [_vp, _i, _l, _i, _i, _vp, _vp],
     "loqa_state_scan": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp,
                         _vp, _i, _i, _i, _vp],
@@ -237,15 +241,16 @@ _SEQMIX_SIGS = {
     "loqa_rms1p_norm": [_vp, _vp, _vp, _f, _vp, _i, _i, _i, _vp],
     "loqa_scaled_add_rms1p": [_vp, _vp, _i, _vp, _vp, _f, _vp, _i, _i, _i, _vp],
     "loqa_qk_prep_append": [_vp, _i, _l, _i, _i, _i, _i, _i, _vp, _i, _i, _f, _f, _i, _vp, _vp,
-                            _vp, _i, _i, _vp, _vp, _i, _vp, _vp, _vp],
+                            _vp, _i, _i, _vp, _vp, _i, _vp, _vp, _i, _vp, _l, _f, *_SIDE, _vp],
     "loqa_window_attention": [_vp, _i, _vp, _vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _l, _f, _f,
-                              _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp],
+                              _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _l, _i, _vp, _vp, _vp,
+                              _vp],
     "loqa_mamba2_prep": [_vp, _i, _l, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _i, _vp, _vp,
                          _vp, _i, _i, _vp, _vp, _vp],
     "loqa_residual_rms1p": [_vp, _vp, _f, _vp, _f, _vp, _f, _i, _vp, _vp, _vp, _f, _vp, _vp, _i,
                             _i, _i, _vp],
     "loqa_rms_norm_cols": [_vp, _i, _l, _i, _vp, _f, _vp, _i, _i, _vp],
-    "loqa_sigmoid_gate": [_vp, _i, _vp, _l, _i, _i, _i, _i, _vp],
+    "loqa_sigmoid_gate": [_vp, _l, _l, _i, _vp, _l, _vp, _l, _l, _i, _i, _i, _vp],
     "loqa_softcap": [_vp, _l, _f, _vp],
     "loqa_exp_gate_scan": [_vp, _i, _vp, _vp, _f, _vp, _i, _vp, _vp, _vp, _i, _i, _vp, _vp, _vp],
     "loqa_matrix_memory_inputs": [_vp, _i, _l, _i, _i, _i, _vp, _i, _vp],

@@ -629,6 +629,21 @@ def dyt_add_norm(resid, y, post, nxt, out_dtype):
     return dyt_norm(resid, nxt[0], nxt[1], nxt[2], out_dtype)
 
 
+def residual_dyt(resid, addends, nxt, out_dtype):
+    """resid (f32, in place) += sum of ``addends``; returns dyt(resid; nxt) or None."""
+    for y in addends:
+        resid.add_(y.float())
+    return None if nxt is None else dyt_norm(resid, nxt[0], nxt[1], nxt[2], out_dtype)
+
+
+def side_relu2(side):
+    """The side columns of a parallel layer (:class:`seqmix.SideCols`)."""
+    n = side.src.shape[1]
+    side.dst[:, side.zero_from:side.off] = 0
+    side.dst[:, side.off:side.off + n] = side.src.float().relu().square().to(side.dst.dtype)
+    side.dst[:, side.off + n:] = 0
+
+
 def rope_table_pairs(dims: int, max_pos: int, base: float, yarn: tuple | None = None,
                      device=None) -> torch.Tensor:
     """[max_pos, dims/2, 2] f32 (cos, sin) for the interleaved layout (entry 2i
@@ -666,10 +681,12 @@ def rotate_pairs(x, cs, dims: int):
     return out
 
 
-def latent_append(z, norm_w, eps: float, positions, cos_sin, cache, slots, R: int, dims: int):
+def latent_inputs(z, norm_w, eps: float, positions, cos_sin, cache, slots, R: int, dims: int,
+                  dq=None, dq_norm=None, side=None):
     """z [T, R + Dr]: the first R entries RMS-normed (weight ``norm_w``) are
     the latent, the rest the shared rotary key part; both go to the paged
-    cache [blocks, BLK, R + Dr] at ``slots`` (-1: padding row)."""
+    cache [blocks, BLK, R + Dr] at ``slots`` (-1: padding row). Returns the query
+    latent ``dq`` RMS-normed with ``dq_norm`` (None without one)."""
     zf = z.float()
     c = zf[:, :R]
     c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
@@ -679,13 +696,17 @@ def latent_append(z, norm_w, eps: float, positions, cos_sin, cache, slots, R: in
     ok = sl >= 0
     blk = cache.shape[1]
     cache[(sl // blk)[ok], (sl % blk)[ok]] = row[ok]
+    if side is not None:
+        side_relu2(side)
+    return None if dq is None else rms_norm_cols(dq, dq.shape[1], dq_norm, eps, dq.dtype)
 
 
 def latent_attention(qa, qr, cache, cu_q, ctx_lens, block_tables, positions, cos_sin, sink,
-                     scale: float, R: int, dims: int, out):
+                     scale: float, R: int, dims: int, out, window: int = 0):
     """Causal attention of one shared key/value stream per token (the cached
     latent row): score = (qa . c + rot(qr) . k_rot) * scale, softmax whose
-    denominator also holds exp(sink[h]); out[h, t] = sum_j p_j c_j.
+    denominator also holds exp(sink[h]); out[h, t] = sum_j p_j c_j; ``window`` >
+    0: the query at position p sees key j only if p - j < window.
     qa [H, T, R], qr [T, H, Dr] (unrotated), out [H, T, R]."""
     H = qa.shape[0]
     blk = cache.shape[1]
@@ -701,7 +722,10 @@ def latent_attention(qa, qr, cache, cu_q, ctx_lens, block_tables, positions, cos
         s = torch.einsum("htr,lr->htl", qa[:, q0:q1].float(), rows[:, :R])
         s = (s + torch.einsum("thr,lr->htl", qrot[q0:q1], rows[:, R:])) * scale
         qpos = positions[q0:q1].long()
-        s = s.masked_fill(idx[None, None, :] > qpos[None, :, None], float("-inf"))
+        hidden = idx[None, None, :] > qpos[None, :, None]
+        if window > 0:
+            hidden = hidden | (qpos[None, :, None] - idx[None, None, :] >= window)
+        s = s.masked_fill(hidden, float("-inf"))
         if sink is not None:
             s = torch.cat([s, sink.float()[:, None, None].expand(H, q1 - q0, 1)], dim=-1)
         p = torch.softmax(s, dim=-1)[..., :L]
@@ -1006,7 +1030,8 @@ def scaled_add_rms1p(resid, y, ls, nxt, eps: float, out_dtype):
 
 
 def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims: int, eps: float,
-                   q_temp, positions, k_cache, v_cache, slots, out_dtype, q_norm=None, k_norm=None):
+                   q_temp, positions, k_cache, v_cache, slots, out_dtype, q_norm=None, k_norm=None,
+                   v_mix=None, side=None):
     """u [T, >= H D + G D (+ G Dv)]: projected q | k (| v) rows. Per head: the
     first ``dims`` entries of q and k rotate pairwise (2i with 2i + 1) by the
     position's angles, then each head's q and k is divided by its root mean
@@ -1017,14 +1042,23 @@ def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims
     theirs [blocks, BLK, G Dv] at ``slots`` (-1: padding row). Returns q [T, H D].
     With ``q_norm`` [H D] and ``k_norm`` [G D] the norm is another one: q and k
     are RMS-normed over their whole projection with these weights BEFORE the
-    rotation, and no per-head division follows."""
+    rotation, and no per-head division follows; with both [D] per head with
+    shared weights, also before it. ``v_mix`` = (v_first [T, G Dv], lam): the
+    values stored are (1 - lam) v + lam v_first."""
     T = u.shape[0]
     uf = u.float()
     q = uf[:, :H * D].reshape(T, H, D)
     k = uf[:, H * D:(H + G) * D].reshape(T, G, D)
     v = k.reshape(T, G * D) if v_off < 0 else uf[:, v_off:v_off + G * Dv]
     pos = positions[:T].long()
-    if q_norm is not None:
+    if v_mix is not None:
+        v = (1.0 - float(v_mix[1])) * v + float(v_mix[1]) * v_mix[0].float()
+    if side is not None:
+        side_relu2(side)
+    if q_norm is not None and q_norm.numel() == k_norm.numel() == D:
+        q = rms_norm_cols(q.reshape(T * H, D), D, q_norm, eps, torch.float32).view(T, H, D)
+        k = rms_norm_cols(k.reshape(T * G, D), D, k_norm, eps, torch.float32).view(T, G, D)
+    elif q_norm is not None:
         q = rms_norm_cols(q.reshape(T, H * D), H * D, q_norm, eps, torch.float32).view(T, H, D)
         k = rms_norm_cols(k.reshape(T, G * D), G * D, k_norm, eps, torch.float32).view(T, G, D)
     if dims:
@@ -1047,14 +1081,15 @@ def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims
 
 def window_attention(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, positions, scale: float,
                      softcap: float, window: int, keep_first: int, gate, H: int, G: int, D: int,
-                     Dv: int, out_dtype, sink=None):
+                     Dv: int, out_dtype, sink=None, slopes=None):
     """Softmax attention of q [T, H D] over paged K [blocks, BLK, G D] and V
     [blocks, BLK, G Dv]: score = q . k * scale, soft-capped to cap tanh(score /
     cap) when ``softcap`` > 0; a query at position p sees key j <= p, and with
     ``window`` > 0 only if p - j < window or j < keep_first. ``gate`` [T, H Dv]
     multiplies the output by sigmoid(gate) per entry. ``sink`` f32 [H]: the
     softmax denominator of head h also holds exp(sink[h]), a term without a
-    value. Returns [T, H Dv]."""
+    value. ``slopes`` f32 [H]: slopes[h] * (p - j) comes off the capped score.
+    Returns [T, H Dv]."""
     T = q.shape[0]
     blk = k_cache.shape[1]
     rep = H // G
@@ -1078,6 +1113,8 @@ def window_attention(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, position
             s = qf[q0:q1, h] @ kk[:, h // rep].T * scale
             if softcap > 0:
                 s = softcap * torch.tanh(s / softcap)
+            if slopes is not None:
+                s = s - slopes[h].float() * (qpos[:, None] - idx[None, :]).float()
             s = s.masked_fill(~seen, float("-inf"))
             if sink is not None:
                 s = torch.cat([s, sink[h].float().expand(q1 - q0, 1)], dim=-1)
@@ -1145,13 +1182,12 @@ def rms_norm_cols(u, n: int, w, eps: float, out_dtype):
     return (x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w.float()).to(out_dtype)
 
 
-def sigmoid_gate_(o, gate, H: int, Dv: int):
-    """o [T, H, Dvo >= Dv] (in place): the first Dv entries of every head times
-    sigmoid(gate [T, H Dv])."""
+def sigmoid_gate(o, gate, H: int, Dv: int, out):
+    """The first Dv entries of every head of o [T, H, >= Dv] times sigmoid(gate
+    [T, H Dv]) into ``out`` [T, H Dv]."""
     T = o.shape[0]
     g = torch.sigmoid(gate.float()).view(T, H, Dv)
-    o[:, :, :Dv] = (o[:, :, :Dv].float() * g).to(o.dtype)
-    return o
+    return out.copy_((o[:, :, :Dv].float() * g).reshape(T, H * Dv))
 
 
 def softcap_(x, cap: float):

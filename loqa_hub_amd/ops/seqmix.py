@@ -91,6 +91,66 @@ def dyt_add_norm(resid: torch.Tensor, y: torch.Tensor, post: DytParams,
     return h
 
 
+def alibi_slopes(H: int, device=None) -> torch.Tensor:
+    """The geometric slopes of a linear distance bias, f32 [H]: 2^(-8 (h + 1) / H)."""
+    return torch.tensor([2.0 ** (-8.0 * (h + 1) / H) for h in range(H)], dtype=torch.float32,
+                        device=device)
+
+
+def residual_dyt(resid: torch.Tensor, addends: list, nxt: DytParams | None, out_dtype
+                 ) -> torch.Tensor | None:
+    """The residual step of a layer whose sublayer outputs are added as they
+    are: resid (f32, in place) += sum of up to two ``addends`` [rows, d] in one
+    activation dtype, and in the same launch h = dyt(resid; nxt) for the next
+    layer (None: no h)."""
+    if not resid.is_cuda:
+        return ref.residual_dyt(resid, addends, None if nxt is None else nxt.tup(), out_dtype)
+    _f32c(resid, "resid")
+    rows, d = resid.shape
+    assert len(addends) <= 2
+    ys = [None, None]
+    for i, y in enumerate(addends):
+        assert y.shape == resid.shape and y.is_contiguous() and y.dtype == addends[0].dtype
+        ys[i] = y
+    h = None
+    if nxt is not None:
+        assert nxt.w.numel() == d and nxt.b.numel() == d
+        h = torch.empty(rows, d, dtype=out_dtype, device=resid.device)
+    if rows:
+        check(kernels().loqa_residual_dyt(
+            ptr(resid), ptr(ys[0]), ptr(ys[1]), _dt(ys[0]) if addends else 0,
+            ptr(nxt.w) if nxt else None, ptr(nxt.b) if nxt else None, nxt.alpha if nxt else 0.0,
+            ptr(h), _dt(h) if h is not None else 0, rows, d, stream_ptr(resid)), "residual_dyt")
+    return h
+
+
+class SideCols:
+    """Work an input-stage launch does beside its own for a parallel layer,
+    whose ungated feed-forward reads the same rows as the mixer: dst[:, off :
+    off + n] = relu(src)^2 with src [T, n] a column slice of the fused
+    projection, and zeros in dst's columns ``zero_from`` .. off and from off + n
+    to its end (padding between the parts of one output projection)."""
+    __slots__ = ("src", "dst", "off", "zero_from")
+
+    def __init__(self, src: torch.Tensor, dst: torch.Tensor, off: int, zero_from: int):
+        n = src.shape[1]
+        assert src.stride(1) == 1 and dst.is_contiguous() and src.dtype == dst.dtype
+        assert src.shape[0] == dst.shape[0] and 0 <= zero_from <= off and off + n <= dst.shape[1]
+        self.src, self.dst, self.off, self.zero_from = src, dst, off, zero_from
+
+    def args(self) -> tuple:
+        n, ld = self.src.shape[1], self.dst.shape[1]
+        d = self.dst.data_ptr() + self.off * self.dst.element_size()
+        run = 4 * self.src.element_size()
+        vec = n % 4 == 0 and ld % 4 == 0 and self.src.stride(0) % 4 == 0 and \
+            d % run == 0 and self.src.data_ptr() % run == 0
+        return (ptr(self.src), self.src.stride(0), d, ld, n, self.zero_from - self.off,
+                ld - self.off, int(vec))
+
+
+_NO_SIDE = (None, 0, None, 0, 0, 0, 0, 0)
+
+
 def rope_table_pairs(dims: int, max_pos: int, base: float, yarn: tuple | None = None,
                      device=None) -> torch.Tensor:
     """(cos, sin) table of the interleaved rotary layout, optionally YaRN-scaled
@@ -98,13 +158,18 @@ def rope_table_pairs(dims: int, max_pos: int, base: float, yarn: tuple | None = 
     return ref.rope_table_pairs(dims, max_pos, base, yarn, device)
 
 
-def latent_append(z: torch.Tensor, norm_w: torch.Tensor, eps: float, positions: torch.Tensor,
+def latent_inputs(z: torch.Tensor, norm_w: torch.Tensor, eps: float, positions: torch.Tensor,
                   cos_sin: torch.Tensor, cache: torch.Tensor, slots: torch.Tensor, R: int,
-                  dims: int) -> None:
-    """RMS-norm the latent part of z [T, R + Dr], rotate its rotary key part and
-    store both in the paged latent cache [blocks, BLK, R + Dr] (one launch)."""
+                  dims: int, dq: torch.Tensor | None = None, dq_norm: torch.Tensor | None = None,
+                  side: SideCols | None = None) -> torch.Tensor | None:
+    """The input stage of latent attention, one launch: RMS-norm the latent part
+    of z [T, R + Dr], rotate its rotary key part and store both in the paged
+    latent cache [blocks, BLK, R + Dr]. ``dq`` [T, Rq] (a column slice of the
+    same projection): the query latent, returned RMS-normed with the weight
+    ``dq_norm``. ``side``: see :class:`SideCols`."""
     if not z.is_cuda:
-        return ref.latent_append(z, norm_w, eps, positions, cos_sin, cache, slots, R, dims)
+        return ref.latent_inputs(z, norm_w, eps, positions, cos_sin, cache, slots, R, dims, dq,
+                                 dq_norm, side)
     T, W = z.shape
     assert z.stride(1) == 1 and cache.is_contiguous() and cache.dtype == z.dtype
     assert cache.shape[2] == W and 0 < R <= W and dims % 2 == 0 and dims <= W - R
@@ -112,20 +177,32 @@ def latent_append(z: torch.Tensor, norm_w: torch.Tensor, eps: float, positions: 
     _i32c(slots, "slots")
     assert norm_w.numel() == R and cos_sin.shape[1] * 2 == dims
     assert positions.numel() >= T and slots.numel() >= T
+    cq, Rq = None, 0
+    if dq is not None:
+        _f32c(dq_norm, "dq_norm")
+        Rq = dq.shape[1]
+        assert dq.shape[0] == T and dq.stride(1) == 1 and dq.dtype == z.dtype and dq_norm.numel() == Rq
+        cq = torch.empty(T, Rq, dtype=z.dtype, device=z.device)
+    if side is not None:
+        assert side.src.shape[0] == T and side.src.dtype == z.dtype
     if T:
-        check(kernels().loqa_latent_append(
+        check(kernels().loqa_latent_inputs(
             ptr(z), _dt(z), z.stride(0), ptr(norm_w), eps, ptr(positions), ptr(cos_sin),
             cos_sin.shape[0], ptr(cache), cache.shape[1], cache.shape[0], ptr(slots), T, R, W - R,
-            dims, stream_ptr(z)), "latent_append")
+            dims, ptr(dq), dq.stride(0) if Rq else 0, ptr(dq_norm), Rq, ptr(cq),
+            *(side.args() if side is not None else _NO_SIDE), stream_ptr(z)), "latent_inputs")
+    return cq
 
 
 def latent_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, cu_q: torch.Tensor,
                      ctx_lens: torch.Tensor, block_tables: torch.Tensor, positions: torch.Tensor,
                      cos_sin: torch.Tensor, sink: torch.Tensor | None, scale: float, R: int,
-                     dims: int, max_ctx: int = 0, out: torch.Tensor | None = None) -> torch.Tensor:
+                     dims: int, max_ctx: int = 0, out: torch.Tensor | None = None,
+                     window: int = 0) -> torch.Tensor:
     """Causal attention over the paged latent cache, all heads sharing each
     cached row: score = (qa . c + rot(qr) . k_rot) * scale; softmax with
-    ``sink`` [H] (f32, optional) in the denominator; out = sum_j p_j c_j.
+    ``sink`` [H] (f32, optional) in the denominator; out = sum_j p_j c_j. With
+    ``window`` > 0 the query at position p sees key j only if p - j < window.
     qa [H, T, R] (queries already folded into latent space), qr [T, H, Dr]
     (unrotated; may be a strided view), out [H, T, R]."""
     H, T, _ = qa.shape
@@ -133,7 +210,7 @@ def latent_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, cu
         out = torch.empty(H, T, R, dtype=qa.dtype, device=qa.device)
     if not qa.is_cuda:
         return ref.latent_attention(qa, qr, cache, cu_q, ctx_lens, block_tables, positions,
-                                    cos_sin, sink, scale, R, dims, out)
+                                    cos_sin, sink, scale, R, dims, out, window)
     Dr = cache.shape[2] - R
     assert qa.shape[2] == R and qa.stride(2) == 1 and qr.shape == (T, H, Dr) and qr.stride(2) == 1
     assert qa.dtype == cache.dtype == qr.dtype == out.dtype and cache.is_contiguous()
@@ -147,14 +224,16 @@ def latent_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, cu
     assert cu_q.numel() == B + 1 and block_tables.shape[0] == B and positions.numel() >= T
     # few query rows over a long context: split the keys over workgroups
     hg = (H + 3) // 4
-    ns = 1 if T * hg >= 512 else max(1, min(32, -(-int(max_ctx) // 128), 1024 // max(1, T * hg)))
+    keys = min(int(max_ctx), window) if window > 0 else int(max_ctx)
+    ns = 1 if T * hg >= 512 else max(1, min(32, -(-keys // 128), 1024 // max(1, T * hg)))
     ws = torch.empty(ns * T * H * (R + 2), dtype=torch.float32, device=qa.device) if ns > 1 else None
     if T:
         check(kernels().loqa_latent_attention(
             ptr(qa), qa.stride(1), qa.stride(0), ptr(qr), qr.stride(0), qr.stride(1), _dt(qa),
             ptr(cache), cache.shape[1], cache.shape[0], ptr(cu_q), ptr(ctx_lens), ptr(block_tables),
             block_tables.shape[1], ptr(positions), ptr(cos_sin), cos_sin.shape[0], ptr(sink),
-            float(scale), B, H, T, R, Dr, dims, ptr(out), ns, ptr(ws), stream_ptr(qa)),
+            float(scale), B, H, T, R, Dr, dims, ptr(out), ns, ptr(ws), int(window),
+            stream_ptr(qa)),
             "latent_attention")
     return out
 
@@ -172,18 +251,20 @@ def prefill_head_sizes(dk: int, dv: int) -> tuple[int, int] | None:
 
 
 def latent_gather(cache: torch.Tensor, block_tables: torch.Tensor, cu_k: torch.Tensor,
-                  total_k: int, max_ctx: int, R: int) -> tuple[torch.Tensor, torch.Tensor]:
-    """Every sequence's cached rows in position order, as contiguous latents
-    [total_k, R] and rotary key parts [total_k, Dr] (bf16, GPU)."""
+                  ctx_lens: torch.Tensor, total_k: int, max_ctx: int, R: int
+                  ) -> tuple[torch.Tensor, torch.Tensor]:
+    """The last cu_k[b + 1] - cu_k[b] of each sequence's ``ctx_lens[b]`` cached
+    rows in position order, as contiguous latents [total_k, R] and rotary key
+    parts [total_k, Dr] (bf16, GPU)."""
     assert cache.is_cuda and cache.dtype == torch.bfloat16 and cache.is_contiguous()
-    _i32c(block_tables, "block_tables"); _i32c(cu_k, "cu_k")
+    _i32c(block_tables, "block_tables"); _i32c(cu_k, "cu_k"); _i32c(ctx_lens, "ctx_lens")
     B, Dr = block_tables.shape[0], cache.shape[2] - R
-    assert cu_k.numel() == B + 1
+    assert cu_k.numel() == B + 1 and ctx_lens.numel() == B
     cl = torch.empty(total_k, R, dtype=cache.dtype, device=cache.device)
     kr = torch.empty(total_k, Dr, dtype=cache.dtype, device=cache.device)
     check(kernels().loqa_latent_gather(ptr(cache), cache.shape[1], ptr(block_tables),
-                                       block_tables.shape[1], ptr(cu_k), B, int(max_ctx), R, Dr,
-                                       ptr(cl), ptr(kr), stream_ptr(cache)), "latent_gather")
+                                       block_tables.shape[1], ptr(cu_k), ptr(ctx_lens), B,
+                                       int(max_ctx), R, Dr, ptr(cl), ptr(kr), stream_ptr(cache)), "latent_gather")
     return cl, kr
 
 
@@ -210,29 +291,42 @@ def rope_pairs_(x: torch.Tensor, off: int, dims: int, positions: torch.Tensor,
 
 
 def latent_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_q: torch.Tensor,
-                   cu_k: torch.Tensor, positions: torch.Tensor, sink: torch.Tensor | None,
-                   scale: float, max_q: int) -> torch.Tensor:
+                   cu_k: torch.Tensor, ctx_lens: torch.Tensor, positions: torch.Tensor,
+                   sink: torch.Tensor | None, scale: float, max_q: int, Dv: int, window: int = 0,
+                   gate: torch.Tensor | None = None, out: torch.Tensor | None = None
+                   ) -> torch.Tensor:
     """Causal flash attention of a prompt pass on the matrix cores: q [T, H, DK]
-    (rotated), k [L, H, DK], v [L, H, DV] per-head keys / values of the
-    gathered contexts (``cu_k``), a query at absolute position p sees keys
-    0 .. p of its sequence; ``sink`` [H] joins the softmax denominator.
-    Returns [T, H * DV] (bf16)."""
+    (rotated), k [L, H, DK], v [L, H, DV] per-head keys / values of the gathered
+    contexts (``cu_k``: the last keys of each sequence's ``ctx_lens``), a query at
+    absolute position p sees the keys up to p of its sequence, with ``window`` > 0
+    only p - window + 1 .. p; ``sink`` [H] joins the softmax denominator; ``gate``
+    [T, H Dv] (may be a column slice) multiplies the output by sigmoid(gate).
+    Writes the model's Dv <= DV entries per head to ``out`` [T, >= H Dv] (may be
+    a column slice of a wider row; made here when None) and returns it (bf16)."""
     T, H, DK = q.shape
     DV = v.shape[2]
     assert q.is_cuda and q.dtype == k.dtype == v.dtype == torch.bfloat16
     assert q.stride(2) == 1 and q.stride(1) == DK and k.is_contiguous() and v.is_contiguous()
     assert k.shape[1:] == (H, DK) and v.shape[:2] == k.shape[:2]
-    assert DK in PREFILL_DK and DV in PREFILL_DV
+    assert DK in PREFILL_DK and DV in PREFILL_DV and 0 < Dv <= DV and window >= 0
     _i32c(cu_q, "cu_q"); _i32c(cu_k, "cu_k"); _i32c(positions, "positions")
+    _i32c(ctx_lens, "ctx_lens")
     B = cu_q.numel() - 1
-    assert cu_k.numel() == B + 1
+    assert cu_k.numel() == B + 1 and ctx_lens.numel() == B
     if sink is not None:
         _f32c(sink, "sink")
-    o = torch.empty(T, H * DV, dtype=q.dtype, device=q.device)
-    check(kernels().loqa_latent_prefill(ptr(q), q.stride(0), ptr(k), ptr(v), ptr(o), ptr(cu_q),
-                                        ptr(cu_k), ptr(positions), ptr(sink), float(scale), B, H,
-                                        int(max_q), DK, DV, stream_ptr(q)), "latent_prefill")
-    return o
+        assert sink.numel() == H
+    if gate is not None:
+        assert gate.shape == (T, H * Dv) and gate.stride(1) == 1 and gate.dtype == q.dtype
+    if out is None:
+        out = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device)
+    assert out.shape == (T, H * Dv) and out.stride(1) == 1 and out.dtype == q.dtype
+    check(kernels().loqa_latent_prefill(
+        ptr(q), q.stride(0), ptr(k), ptr(v), ptr(out), out.stride(0), ptr(cu_q), ptr(cu_k),
+        ptr(ctx_lens), ptr(positions), ptr(sink), float(scale), int(window), ptr(gate),
+        gate.stride(0) if gate is not None else 0, B, H, int(max_q), DK, DV, Dv, stream_ptr(q)),
+        "latent_prefill")
+    return out
 
 
 def lightning_scan(qkv: torch.Tensor, H: int, D: int, Dv: int, state: torch.Tensor,
@@ -669,7 +763,8 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
                    cos_sin: torch.Tensor | None, dims: int, eps: float, q_temp: tuple | None,
                    positions: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                    slots: torch.Tensor, out_dtype, q_norm: torch.Tensor | None = None,
-                   k_norm: torch.Tensor | None = None) -> torch.Tensor:
+                   k_norm: torch.Tensor | None = None, v_mix: tuple | None = None,
+                   side: SideCols | None = None) -> torch.Tensor:
     """One launch between the fused q | k (| v) projection u [T, W] and
     attention: per head the first ``dims`` entries of q and k rotate pairwise
     (interleaved layout, table ``cos_sin`` [positions, dims / 2, 2]), then q and
@@ -681,14 +776,27 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
     [T, H D]. Statistics, angles and the temperature are f32. With ``q_norm``
     [H D] and ``k_norm`` [G D] (f32) the norm is another one: q and k are
     RMS-normed over their whole projection with these weights BEFORE the
-    rotation, and no per-head division follows."""
+    rotation, and no per-head division follows; with both [D] they are
+    RMS-normed per head with weights shared by the heads, also before it (sizes
+    that fit both readings, H = G = 1, mean the same). ``v_mix`` = (v_first [T,
+    G Dv], lam): the stored values are (1 - lam) v + lam v_first. ``side``: see
+    :class:`SideCols`."""
     assert (q_norm is None) == (k_norm is None)
     if not u.is_cuda:
         return ref.qk_prep_append(u, H, G, D, Dv, v_off, cos_sin, dims, eps, q_temp, positions,
-                                  k_cache, v_cache, slots, out_dtype, q_norm, k_norm)
+                                  k_cache, v_cache, slots, out_dtype, q_norm, k_norm, v_mix, side)
+    norm = 0
     if q_norm is not None:
         _f32c(q_norm, "q_norm"); _f32c(k_norm, "k_norm")
-        assert q_norm.numel() == H * D and k_norm.numel() == G * D
+        norm = 2 if q_norm.numel() == k_norm.numel() == D else 1
+        assert norm == 2 or (q_norm.numel() == H * D and k_norm.numel() == G * D)
+    vf, lam = None, 0.0
+    if v_mix is not None:
+        vf, lam = v_mix
+        assert v_off >= 0 and vf.shape == (u.shape[0], G * Dv) and vf.stride(1) == 1
+        assert vf.dtype == u.dtype
+    if side is not None:
+        assert side.src.shape[0] == u.shape[0] and side.src.dtype == u.dtype
     T, W = u.shape
     assert u.stride(1) == 1 and (H + G) * D <= W
     assert v_off < 0 and Dv == D or v_off >= (H + G) * D and v_off + G * Dv <= W
@@ -708,11 +816,16 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
             ptr(u), _dt(u), u.stride(0), H, G, D, Dv, int(v_off), ptr(cos_sin) if dims else None,
             cos_sin.shape[0] if dims else 0, dims, float(eps), coef, every, ptr(positions),
             ptr(k_cache), ptr(v_cache), k_cache.shape[1], k_cache.shape[0], ptr(slots), ptr(q), T,
-            ptr(q_norm), ptr(k_norm), stream_ptr(u)), "qk_prep_append")
+            ptr(q_norm), ptr(k_norm), norm, ptr(vf), vf.stride(0) if vf is not None else 0,
+            float(lam), *(side.args() if side is not None else _NO_SIDE), stream_ptr(u)),
+            "qk_prep_append")
     return q
 
 
-WINDOW_MFMA_D = (64, 128)         # head sizes the matrix-core form is built for
+def window_mfma_sizes(D: int, Dv: int) -> bool:
+    """Head sizes the matrix-core form covers (built for 64 / 128 / 256 and 64 /
+    128; multiples of 8 in between are padded with zeros in LDS)."""
+    return D % 8 == 0 and 0 < D <= 256 and Dv % 8 == 0 and 0 < Dv <= 128
 
 
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -720,7 +833,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                      positions: torch.Tensor, scale: float, softcap: float, window: int,
                      keep_first: int, gate: torch.Tensor | None, H: int, G: int, D: int, Dv: int,
                      max_q: int = 0, matrix_cores: bool | None = None, max_ctx: int = 0,
-                     key_splits: int | None = None, sink: torch.Tensor | None = None
+                     key_splits: int | None = None, sink: torch.Tensor | None = None,
+                     slopes: torch.Tensor | None = None, out: torch.Tensor | None = None
                      ) -> torch.Tensor:
     """Softmax attention over paged K [blocks, BLK, G D] and V [blocks, BLK,
     G Dv] (query head h reads key/value head h // (H / G)): score = q . k *
@@ -734,11 +848,17 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     with few rows over long contexts (``max_ctx``) deals each row's keys out to
     ``key_splits`` workgroups (chosen here when None) and merges their partial
     results in a second launch. ``sink`` f32 [H]: head h's softmax denominator
-    also holds exp(sink[h]), a term that carries no value."""
+    also holds exp(sink[h]), a term that carries no value. ``slopes`` f32 [H]: a
+    linear distance bias, slopes[h] * (p - j) comes off the (capped) score.
+    ``out`` [T, H Dv]: where to write (may be a column slice of a wider row)."""
     if not q.is_cuda:
-        return ref.window_attention(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, positions,
-                                    scale, softcap, window, keep_first, gate, H, G, D, Dv, q.dtype,
-                                    sink)
+        o = ref.window_attention(q, k_cache, v_cache, cu_q, ctx_lens, block_tables, positions,
+                                 scale, softcap, window, keep_first, gate, H, G, D, Dv, q.dtype,
+                                 sink, slopes)
+        return o if out is None else out.copy_(o)
+    if slopes is not None:
+        _f32c(slopes, "slopes")
+        assert slopes.numel() == H
     if sink is not None:
         _f32c(sink, "sink")
         assert sink.numel() == H
@@ -756,11 +876,13 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     if gate is not None:
         assert gate.shape == (T, H * Dv) and gate.stride(1) == 1 and gate.dtype == q.dtype
         gs = gate.stride(0)
-    o = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device)
+    o = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device) if out is None else out
+    assert o.shape == (T, H * Dv) and o.stride(1) == 1 and o.dtype == q.dtype
     if matrix_cores is None:
         matrix_cores = max_q >= 16
-    mfma = bool(matrix_cores) and q.dtype == torch.bfloat16 and D in WINDOW_MFMA_D \
-        and Dv in WINDOW_MFMA_D
+    mfma = bool(matrix_cores) and q.dtype == torch.bfloat16 and window_mfma_sizes(D, Dv) \
+        and o.stride(0) % 4 == 0 and o.data_ptr() % 8 == 0 \
+        and (gate is None or (gs % 4 == 0 and gate.data_ptr() % 8 == 0))
     part = None
     if key_splits is None:
         # 64-key windows a row can have, four (one per wave) to a workgroup
@@ -777,8 +899,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             ptr(q), _dt(q), ptr(k_cache), ptr(v_cache), k_cache.shape[1], k_cache.shape[0],
             ptr(cu_q), ptr(ctx_lens), ptr(block_tables), block_tables.shape[1], ptr(positions),
             ptr(gate), gs, float(scale), float(softcap), int(window), int(keep_first), B, T, H, G,
-            D, Dv, int(max_q), int(mfma), ptr(o), int(key_splits), ptr(part), ptr(sink),
-            stream_ptr(q)), "window_attention")
+            D, Dv, int(max_q), int(mfma), ptr(o), o.stride(0), int(key_splits), ptr(part), ptr(sink),
+            ptr(slopes), stream_ptr(q)), "window_attention")
     return o
 
 
@@ -877,19 +999,25 @@ def rms_norm_cols(u: torch.Tensor, n: int, w: torch.Tensor, eps: float, out_dtyp
     return y
 
 
-def sigmoid_gate_(o: torch.Tensor, gate: torch.Tensor, H: int, Dv: int) -> torch.Tensor:
-    """In place: the first Dv entries of every head of o [T, H, Dvo] (Dvo >= Dv:
-    heads may be padded) times sigmoid(gate [T, H Dv]); ``gate`` may be a
-    column slice of a wider projection."""
+def sigmoid_gate(o: torch.Tensor, gate: torch.Tensor, H: int, Dv: int,
+                 out: torch.Tensor | None = None) -> torch.Tensor:
+    """The first Dv entries of every head of o [T, H, >= Dv] (any strides over
+    tokens and heads: padded or head-major) times sigmoid(gate [T, H Dv]), which
+    may be a column slice of a wider projection, into ``out`` [T, H Dv] (may be
+    a column slice too; made here when None)."""
+    T = o.shape[0]
+    if out is None:
+        out = torch.empty(T, H * Dv, dtype=o.dtype, device=o.device)
     if not o.is_cuda:
-        return ref.sigmoid_gate_(o, gate, H, Dv)
-    T, Ho, Dvo = o.shape
-    assert Ho == H and Dvo >= Dv and o.is_contiguous()
+        return ref.sigmoid_gate(o, gate, H, Dv, out)
+    assert o.shape[1] == H and o.shape[2] >= Dv and o.stride(2) == 1
     assert gate.shape == (T, H * Dv) and gate.stride(1) == 1 and gate.dtype == o.dtype
+    assert out.shape == (T, H * Dv) and out.stride(1) == 1 and out.dtype == o.dtype
     if T:
-        check(kernels().loqa_sigmoid_gate(ptr(o), _dt(o), ptr(gate), gate.stride(0), T, H, Dvo, Dv,
+        check(kernels().loqa_sigmoid_gate(ptr(o), o.stride(0), o.stride(1), _dt(o), ptr(gate),
+                                          gate.stride(0), ptr(out), out.stride(0), Dv, T, H, Dv,
                                           stream_ptr(o)), "sigmoid_gate")
-    return o
+    return out
 
 
 def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:

@@ -156,9 +156,8 @@ def test_small_steps(device):
     assert (got.cpu().double() - O.norm_plain(u[:, :19].double(), w.double(), 1e-4)).abs().max() < 1e-5
     o = torch.randn(7, 3, 8, generator=g)
     gt = torch.randn(7, 40, generator=g)
-    got = seqmix.sigmoid_gate_(o.to(device).clone(), gt.to(device)[:, 4:4 + 15], 3, 5)
-    want = o.double().clone()
-    want[:, :, :5] *= torch.sigmoid(gt[:, 4:19].double()).view(7, 3, 5)
+    got = seqmix.sigmoid_gate(o.to(device), gt.to(device)[:, 4:4 + 15], 3, 5).view(7, 3, 5)
+    want = o[:, :, :5].double() * torch.sigmoid(gt[:, 4:19].double()).view(7, 3, 5)
     assert (got.cpu().double() - want).abs().max() < 1e-6
     z = torch.randn(5, 33, generator=g) * 20
     got = seqmix.softcap_(z.to(device).clone(), 7.0)
