@@ -878,8 +878,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         gs = gate.stride(0)
     o = torch.empty(T, H * Dv, dtype=q.dtype, device=q.device) if out is None else out
     assert o.shape == (T, H * Dv) and o.stride(1) == 1 and o.dtype == q.dtype
-    if matrix_cores is None:
-        matrix_cores = max_q >= 16
+    if matrix_cores is None:         # heads far below the built sizes would be mostly padding
+        matrix_cores = max_q >= 16 and D >= 32 and Dv >= 32
     mfma = bool(matrix_cores) and q.dtype == torch.bfloat16 and window_mfma_sizes(D, Dv) \
         and o.stride(0) % 4 == 0 and o.data_ptr() % 8 == 0 \
         and (gate is None or (gs % 4 == 0 and gate.data_ptr() % 8 == 0))

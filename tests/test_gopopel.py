@@ -1,0 +1,829 @@
+"""The Gopopel family through the framework (registry, weights, engine step,
+hybrid cache, scheduler) against the plain float64 oracle in
+``gopopel_oracle.py``. Every test builds its own small configuration and seeded
+weights. The same tests run on the CPU (reference ops) and, marked ``gpu``, on
+the HIP kernels.
+"""
+import json
+import math
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+import gopopel_oracle as O
+from loqa_hub_amd.engine.llm_engine import GenRequest, LLMEngine
+from loqa_hub_amd.models.configs import gopopel_config_from_json
+from loqa_hub_amd.models.gopopel import (GopopelWeights, config_to_json, random_state_dict,
+                                         stack_rows)
+from loqa_hub_amd.models.registry import family_of, lm_config_from_json
+from loqa_hub_amd.ops import seqmix
+from loqa_hub_amd.ops.seqmix import DytParams, SideCols
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+TOL = {torch.float32: 2e-4, torch.bfloat16: 6e-2}
+F64 = torch.float64
+
+
+def engine(cfg_json, sd, device, dtype=torch.float32, max_tokens=256, block=16, max_seqs=4):
+    cfg = lm_config_from_json(cfg_json, "t")
+    w = GopopelWeights(cfg, sd, device, dtype, max_positions=max_tokens)
+    return LLMEngine(cfg, device, weights=w, max_seqs=max_seqs, max_seq_len=max_tokens,
+                     block_size=block, num_blocks=max_tokens // block, use_graphs=False, dtype=dtype)
+
+
+def rel_err(got, want, q: float = 1.0) -> float:
+    """RMS difference (mean removed per row) over the RMS of the wanted logits:
+    the worst row, or the ``q`` quantile of the rows."""
+    d = got.double().cpu() - want.double()
+    d = d - d.mean(-1, keepdim=True)
+    w = want - want.mean(-1, keepdim=True)
+    return float((d.pow(2).mean(-1).sqrt() / w.pow(2).mean().sqrt()).quantile(q))
+
+
+def feed(eng, seq, toks, cuts):
+    """Feed ``toks`` to one sequence in portions of ``cuts`` sizes (cycled);
+    returns the logits of every position."""
+    out, i, k = [], 0, 0
+    while i < len(toks):
+        n = min(cuts[k % len(cuts)], len(toks) - i)
+        out.append(eng.step_logits([seq], [toks[i:i + n]], [list(range(n))]))
+        i, k = i + n, k + 1
+    return torch.cat(out)
+
+
+def tokens(n, vocab, seed):
+    g = torch.Generator().manual_seed(seed)
+    return torch.randint(0, vocab, (n,), generator=g).tolist()
+
+
+# both mixer kinds in a mixed order, grouped and ungrouped heads, a layer
+# without a feed-forward, a layer without value mixing BEFORE and after the first
+# mixing one, value layouts of equal width but other head counts
+FULL = [(O.latent(), O.dense_ff()),
+        (O.biased(heads=3, kv_heads=3, dim=8, vdim=6, window=11, v_mix=False), O.dense_ff(24)),
+        (O.biased(), O.dense_ff()),
+        (O.latent(heads=2, dim=6, rot_dim=8, vdim=4, kv_rank=9, q_rank=7, window=21), None),
+        (O.biased(heads=4, kv_heads=4, dim=10, vdim=5, window=17), O.dense_ff(16)),
+        (O.biased(heads=2, kv_heads=1, dim=16, vdim=20, window=3), None)]
+
+
+@pytest.fixture(scope="module")
+def full_model():
+    cfg = O.make_config(FULL)
+    return cfg, O.make_weights(cfg, 1)
+
+
+def test_registry_reads_config(full_model):
+    cfg_json, _ = full_model
+    cfg = lm_config_from_json(json.loads(json.dumps(cfg_json)))
+    assert family_of(cfg).name == "gopopel" and family_of(cfg_json).hybrid
+    assert cfg.n_layers == len(FULL) and cfg.layers[3].mlp is None and cfg.embed_scale == 1.7
+    assert cfg.first_v_mix == 2 and not cfg.layers[1].mixer.v_mix
+    assert cfg.layers[2].mixer.window == 6 and cfg.layers[2].mixer.sink and cfg.layers[2].mixer.alibi
+    assert cfg.layers[0].mixer.window == 9 and cfg.layers[0].mixer.gate
+    assert cfg.layers[0].mixer.q_rank == 14 and cfg.layers[0].mlp.act == "relu2"
+    assert config_to_json(cfg) == json.loads(json.dumps(cfg_json))
+    for li, path, val in ((2, ("kv_heads",), 3), (0, ("rot", "dims"), 6), (0, ("rot", "dims"), 3),
+                          (4, ("vdim",), 7), (0, ("mask", "size"), -1), (0, ("q_rank",), 0)):
+        bad = json.loads(json.dumps(cfg_json))
+        m = bad["layers"][li]["mixer"]
+        for k in path[:-1]:
+            m = m[k]
+        m[path[-1]] = val
+        with pytest.raises(ValueError):
+            gopopel_config_from_json(bad)
+    for key, val in (("type", "attention_9"), ("mlp", {"kind": "moe", "ff": 3})):
+        bad = json.loads(json.dumps(cfg_json))
+        bad["layers"][0][key] = val
+        with pytest.raises(ValueError):
+            gopopel_config_from_json(bad)
+    sd = random_state_dict(cfg, 0)
+    want = O.make_weights(cfg_json, 0)
+    mine = {k: tuple(v.shape) for k, v in sd.items()}
+    # the blend weight of a layer that does not mix is not read
+    assert {k: tuple(v.shape) for k, v in want.items() if k != "l1.mix.vmix"} == mine
+
+
+def test_weights_check_shapes(full_model):
+    cfg_json, sd = full_model
+    cfg = lm_config_from_json(cfg_json)
+    for name in ("l0.mix.uk", "l2.mix.v", "l4.mlp.up", "l2.mix.q.norm", "head", "l1.norm1.b"):
+        bad = dict(sd)
+        bad[name] = sd[name][..., :-1] if sd[name].dim() == 1 else sd[name][:-1]
+        with pytest.raises(ValueError):
+            GopopelWeights(cfg, bad, "cpu", torch.float32, 64)
+
+
+# ------------------------------------------------------ each mechanism alone
+def _meta(lens, starts, device):
+    cu = torch.tensor([0] + lens).cumsum(0).to(torch.int32)
+    pos = torch.cat([s + torch.arange(n) for n, s in zip(lens, starts)]).to(torch.int32)
+    return cu.to(device), pos.to(device)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("d", [37, 40, 256, 4100])
+@pytest.mark.parametrize("rows", [5, 600])
+def test_residual_step(device, d, rows):
+    g = torch.Generator().manual_seed(0)
+    x = torch.randn(rows, d, generator=g)
+    ys = [torch.randn(rows, d, generator=g) for _ in range(2)]
+    w, b = 1 + torch.randn(d, generator=g) * 0.3, torch.randn(d, generator=g) * 0.2
+    p = DytParams(w.to(device), b.to(device), 0.6)
+    for ydt in (torch.float32, torch.bfloat16):
+        for n in (0, 1, 2):
+            r = x.to(device).clone()
+            adds = [y.to(ydt).to(device) for y in ys[:n]]
+            h = seqmix.residual_dyt(r, adds, p, torch.float32)
+            want = x.double() + sum(y.double().cpu() for y in adds)
+            assert (r.cpu().double() - want).abs().max() < 1e-5
+            assert (h.cpu().double() - O.dynamic_tanh(want, w.double(), b.double(), 0.6)).abs().max() < 1e-5
+    r = x.to(device).clone()
+    assert seqmix.residual_dyt(r, [ys[0].to(device)], None, torch.float32) is None
+    assert (r.cpu().double() - (x.double() + ys[0].double())).abs().max() < 1e-5
+    h = seqmix.residual_dyt(x.to(device).clone(), [], p, torch.bfloat16)
+    assert (h.float().cpu() - O.dynamic_tanh(x, w, b, 0.6)).abs().max() < 0.02
+
+
+def test_stacked_projections():
+    g = torch.Generator().manual_seed(1)
+    parts = [torch.randn(n, 6, generator=g) for n in (3, 8, 13)]
+    w, offs = stack_rows(parts)
+    assert offs == [0, 8, 16] and w.shape == (32, 6)
+    for t, o in zip(parts, offs):
+        assert torch.equal(w[o:o + t.shape[0]], t)
+    assert w[3:8].abs().sum() == 0 and w[29:].abs().sum() == 0
+
+
+def _side_case(device, dtype, T, W, src_off, n, ld, off, zero_from, seed=3):
+    g = torch.Generator().manual_seed(seed)
+    u = torch.randn(T, W, generator=g).to(dtype)
+    dst = torch.full((T, ld), 7.0).to(dtype).to(device)
+    want = torch.full((T, ld), 7.0, dtype=F64)
+    want[:, zero_from:] = 0
+    want[:, off:off + n] = torch.relu(u[:, src_off:src_off + n].double()) ** 2
+    ud = u.to(device)
+    return u, ud, SideCols(ud[:, src_off:src_off + n], dst, off, zero_from), dst, want
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H,G,D,Dv,n,ld,off,zero_from", [
+    (4, 2, 16, 16, 40, 112, 64, 64), (3, 1, 7, 5, 9, 40, 16, 15), (2, 2, 96, 48, 300, 400, 96, 96),
+    (1, 1, 1, 1, 1, 3, 1, 1), (5, 5, 6, 3, 33, 51, 15, 15)])
+def test_attention_inputs(device, dtype, H, G, D, Dv, n, ld, off, zero_from):
+    """q | k | v rows -> per-head RMS norms with shared weights, value mixing and
+    the paged append, beside the squared feed-forward columns; aligned and
+    unaligned sizes, padding rows, with and without an earlier layer's values."""
+    T, blk = 11, 4
+    v_off, eps = (H + G) * D, 1e-3
+    src_off = -(-(v_off + G * Dv) // 8) * 8
+    u, ud, side, dst, wside = _side_case(device, dtype, T, src_off + n + 3, src_off, n, ld, off, zero_from)
+    g = torch.Generator().manual_seed(5)
+    qn, kn = 1 + torch.randn(D, generator=g), 1 + torch.randn(D, generator=g)
+    vf = torch.randn(T, G * Dv + 2, generator=g).to(dtype)
+    pos = torch.arange(T, dtype=torch.int32)
+    slots = torch.tensor([3, 2, 1, 0, 7, 6, 5, 4, -1, 9, 8], dtype=torch.int32)
+    tol = 2e-5 if dtype == torch.float32 else 0.04
+    for lam in (None, 0.3):
+        kc = torch.zeros(3, blk, G * D, device=device, dtype=dtype)
+        vc = torch.zeros(3, blk, G * Dv, device=device, dtype=dtype)
+        q = seqmix.qk_prep_append(ud, H, G, D, Dv, v_off, None, 0, eps, None, pos.to(device), kc, vc,
+                                  slots.to(device), dtype, qn.to(device), kn.to(device),
+                                  None if lam is None else (vf.to(device)[:, 1:1 + G * Dv], lam), side)
+        x = u.double()
+        wq = O.norm_plain(x[:, :H * D].view(T, H, D), qn.double(), eps)
+        wk = O.norm_plain(x[:, H * D:v_off].view(T, G, D), kn.double(), eps)
+        wv = O.mix_values(x[:, v_off:v_off + G * Dv],
+                          None if lam is None else vf[:, 1:1 + G * Dv].double(), lam)
+        ok = slots >= 0
+        assert (q.cpu().double().view(T, H, D) - wq).abs().max() < tol
+        kk = kc.view(-1, G, D)[slots[ok].long()].cpu().double()
+        assert (kk - wk[ok]).abs().max() < tol
+        vv = vc.view(-1, G * Dv)[slots[ok].long()].cpu().double()
+        assert (vv - wv[ok]).abs().max() < tol
+        assert ((dst.cpu().double() - wside).abs() <= 1e-6 + (0.01 if dtype != torch.float32 else 1e-6)
+                * wside.abs()).all()
+        dst.fill_(7.0)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("R,Dr,dims,Rq,n", [(16, 8, 8, 24, 40), (9, 6, 4, 5, 7), (130, 2, 2, 0, 0),
+                                            (3, 4, 0, 300, 5)])
+def test_latent_inputs(device, dtype, R, Dr, dims, Rq, n):
+    """Latent norm, rotated key part and append, the query latent's norm, and the
+    squared feed-forward columns of the same rows."""
+    T, blk, base, eps = 9, 4, 70.0, 1e-3
+    up = Rq + R + Dr
+    u, ud, side, dst, wside = _side_case(device, dtype, T, up + n + 1, up, n, n + 6, 4, 3)
+    g = torch.Generator().manual_seed(6)
+    nw, qw = torch.randn(R, generator=g), torch.randn(max(Rq, 1), generator=g)
+    pos = torch.tensor([0, 1, 2, 9, 10, 17, 30, 31, 32], dtype=torch.int32)
+    slots = torch.tensor([3, 2, 1, 0, 7, -1, 5, 4, 8], dtype=torch.int32)
+    cs = seqmix.rope_table_pairs(dims, 40, base, None, device)
+    cache = torch.zeros(3, blk, R + Dr, device=device, dtype=dtype)
+    cq = seqmix.latent_inputs(ud[:, Rq:up], nw.to(device), eps, pos.to(device), cs, cache,
+                              slots.to(device), R, dims, ud[:, :Rq] if Rq else None,
+                              qw.to(device) if Rq else None, side if n else None)
+    x = u.double()
+    tol = 2e-5 if dtype == torch.float32 else 0.04
+    want = torch.cat([O.norm_plain(x[:, Rq:Rq + R], nw.double(), eps),
+                      O.rotate_pairs(x[:, None, Rq + R:up], dims, base, pos)[:, 0]], -1)
+    ok = slots >= 0
+    got = cache.view(-1, R + Dr)[slots[ok].long()].cpu().double()
+    assert (got - want[ok]).abs().max() < tol
+    if Rq:
+        assert (cq.cpu().double() - O.norm_plain(x[:, :Rq], qw.double(), eps)).abs().max() < tol
+    else:
+        assert cq is None
+    if n:
+        assert ((dst.cpu().double() - wside).abs() <= 1e-6 + 0.01 * wside.abs()).all()
+
+
+def _paged(rows, lens, blk, device, seed=0):
+    """Per-sequence row sets -> page tensors with shuffled pages, and the table."""
+    nb = sum(-(-n // blk) for n in lens) + 2
+    perm = torch.randperm(nb, generator=torch.Generator().manual_seed(seed)).tolist()
+    pages = [torch.full((nb, blk, r[0].shape[1]), 7.0) for r in rows]
+    bt = torch.zeros(len(lens), max(-(-n // blk) for n in lens), dtype=torch.int32)
+    for b, n in enumerate(lens):
+        for j in range(-(-n // blk)):
+            page = perm.pop()
+            bt[b, j] = page
+            m = min(blk, n - j * blk)
+            for pt, r in zip(pages, rows):
+                pt[page, :m] = r[b][j * blk:j * blk + m]
+    return [pt.to(device) for pt in pages], bt.to(device)
+
+
+def _attn_case(device, dtype, H, G, D, Dv, window, lens, feeds, mfma=None, spike=None, seed=2,
+               splits=None, low=False):
+    """Sequences of ``lens`` keys whose last ``feeds`` positions are this step's
+    queries, with a distance bias and a learned sink, written into a column
+    slice of a wider row. ``spike`` = (distance back, strength): the key that
+    far behind each query gets a large score. ``low``: every score far below
+    zero, so that the sink takes almost all of the weight (a bias measured from
+    position 0 instead of from the query would change its share)."""
+    g = torch.Generator().manual_seed(seed)
+    B = len(lens)
+    ks = [torch.randn(n, G * D, generator=g).to(dtype).float() for n in lens]
+    vs = [torch.randn(n, G * Dv, generator=g).to(dtype).float() for n in lens]
+    qs = [torch.randn(n, H * D, generator=g) for n in lens]
+    if low:
+        for b in range(B):
+            ks[b] = (ks[b].abs() + 0.5).to(dtype).float()
+            qs[b] = -(qs[b].abs() + 0.5)
+    if spike is not None:
+        back, strength = spike
+        for b, n in enumerate(lens):
+            for i in range(back, n):
+                kk = ks[b][i - back].view(G, D)
+                qs[b][i] = (kk.repeat_interleave(H // G, 0) * strength / D).reshape(-1)
+    qs = [q.to(dtype).float() for q in qs]
+    (kc, vc), bt = _paged([ks, vs], lens, 16, device, seed)
+    starts = [n - f for n, f in zip(lens, feeds)]
+    cu, pos = _meta(feeds, starts, device)
+    q = torch.cat([qs[b][starts[b]:] for b in range(B)])
+    ctx = torch.tensor(lens, dtype=torch.int32, device=device)
+    scale = 1.0 / math.sqrt(D)
+    sink = torch.randn(H, generator=g)
+    slopes = seqmix.alibi_slopes(H, device)
+    assert slopes.tolist() == pytest.approx(O.slopes(H))
+    wide = torch.full((q.shape[0], H * Dv + 8), 3.0, device=device, dtype=dtype)
+    seqmix.window_attention(q.to(device, dtype), kc.to(dtype), vc.to(dtype), cu, ctx, bt, pos, scale,
+                            0.0, window, 0, None, H, G, D, Dv, max(feeds), matrix_cores=mfma,
+                            max_ctx=max(lens), key_splits=splits, sink=sink.to(device),
+                            slopes=slopes, out=wide[:, :H * Dv])
+    assert (wide[:, H * Dv:] == 3.0).all()
+    want = []
+    for b, n in enumerate(lens):
+        o = O.attention(qs[b].double().view(n, H, D), ks[b].double().view(n, G, D),
+                        vs[b].double().view(n, G, Dv), scale, window, O.slopes(H), sink.double())
+        want.append(o[starts[b]:].reshape(-1, H * Dv))
+    return wide[:, :H * Dv].cpu().double(), torch.cat(want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("H,G,D,Dv,window", [(4, 2, 16, 16, 5), (3, 3, 8, 24, 64), (6, 1, 64, 64, 37),
+                                             (8, 1, 24, 8, 0), (2, 2, 6, 130, 1), (5, 5, 7, 3, 90)])
+def test_biased_attention_with_sink(device, H, G, D, Dv, window):
+    for low in (False, True):
+        got, want = _attn_case(device, torch.float32, H, G, D, Dv, window, [150, 1, 37, 90],
+                               [150, 1, 1, 23], low=low)
+        assert (got - want).abs().max() < 2e-5
+    if device == "cuda":
+        for splits in (2, 5):
+            got, want = _attn_case(device, torch.float32, H, G, D, Dv, window, [700, 3, 64, 65],
+                                   [1, 1, 1, 2], mfma=False, splits=splits, low=True)
+            assert (got - want).abs().max() < 2e-5
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("back", [0, 1, 4, 5, 6, 63, 64, 65, 127, 128, 129])
+def test_window_edges_of_biased_attention(device, back):
+    """A key ``back`` positions behind every query carries almost all of the
+    softmax weight if it is visible: windows of 5, 64 and 128 keys, in a prompt
+    portion and in single tokens."""
+    for window in (5, 64, 128):
+        for feeds in ([300], [1]):
+            got, want = _attn_case(device, torch.float32, 2, 1, 16, 16, window, [300], feeds,
+                                   spike=(back, 60.0))
+            assert (got - want).abs().max() < 3e-5, (window, feeds)
+
+
+def _latent_case(device, dtype, H, D, Dr, Dv, R, window, lens, feeds, prompt, spike=None, seed=4,
+                 gate=True):
+    """Windowed latent attention between its projections (``latent_heads``) on
+    given queries, latents and rotary key parts, against the oracle's softmax
+    over materialised keys. ``prompt``: allow the matrix-core prompt path.
+    ``spike`` = (distance back, strength)."""
+    from types import SimpleNamespace
+    from loqa_hub_amd.models.configs import LatentAttnConfig, RotaryConfig
+    from loqa_hub_amd.models.pipizen import latent_heads, latent_prompt_layout
+    g = torch.Generator().manual_seed(seed)
+    B, base, scale = len(lens), 80.0, (D + Dr) ** -0.5
+    m = LatentAttnConfig(H, D, Dr, Dv, R, scale, RotaryConfig(Dr, base), q_rank=1, gate=gate,
+                         window=window)
+
+    def r(*shape):
+        return torch.randn(*shape, generator=g).to(dtype).float()
+    wuk, wuv = r(H, D, R) / R ** 0.5, r(H, Dv, R) / R ** 0.5
+    wuk, wuv = wuk.to(dtype).float(), wuv.to(dtype).float()
+    cs_ = [r(n, R) for n in lens]
+    krs = [O.rotate_pairs(r(n, 1, Dr).double(), Dr, base)[:, 0].to(dtype).float() for n in lens]
+    qs = [r(n, H, D + Dr) for n in lens]
+    if spike is not None:
+        back, strength = spike
+        for b, n in enumerate(lens):
+            kk = torch.einsum("hdr,nr->nhd", wuk, cs_[b])
+            for i in range(back, n):
+                k = kk[i - back]
+                qs[b][i, :, :D] = k * strength / k.pow(2).sum(-1, keepdim=True) / scale
+                qs[b][i, :, D:] = 0
+        qs = [q.to(dtype).float() for q in qs]
+    gates = [r(n, H * Dv) for n in lens]
+    (pages,), bt = _paged([[torch.cat([c, k], -1) for c, k in zip(cs_, krs)]], lens, 16, device, seed)
+    starts = [n - f for n, f in zip(lens, feeds)]
+    cu, pos = _meta(feeds, starts, device)
+    dev = torch.device(device)
+    L = {"wq": torch.zeros(H * (D + Dr), 8, dtype=dtype, device=dev), "qw": D + Dr,
+         "wuk": wuk.to(dev, dtype), "wuv_t": wuv.transpose(1, 2).contiguous().to(dev, dtype),
+         "sink": None, "cos_sin": seqmix.rope_table_pairs(Dr, max(lens), base, None, dev)}
+    if prompt:
+        latent_prompt_layout(L, m, dtype, dev)
+        assert "prompt_sizes" in L
+    q = torch.cat([q[s:] for q, s in zip(qs, starts)])
+    q = torch.nn.functional.pad(q, (0, L["qw"] - D - Dr)).reshape(q.shape[0], -1).to(dev, dtype)
+    reach = [min(n, f + window - 1) if window else n for n, f in zip(lens, feeds)]
+
+    def cum(x):
+        return torch.tensor([0] + x).cumsum(0).to(torch.int32).to(dev)
+    meta = SimpleNamespace(max_q=max(feeds), max_ctx=max(lens), cu_q=cu, positions=pos,
+                           ctx_lens=torch.tensor(lens, dtype=torch.int32, device=dev),
+                           block_tables=bt, cu_k=cum(lens), total_k=sum(lens),
+                           window_k={window: (cum(reach), sum(reach))})
+    gt = torch.cat([x[s:] for x, s in zip(gates, starts)]).to(dev, dtype) if gate else None
+    wide = torch.full((q.shape[0], H * Dv + 8), 3.0, device=dev, dtype=dtype)
+    latent_heads(L, m, q, pages.to(dtype), meta, 1 if prompt else 10 ** 9, gt, wide[:, :H * Dv])
+    assert (wide[:, H * Dv:] == 3.0).all()
+    want = []
+    for b, n in enumerate(lens):
+        k = torch.cat([torch.einsum("hdr,nr->nhd", wuk.double(), cs_[b].double()),
+                       krs[b].double()[:, None].expand(n, H, Dr)], -1)
+        v = torch.einsum("hdr,nr->nhd", wuv.double(), cs_[b].double())
+        qq = torch.cat([qs[b].double()[..., :D],
+                        O.rotate_pairs(qs[b].double()[..., D:], Dr, base)], -1)
+        o = O.attention(qq, k, v, scale, window).reshape(n, H * Dv)
+        if gate:
+            o = o * torch.sigmoid(gates[b].double())
+        want.append(o[starts[b]:])
+    return wide[:, :H * Dv].cpu().double(), torch.cat(want)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("H,D,Dr,Dv,R,window", [(3, 8, 4, 10, 12, 7), (1, 5, 6, 3, 7, 64),
+                                                (6, 32, 32, 48, 96, 129), (4, 4, 2, 6, 8, 1),
+                                                (2, 16, 8, 16, 33, 0)])
+def test_windowed_latent_attention(device, H, D, Dr, Dv, R, window):
+    for gate in (True, False):
+        got, want = _latent_case(device, torch.float32, H, D, Dr, Dv, R, window, [150, 1, 37, 90],
+                                 [150, 1, 1, 23], False, gate=gate)
+        assert (got - want).abs().max() < 3e-5
+    got, want = _latent_case(device, torch.float32, H, D, Dr, Dv, R, window, [700, 3, 64, 65],
+                             [1, 1, 1, 2], False)
+    assert (got - want).abs().max() < 3e-5
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("back", [0, 1, 4, 5, 6, 63, 64, 65, 127, 128, 129])
+def test_window_edges_of_latent_attention(device, back):
+    for window in (5, 64, 128):
+        for feeds in ([300], [1]):
+            got, want = _latent_case(device, torch.float32, 2, 8, 4, 8, 16, window, [300], feeds,
+                                     False, spike=(back, 25.0))
+            assert (got - want).abs().max() < 5e-5, (window, feeds)
+
+
+# --------------------------------------------------------- the whole model
+@pytest.mark.parametrize("device", DEVICES)
+def test_residual_after_every_layer(device, full_model):
+    cfg, sd = full_model
+    toks = tokens(29, cfg["vocab"], 10)
+    want = []
+    O.forward(cfg, sd, toks, want)
+    eng = engine(cfg, sd, device)
+    max_q, max_ctx, host = eng._meta([eng.open_sequence()], [toks], decode=False)
+    host["logit_idx"] = np.asarray([0], np.int64)
+    meta = eng._build_meta(eng._to_device(host), max_q, max_ctx, False)
+    got = []
+    eng.model.forward(meta, eng.kv, got)
+    assert len(got) == len(want) == len(FULL)
+    for r, (a, b) in enumerate(zip(got, want)):
+        assert (a.cpu().double() - b).abs().max() < 1e-4 * float(b.abs().max()), r
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_whole_prompt(device, dtype, full_model):
+    cfg, sd = full_model
+    toks = tokens(70, cfg["vocab"], 11)
+    want = O.forward(cfg, sd, toks)
+    eng = engine(cfg, sd, device, dtype)
+    got = eng.step_logits([eng.open_sequence()], [toks], [list(range(len(toks)))])
+    if dtype == torch.float32:
+        assert rel_err(got, want) < TOL[dtype]
+    else:
+        # a width this small averages little of the 16-bit rounding away: the
+        # typical row is what is pinned
+        assert rel_err(got, want, 0.5) < TOL[dtype] and rel_err(got, want) < 0.2
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("cuts", [[1], [2], [3, 2, 7], [16], [17, 1, 1, 30], [5, 64]],
+                         ids=lambda c: "x".join(map(str, c)))
+def test_portions_and_decode(device, cuts, full_model):
+    """Token-by-token decoding and portions of any size (down to two tokens,
+    across page borders at 16 and the windows' edges) give the whole prompt's
+    logits."""
+    cfg, sd = full_model
+    toks = tokens(53, cfg["vocab"], 12)
+    want = O.forward(cfg, sd, toks)
+    eng = engine(cfg, sd, device)
+    got = feed(eng, eng.open_sequence(), toks, cuts)
+    assert rel_err(got, want) < TOL[torch.float32]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_unequal_batch_and_reuse(device, dtype, full_model):
+    """Four unequal requests, portions beside single tokens in one step; two
+    end early and two new ones take over their pages. Every request's logits
+    equal the ones it gets alone (oracle); values are mixed with the values of
+    the same token of the same request whatever its place in the batch."""
+    cfg, sd = full_model
+    V = cfg["vocab"]
+    reqs = {n: tokens(L, V, 20 + i) for i, (n, L) in
+            enumerate([("a", 41), ("b", 1), ("c", 18), ("d", 33), ("e", 25), ("f", 47)])}
+    want = {n: O.forward(cfg, sd, t) for n, t in reqs.items()}
+    eng = engine(cfg, sd, device, dtype, max_tokens=192, max_seqs=4)
+    plan = {"a": [7, 1, 1, 16, 2, 1, 13], "b": [1], "c": [2, 15, 1], "d": [16, 16, 1],
+            "e": [3, 1, 21], "f": [30, 1, 16]}
+    at = {n: 0 for n in reqs}
+    live, waiting, got = {}, ["a", "b", "c", "d", "e", "f"], {n: [] for n in reqs}
+    steps = 0
+    while waiting or live:
+        while waiting and len(live) < 4:
+            n = waiting.pop(0)
+            live[n] = eng.open_sequence()
+        names = list(live)
+        feeds, wants = [], []
+        for n in names:
+            k = plan[n].pop(0)
+            feeds.append(reqs[n][at[n]:at[n] + k])
+            wants.append(list(range(k)))
+            at[n] += k
+        out = eng.step_logits([live[n] for n in names], feeds, wants)
+        o = 0
+        for n, f in zip(names, feeds):
+            got[n].append(out[o:o + len(f)])
+            o += len(f)
+            if at[n] == len(reqs[n]):
+                eng.close_sequence(live.pop(n))
+        steps += 1
+    assert steps > 5
+    for n in reqs:
+        err = rel_err(torch.cat(got[n]), want[n], 1.0 if dtype == torch.float32 else 0.5)
+        assert err < TOL[dtype], n
+    assert eng.kv.pool.free_blocks() == 192 // 16
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_pages_reused_clean(device, full_model):
+    """A pool of exactly one request's size, every page overwritten with junk
+    between requests: the next request must not see it."""
+    cfg, sd = full_model
+    eng = engine(cfg, sd, device, max_tokens=48, max_seqs=1)
+    for i, n in enumerate([40, 48, 3, 33]):
+        toks = tokens(n, cfg["vocab"], 30 + i)
+        seq = eng.open_sequence()
+        got = feed(eng, seq, toks, [9, 1, 2])
+        eng.close_sequence(seq)
+        assert rel_err(got, O.forward(cfg, sd, toks)) < TOL[torch.float32], i
+        for a, b in eng.kv.kv_rows.values():
+            a.fill_(50.0), b.fill_(-50.0)
+        for t in eng.kv.latent.values():
+            t.fill_(30.0)
+    assert eng.kv.pool.free_blocks() == 3
+
+
+def _peaked(mixer, window):
+    """A single layer of one mixer whose scores are sharp enough that one key
+    more or less shows in the logits."""
+    kind, m = mixer
+    m = dict(m, mask={"size": window})
+    cfg = O.make_config([((kind, m), O.dense_ff(16))], width=16)
+    sd = O.make_weights(cfg, 8)
+    if kind == "attention":
+        sd["l0.mix.q.norm"] *= 3.0
+        sd["l0.mix.sink"] -= 2.0
+    return cfg, sd
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("mixer", [O.biased(heads=2, kv_heads=1, dim=8, vdim=8),
+                                   O.latent(heads=2, dim=8, rot_dim=4, vdim=8, kv_rank=8, q_rank=8,
+                                            scale=1.5)], ids=lambda m: m[0])
+@pytest.mark.parametrize("window", [16, 17, 32, 33, 1])
+def test_window_edges_in_prompts_and_decoding(device, mixer, window):
+    """Windows that end on, just before and just after a page border; the keys
+    just inside and just outside pass the edge in portions and in decoding. A
+    window that is one key off would miss the tolerance many times over."""
+    cfg, sd = _peaked(mixer, window)
+    toks = tokens(70, cfg["vocab"], 14)
+    want = O.forward(cfg, sd, toks)
+    off = json.loads(json.dumps(cfg))
+    off["layers"][0]["mixer"]["mask"]["size"] = window + 1
+    assert rel_err(O.forward(off, sd, toks), want) > 20 * TOL[torch.float32]
+    for cuts in ([70], [40] + [1] * 30, [15, 2, 16]):
+        eng = engine(cfg, sd, device)
+        got = feed(eng, eng.open_sequence(), toks, cuts)
+        assert rel_err(got, want) < TOL[torch.float32], cuts
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("mixer", [O.biased(heads=8, kv_heads=2, dim=8, vdim=8, scale=1.0),
+                                   O.latent(heads=2, dim=8, rot_dim=2, vdim=8, kv_rank=8, q_rank=8,
+                                            scale=2.0, base=1e6)], ids=lambda m: m[0])
+def test_far_keys(device, mixer):
+    """Hundreds of visible keys; the flattest head's bias spans only a few
+    units over the whole window, so far keys compete."""
+    cfg, sd = _peaked(mixer, 250)
+    toks = tokens(300, cfg["vocab"], 15)
+    want = O.forward(cfg, sd, toks)
+    for cuts in ([300], [290] + [1] * 10, [130, 2, 59]):
+        eng = engine(cfg, sd, device, max_tokens=304)
+        got = feed(eng, eng.open_sequence(), toks, cuts)
+        assert rel_err(got, want) < TOL[torch.float32], cuts
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_first_tokens(device, full_model):
+    cfg, sd = full_model
+    for n in (1, 2, 3):
+        toks = tokens(n, cfg["vocab"], 16 + n)
+        eng = engine(cfg, sd, device)
+        got = feed(eng, eng.open_sequence(), toks, [1])
+        assert rel_err(got, O.forward(cfg, sd, toks)) < TOL[torch.float32]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_other_sizes(device, dtype):
+    """Sizes that are unequal where a usual model makes them equal, single and
+    many heads, odd sizes, a window of one, an embedding scale of 1, no layer
+    that mixes values, a single mixing layer (whose blend weight is unused)."""
+    layers = [
+        (O.biased(heads=1, kv_heads=1, dim=10, vdim=3, window=1, v_mix=False), None),
+        (O.latent(heads=1, dim=5, rot_dim=6, vdim=3, kv_rank=7, q_rank=5, window=30), O.dense_ff(9)),
+        (O.biased(heads=6, kv_heads=3, dim=5, vdim=7, window=100, v_mix=False), O.dense_ff(11)),
+        (O.latent(heads=5, dim=2, rot_dim=8, vdim=7, kv_rank=3, q_rank=20, scale=0.3, window=2), None)]
+    for extra in ([], [(O.biased(heads=12, kv_heads=4, dim=3, vdim=1, window=40), O.dense_ff(8))]):
+        cfg = O.make_config(layers + extra, width=20, vocab=31, embed_scale=1.0)
+        sd = O.make_weights(cfg, 10)
+        toks = tokens(45, 31, 17)
+        want = O.forward(cfg, sd, toks)
+        eng = engine(cfg, sd, device, dtype)
+        got = feed(eng, eng.open_sequence(), toks, [19, 1, 2])
+        if dtype == torch.float32:
+            assert rel_err(got, want) < TOL[dtype]
+        else:
+            assert rel_err(got, want, 0.5) < TOL[dtype] and rel_err(got, want, 0.9) < 0.2
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_value_mixing_extremes(device):
+    """A stack of identical mixing layers with the blend weight at 0 and at 1:
+    at 0 every layer keeps its own values, at 1 it takes the first one's."""
+    layers = [(O.biased(heads=2, kv_heads=2, dim=8, vdim=8, window=12), O.dense_ff(16))] * 3
+    cfg = O.make_config(layers, width=16)
+    toks = tokens(40, cfg["vocab"], 19)
+    outs = []
+    for lam in (0.0, 1.0):
+        sd = O.make_weights(cfg, 12)
+        for i in range(3):
+            sd[f"l{i}.mix.vmix"] = torch.tensor(lam)
+        want = O.forward(cfg, sd, toks)
+        eng = engine(cfg, sd, device)
+        got = feed(eng, eng.open_sequence(), toks, [21, 1, 6])
+        assert rel_err(got, want) < TOL[torch.float32]
+        outs.append(want)
+    assert rel_err(outs[0], outs[1]) > 0.05
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_long_decode(device):
+    layers = [(O.biased(heads=2, kv_heads=1, dim=8, vdim=8, window=24), O.dense_ff(16)),
+              (O.latent(heads=2, dim=8, rot_dim=4, vdim=8, window=40), None),
+              (O.biased(heads=2, kv_heads=1, dim=8, vdim=8, window=70), O.dense_ff(16))]
+    cfg = O.make_config(layers, width=16, vocab=40)
+    sd = O.make_weights(cfg, 11)
+    toks = tokens(150, 40, 18)
+    want = O.forward(cfg, sd, toks)
+    eng = engine(cfg, sd, device)
+    got = feed(eng, eng.open_sequence(), toks, [10] + [1] * 140)
+    assert rel_err(got, want) < TOL[torch.float32]
+
+
+def _greedy(cfg, sd, p, n_new):
+    seq = list(p)
+    for _ in range(n_new):
+        seq.append(int(O.forward(cfg, sd, seq)[-1].argmax()))
+    return seq[len(p):]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_greedy_generation_through_scheduler(device, full_model):
+    """Schema-less requests through ``submit_batch`` (continuous batching:
+    inline prompts, chunked prompts in mixed steps, decode steps) produce the
+    oracle's greedy continuation; a prompt that shares its first pages with an
+    earlier one takes them from the prefix cache."""
+    cfg, sd = full_model
+    V = cfg["vocab"]
+    prompts = [tokens(n, V, 40 + i) for i, n in enumerate([5, 90, 23, 70])]
+    prompts.append(prompts[1][:64] + tokens(9, V, 47))
+    n_new = 6
+    want = [_greedy(cfg, sd, p, n_new) for p in prompts]
+    eng = engine(cfg, sd, device, max_tokens=512, max_seqs=4)
+    eng.chunk_prefill = 32          # prompts longer than inline_prefill go in 32-token chunks
+    eng.inline_prefill = 8
+    reqs = [GenRequest(p, None, max_new_tokens=n_new) for p in prompts]
+    try:
+        eng.submit_batch(reqs[:2]).result(timeout=300)
+        f1 = eng.submit_batch(reqs[2:3])
+        f2 = eng.submit_batch(reqs[3:4])
+        f1.result(timeout=300), f2.result(timeout=300)
+        hits = eng.stats["prefix_hit_tokens"]
+        eng.submit_batch(reqs[4:]).result(timeout=300)
+        assert eng.stats["prefix_hit_tokens"] - hits == 64
+    finally:
+        eng.stop()
+    for r, w in zip(reqs, want):
+        assert r.done and r.grammar.emitted == w
+
+
+def test_generate_entry_point(full_model):
+    cfg, sd = full_model
+    p = tokens(12, cfg["vocab"], 50)
+    eng = engine(cfg, sd, "cpu")
+    r = eng.generate([GenRequest(p, None, max_new_tokens=3)])[0]
+    assert r.grammar.emitted == _greedy(cfg, sd, p, 3)
+
+
+def test_checkpoint_round_trip(tmp_path, full_model):
+    """save -> config.json + safetensors -> registry -> the same logits."""
+    from loqa_hub_amd.models.loader import save_gopopel
+    from loqa_hub_amd.models.registry import lm_config_of_checkpoint, load_lm_weights
+    cfg_json, sd = full_model
+    cfg = lm_config_from_json(cfg_json, "t")
+    save_gopopel(cfg, {k: v.to(torch.bfloat16) for k, v in sd.items()}, str(tmp_path / "ck"))
+    cfg2 = lm_config_of_checkpoint(str(tmp_path / "ck"), "t")
+    assert cfg2 == cfg and family_of(cfg2).name == "gopopel"
+    w = load_lm_weights(cfg2, str(tmp_path / "ck"), "cpu", dtype=torch.float32, max_positions=64)
+    eng = LLMEngine(cfg2, "cpu", weights=w, max_seqs=1, max_seq_len=64, block_size=16, num_blocks=4,
+                    use_graphs=False, dtype=torch.float32)
+    toks = tokens(30, cfg_json["vocab"], 51)
+    got = eng.step_logits([eng.open_sequence()], [toks], [list(range(30))])
+    assert rel_err(got, O.forward(cfg_json, sd, toks)) < TOL[torch.float32]
+
+
+def test_trace_replay_program(tmp_path, full_model):
+    """The replay command on a checkpoint folder: steps on stdin, logits files
+    and ``done`` lines out; a request that sits out a step goes on later."""
+    from loqa_hub_amd.models.loader import write_safetensors
+    cfg, sd = full_model
+    model = tmp_path / "m"
+    model.mkdir()
+    (model / "config.json").write_text(json.dumps(cfg))
+    write_safetensors({k: v.to(torch.bfloat16) for k, v in sd.items()},
+                      str(model / "model.safetensors"))
+    a, b = tokens(20, cfg["vocab"], 60), tokens(9, cfg["vocab"], 61)
+    steps = [
+        {"step": 0, "entries": [{"id": "a", "tokens": a[:11], "want": [0, 10]}], "end": []},
+        {"step": 1, "entries": [{"id": "b", "tokens": b[:8], "want": []}], "end": []},
+        {"step": 2, "entries": [{"id": "a", "tokens": a[11:], "want": [8]},
+                                {"id": "b", "tokens": b[8:], "want": [0]}], "end": ["a", "b"]},
+    ]
+    out = tmp_path / "out"
+    p = subprocess.run([sys.executable, "-m", "loqa_hub_amd.cli.trace_run", "--model", str(model),
+                        "--dtype", "float32", "--out", str(out), "--max-tokens", "64",
+                        "--device", "cpu"],
+                       input="\n".join(json.dumps(s) for s in steps) + "\n", text=True,
+                       capture_output=True, cwd=ROOT, timeout=300)
+    assert p.returncode == 0, p.stderr
+    assert [ln for ln in p.stdout.splitlines() if ln.startswith("done")] == \
+        ["done 0", "done 1", "done 2"]
+    V = cfg["vocab"]
+    wa, wb = O.forward(cfg, sd, a), O.forward(cfg, sd, b)
+    g0 = torch.from_numpy(np.fromfile(out / "0.f32", dtype="<f4").reshape(-1, V))
+    g2 = torch.from_numpy(np.fromfile(out / "2.f32", dtype="<f4").reshape(-1, V))
+    assert not (out / "1.f32").exists()
+    assert rel_err(g0, wa[[0, 10]]) < TOL[torch.float32]
+    assert rel_err(g2, torch.stack([wa[19], wb[8]])) < TOL[torch.float32]
+
+
+# ------------------------------------------- matrix-core paths (bf16, GPU only)
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,G,D,Dv,window", [(4, 2, 64, 64, 0), (6, 2, 128, 128, 48), (8, 1, 64, 128, 70),
+                                             (3, 3, 80, 48, 130), (2, 1, 24, 8, 33), (4, 4, 112, 72, 64),
+                                             (2, 2, 200, 104, 65), (5, 5, 256, 64, 1)])
+def test_biased_attention_matrix_cores(H, G, D, Dv, window):
+    """The prompt-portion kernel (built and zero-padded head sizes) against the
+    oracle and against the keys-parallel form, also where the sink outweighs
+    every key."""
+    for low in (False, True):
+        lens, feeds = [700, 1, 333, 90, 450], [700, 1, 70, 17, 1]
+        a, want = _attn_case("cuda", torch.bfloat16, H, G, D, Dv, window, lens, feeds, mfma=True,
+                             low=low)
+        b, _ = _attn_case("cuda", torch.bfloat16, H, G, D, Dv, window, lens, feeds, mfma=False,
+                          low=low)
+        scale = float(want.abs().max())
+        assert (a - want).abs().max() < 0.03 * scale and (b - want).abs().max() < 0.03 * scale
+    # medium feeds: narrower row blocks
+    for feeds in ([60, 1], [100, 33]):
+        a, want = _attn_case("cuda", torch.bfloat16, H, G, D, Dv, window, [300, 77], feeds, mfma=True)
+        assert (a - want).abs().max() < 0.03 * float(want.abs().max())
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("back", [0, 31, 63, 64, 65, 127, 128])
+def test_matrix_core_window_edges(back):
+    for window in (32, 64, 128):
+        for D, Dv in ((64, 64), (96, 80)):
+            got, want = _attn_case("cuda", torch.bfloat16, 2, 1, D, Dv, window, [400], [330],
+                                   mfma=True, spike=(back, 60.0))
+            assert (got - want).abs().max() < 0.03 * float(want.abs().max()), (window, D)
+        got, want = _latent_case("cuda", torch.bfloat16, 2, 32, 16, 40, 48, window, [400], [330],
+                                 True, spike=(back, 25.0))
+        assert (got - want).abs().max() < 0.04 * float(want.abs().max()), window
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,D,Dr,Dv,R,window", [(3, 32, 32, 64, 48, 0), (2, 64, 32, 80, 64, 100),
+                                                (4, 128, 64, 128, 96, 129), (5, 17, 6, 21, 24, 33),
+                                                (1, 100, 60, 30, 40, 1)])
+def test_windowed_latent_prompt_pass(H, D, Dr, Dv, R, window):
+    """The prompt path (keys gathered from the windows only, flash attention with
+    the gate in its epilogue, unaligned value sizes) against the oracle and
+    against the folded form."""
+    lens, feeds = [700, 1, 333, 90, 450], [700, 1, 70, 17, 1]
+    a, want = _latent_case("cuda", torch.bfloat16, H, D, Dr, Dv, R, window, lens, feeds, True)
+    b, _ = _latent_case("cuda", torch.bfloat16, H, D, Dr, Dv, R, window, lens, feeds, False)
+    scale = float(want.abs().max())
+    assert (a - want).abs().max() < 0.04 * scale and (b - want).abs().max() < 0.04 * scale
+
+
+@pytest.mark.gpu
+def test_serving_sizes_bf16():
+    """A model with matrix-core head sizes in bfloat16: whole prompt, portions
+    and decoding agree with the oracle within 16-bit rounding, and with each
+    other more closely than with it."""
+    layers = [(O.biased(heads=4, kv_heads=2, dim=64, vdim=64, window=40), O.dense_ff(96)),
+              (O.latent(heads=2, dim=32, rot_dim=32, vdim=64, kv_rank=48, q_rank=64, window=90),
+               O.dense_ff(96)),
+              (O.biased(heads=2, kv_heads=2, dim=80, vdim=64, window=150), O.dense_ff(96))]
+    cfg = O.make_config(layers, width=128, vocab=90)
+    sd = O.make_weights(cfg, 12)
+    toks = tokens(300, 90, 14)
+    want = O.forward(cfg, sd, toks)
+    eng = engine(cfg, sd, "cuda", torch.bfloat16, max_tokens=304)
+    for cuts in ([300], [250, 30] + [1] * 20, [33, 2, 70]):
+        seq = eng.open_sequence()
+        got = feed(eng, seq, toks, cuts)
+        eng.close_sequence(seq)
+        assert rel_err(got, want, 0.5) < TOL[torch.bfloat16] and rel_err(got, want, 0.9) < 0.25, cuts
