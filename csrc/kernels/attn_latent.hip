@@ -12,8 +12,13 @@
 //   on the key part (pairs 2i, 2i+1 of the first `dims` entries), store at the
 //   slot; optionally the RMS norm of a query latent in the same rows, and the
 //   side columns of a parallel layer.
-// latent_attn_kernel: one workgroup per (query token, group of 4 heads,
-//   key split). Key tiles are staged once in LDS (f32, odd row stride) for the
+// latent_attn_mfma_kernel (bf16; R a multiple of 16 up to 512, R + Dr one of 8 up
+//   to 640): one workgroup per (query token, group of 16 heads, key split). Tiles
+//   of 32 keys are staged in LDS once for the 16 heads; scores and outputs run on
+//   the matrix cores with the head on the MFMA column, so the online softmax is
+//   per lane.
+// latent_attn_kernel (f32 and other sizes; latent_attn2_kernel is its form for
+//   even sizes): one workgroup per (query token, group of 4 heads, key split). Key tiles are staged once in LDS (f32, odd row stride) for the
 //   group's heads; each wave owns one head: a lane scores one key of the tile,
 //   the online softmax runs across the wave, and for P.C each lane owns output
 //   entries r = lane + 64 i. Prompt portions, single decode tokens and mixed
@@ -33,40 +38,68 @@ struct LatInParams {
   void* cache; long cache_rows; const int* slots;
   int R, Dr, dims;
   const void* dq; long lddq; const float* qw; int Rq; void* cq;   // query latent [T, Rq], or Rq == 0
+  int vz, vq;                            // the rows can be accessed in runs of four
 };
+
+// The workgroups of a token: the last one norms and stores the cache row, the
+// first one norms the query latent (the same workgroup when there is one), all
+// share the side columns. Rows go in
+// runs of N = 4 entries where they are aligned, else one by one.
+template <typename T, int N>
+__device__ __forceinline__ float li_sumsq(const T* x, int n) {
+  float s = 0.f;
+#pragma unroll 2
+  for (int i = N * threadIdx.x; i < n; i += N * 128) {
+    float f[N];
+    ld_run<T, N>(x + i, f);
+#pragma unroll
+    for (int k = 0; k < N; ++k) s += f[k] * f[k];
+  }
+  return s;
+}
+template <typename T, int N>
+__device__ __forceinline__ void li_scale(const T* x, const float* w, float inv, T* y, int n) {
+#pragma unroll 2
+  for (int i = N * threadIdx.x; i < n; i += N * 128) {
+    float f[N], ww[N];
+    ld_run<T, N>(x + i, f);
+    ld_run<float, N>(w + i, ww);
+#pragma unroll
+    for (int k = 0; k < N; ++k) f[k] *= inv * ww[k];
+    st_run<T, N>(y + i, f);
+  }
+}
 
 template <typename T>
 __global__ __launch_bounds__(128) void latent_inputs_kernel(LatInParams p, SideCols side) {
   __shared__ float part[2][2];
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const bool do_q = p.Rq && blockIdx.y == 0, do_z = blockIdx.y + 1 == gridDim.y;   // uniform
   const T* zr = (const T*)p.z + (size_t)t * p.ldz;
   const T* qr = p.Rq ? (const T*)p.dq + (size_t)t * p.lddq : nullptr;
-  float ss = 0.f, sq = 0.f;
-  for (int i = threadIdx.x; i < p.R; i += 128) {
-    const float v = Act<T>::ld(zr + i);
-    ss += v * v;
+  if (do_q || do_z) {
+    float ss = 0.f, sq = 0.f;
+    if (do_z) ss = p.vz ? li_sumsq<T, 4>(zr, p.R) : li_sumsq<T, 1>(zr, p.R);
+    if (do_q) sq = p.vq ? li_sumsq<T, 4>(qr, p.Rq) : li_sumsq<T, 1>(qr, p.Rq);
+    ss = wave_sum(ss);
+    sq = wave_sum(sq);
+    if (lane == 0) { part[0][wave] = ss; part[1][wave] = sq; }
+    __syncthreads();
   }
-  for (int i = threadIdx.x; i < p.Rq; i += 128) {
-    const float v = Act<T>::ld(qr + i);
-    sq += v * v;
-  }
-  ss = wave_sum(ss);
-  sq = wave_sum(sq);
-  if (lane == 0) { part[0][wave] = ss; part[1][wave] = sq; }
-  __syncthreads();
-  if (p.Rq) {
+  if (do_q) {
     const float inv = 1.f / sqrtf((part[1][0] + part[1][1]) / (float)p.Rq + p.eps);
     T* cq = (T*)p.cq + (size_t)t * p.Rq;
-    for (int i = threadIdx.x; i < p.Rq; i += 128)
-      Act<T>::st(cq + i, Act<T>::ld(qr + i) * inv * p.qw[i]);
+    if (p.vq) li_scale<T, 4>(qr, p.qw, inv, cq, p.Rq);
+    else li_scale<T, 1>(qr, p.qw, inv, cq, p.Rq);
   }
   side_relu2<T>(side, t);
+  if (!do_z) return;
   const int slot = p.slots[t];
   if (slot < 0 || slot >= p.cache_rows) return;    // padding row
   const float inv = 1.f / sqrtf((part[0][0] + part[0][1]) / (float)p.R + p.eps);
   T* row = (T*)p.cache + (size_t)slot * (p.R + p.Dr);
-  for (int i = threadIdx.x; i < p.R; i += 128)
-    Act<T>::st(row + i, Act<T>::ld(zr + i) * inv * p.nw[i]);
+  if (p.vz) li_scale<T, 4>(zr, p.nw, inv, row, p.R);
+  else li_scale<T, 1>(zr, p.nw, inv, row, p.R);
   const int pp = min(max(p.pos[t], 0), p.max_pos - 1);
   const float* csr = p.cs + (size_t)pp * p.dims;     // [dims/2][2]
   for (int i = threadIdx.x; i < p.Dr; i += 128) {
@@ -439,6 +472,240 @@ __global__ __launch_bounds__(LAT_THREADS) void latent_attn2_kernel(LatAttnParams
   }
 }
 
+// ------------------------------------------------------- matrix-core form (bf16)
+#define LM_KT 32            // keys per tile = the depth of one v_mfma_f32_16x16x32_bf16
+#define LM_MAXW 640         // R + Dr
+#define LM_MAXR 512
+#define LM_SST 36           // row stride of the score exchange (floats)
+typedef short lm_v4s __attribute__((ext_vector_type(4)));
+typedef unsigned lm_u32x4 __attribute__((ext_vector_type(4)));
+
+static inline size_t latent_mfma_lds(int W) {
+  const int Wp = (W + 31) / 32 * 32;
+  return (size_t)LM_KT * (Wp + 8) * 2 + 2 * 16 * LM_SST * 4 + LM_KT * 8;
+}
+
+__global__ __launch_bounds__(256) void latent_attn_mfma_kernel(LatAttnParams p) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  constexpr int NKH = LM_MAXW / 32 / 2;                 // 32-entry score steps of half a row
+  constexpr int NOB = LM_MAXR / 16 / 4;                 // 16-entry output blocks of a wave
+  constexpr int NCH = LM_KT * (LM_MAXW / 8) / 256;      // 16-byte chunks of a tile per thread
+  const int W = p.R + p.Dr, NK = (W + 31) / 32, Ws = NK * 32 + 8;
+  float* sp = lds;                                      // [2 halves][16 heads][LM_SST]
+  long long* rowoff = reinterpret_cast<long long*>(sp + 2 * 16 * LM_SST);   // [LM_KT]
+  bf16_t* tile = reinterpret_cast<bf16_t*>(rowoff + LM_KT);                 // [LM_KT][Ws]
+  const int t = blockIdx.x, split = blockIdx.z;
+  // in a scalar register: matrix instructions ignore the lane mask, so branches
+  // around them must be taken by whole waves
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int n = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y * 16 + n;
+  const bool live = h < p.H;
+  const bf16_t* cache = (const bf16_t*)p.cache;
+
+  int nk = 0, lo = 0, b = 0;
+  if (t < p.cu_q[p.B]) {
+    while (b + 1 < p.B && t >= p.cu_q[b + 1]) ++b;
+    nk = min(p.pos[t] + 1, p.ctx[b]);
+    if (p.window > 0) lo = min(max(0, p.pos[t] + 1 - p.window), nk);
+  }
+  int k0 = lo, k1 = nk;
+  if (p.num_splits > 1) {
+    const int per = ((nk - lo + p.num_splits - 1) / p.num_splits + LM_KT - 1) / LM_KT * LM_KT;
+    k0 = min(nk, lo + split * per);
+    k1 = min(nk, k0 + per);
+  }
+  const int* bt = p.bt + (size_t)b * p.max_blocks;
+  const int cpr = W / 8, nch = LM_KT * cpr;
+  lm_u32x4 pre[NCH];
+  auto plan_rows = [&](int kt) {
+    if (threadIdx.x < LM_KT) {
+      const int key = kt + threadIdx.x;
+      rowoff[threadIdx.x] = key < k1
+          ? (long long)(((size_t)bt[key / p.blk] * p.blk + key % p.blk) * W) : -1ll;
+    }
+  };
+  auto fetch = [&]() {
+#pragma unroll
+    for (int j = 0; j < NCH; ++j) {
+      const int c = threadIdx.x + 256 * j;
+      pre[j] = lm_u32x4{0, 0, 0, 0};
+      if (c < nch) {
+        const int row = c / cpr, cc = c - row * cpr;
+        const long long off = rowoff[row];
+        if (off >= 0) pre[j] = *reinterpret_cast<const lm_u32x4*>(cache + off + cc * 8);
+      }
+    }
+  };
+  if (k0 < k1) plan_rows(k0);
+  // columns W .. 32 NK of the tile stay zero (their query entries are zero too,
+  // but what LDS holds at start may be no number)
+  for (int i = threadIdx.x; i < LM_KT * (NK * 32 - W); i += 256) {
+    const int row = i / (NK * 32 - W), c = W + i - row * (NK * 32 - W);
+    tile[row * Ws + c] = 0;
+  }
+  __syncthreads();
+  if (k0 < k1) fetch();
+
+  // this wave scores keys 16 sub .. + 15 of a tile over half the row
+  const int sub = wave & 1, half = wave >> 1;
+  const int s_lo = half ? (NK + 1) / 2 : 0, s_n = half ? NK / 2 : (NK + 1) / 2;
+  bf16x8 qf[NKH];
+  {
+    const bf16_t* qa = (const bf16_t*)p.qa + (size_t)t * p.qa_st + (size_t)(live ? h : 0) * p.qa_sh;
+    const bf16_t* qr = (const bf16_t*)p.qr + (size_t)t * p.qr_st + (size_t)(live ? h : 0) * p.qr_sh;
+    const int pp = min(max(p.pos[t], 0), p.max_pos - 1);
+    const float* csr = p.cs + (size_t)pp * p.dims;
+#pragma unroll
+    for (int s = 0; s < NKH; ++s) {
+      const int e0 = 32 * (s_lo + s) + 8 * g;           // 8 entries, all latent or all rotary (R % 8 == 0)
+      short8 f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) f[i] = 0;
+      if (live && s < s_n && e0 < W) {
+        if (e0 < p.R) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) f[i] = (short)qa[e0 + i];
+        } else {
+          const int j0 = e0 - p.R;
+#pragma unroll
+          for (int i = 0; i < 8; i += 2) {
+            const int j = j0 + i;
+            const float u = bf2f(qr[j]), v = bf2f(qr[j + 1]);
+            if (j < p.dims) {
+              const float c = csr[j], sn = csr[j + 1];
+              f[i] = (short)f2bf(u * c - v * sn);
+              f[i + 1] = (short)f2bf(v * c + u * sn);
+            } else {
+              f[i] = (short)qr[j];
+              f[i + 1] = (short)qr[j + 1];
+            }
+          }
+        }
+      }
+      qf[s] = *reinterpret_cast<bf16x8*>(&f);
+    }
+  }
+  float m = -INFINITY, l = 0.f;
+  float4v acc[NOB];
+#pragma unroll
+  for (int i = 0; i < NOB; ++i) acc[i] = float4v{0.f, 0.f, 0.f, 0.f};
+
+  for (int kt = k0; kt < k1; kt += LM_KT) {
+    __syncthreads();                                    // the previous tile is consumed
+#pragma unroll
+    for (int j = 0; j < NCH; ++j) {
+      const int c = threadIdx.x + 256 * j;
+      if (c < nch) {
+        const int row = c / cpr, cc = c - row * cpr;
+        *reinterpret_cast<lm_u32x4*>(tile + row * Ws + cc * 8) = pre[j];
+      }
+    }
+    if (kt + LM_KT < k1) plan_rows(kt + LM_KT);
+    __syncthreads();
+    if (kt + LM_KT < k1) fetch();
+    {
+      float4v s0{0.f, 0.f, 0.f, 0.f}, s1 = s0;          // two chains
+      const bf16_t* kr = tile + (16 * sub + n) * Ws + 32 * s_lo + 8 * g;
+#pragma unroll
+      for (int s = 0; s < NKH; ++s)
+        if (s < s_n) {
+          const bf16x8 a = *reinterpret_cast<const bf16x8*>(kr + 32 * s);
+          if (s & 1) s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[s], s1, 0, 0, 0);
+          else s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qf[s], s0, 0, 0, 0);
+        }
+      // lane: head n, keys 16 sub + 4 g .. + 3
+      *reinterpret_cast<float4v*>(sp + (half * 16 + n) * LM_SST + 16 * sub + 4 * g) = s0 + s1;
+    }
+    __syncthreads();
+    // every wave: head n, keys 8 g .. 8 g + 7 of the tile
+    bf16x8 pf;
+    float corr;
+    {
+      float sv[8];
+      float mx = -INFINITY;
+#pragma unroll
+      for (int q4 = 0; q4 < 2; ++q4) {
+        const float4v x = *reinterpret_cast<const float4v*>(sp + n * LM_SST + 8 * g + 4 * q4);
+        const float4v y = *reinterpret_cast<const float4v*>(sp + (16 + n) * LM_SST + 8 * g + 4 * q4);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int k = 4 * q4 + i;
+          sv[k] = kt + 8 * g + k < k1 ? (x[i] + y[i]) * p.scale : -INFINITY;
+          mx = fmaxf(mx, sv[k]);
+        }
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m, mx);                    // finite: the tile holds at least one key
+      corr = m == -INFINITY ? 0.f : expf(m - mn);
+      float ls = 0.f;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) {
+        const float e = sv[k] == -INFINITY ? 0.f : expf(sv[k] - mn);
+        ls += e;
+        pf[k] = (__bf16)e;
+      }
+      ls += __shfl_xor(ls, 16, 64);
+      ls += __shfl_xor(ls, 32, 64);
+      l = l * corr + ls;
+      m = mn;
+    }
+    // O^T[entry, head] += C^T[entry, key] P^T[key, head]; C^T by transposed reads:
+    // a group of 16 lanes names 4 rows x 16 entries and gets its entry of the 4 rows
+#pragma unroll
+    for (int i = 0; i < NOB; ++i) {
+      const int c0 = 16 * (4 * i + wave);
+      if (c0 < p.R) {
+        const bf16_t* src = tile + (8 * g + (n >> 2)) * Ws + c0 + 4 * (n & 3);
+        const lm_v4s a0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) lm_v4s*)(src));
+        const lm_v4s a1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (__attribute__((address_space(3))) lm_v4s*)(src + 4 * Ws));
+        short8 a8;
+        a8[0] = a0[0]; a8[1] = a0[1]; a8[2] = a0[2]; a8[3] = a0[3];
+        a8[4] = a1[0]; a8[5] = a1[1]; a8[6] = a1[2]; a8[7] = a1[3];
+        acc[i] *= corr;
+        acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<bf16x8*>(&a8), pf, acc[i],
+                                                         0, 0, 0);
+      }
+    }
+  }
+  if (!live) return;
+  if (p.num_splits > 1) {                               // partial of this key split
+    float* wsr = p.ws + (((size_t)split * p.T + t) * p.H + h) * (p.R + 2);
+    if (wave == 0 && g == 0) { wsr[0] = m; wsr[1] = l; }
+#pragma unroll
+    for (int i = 0; i < NOB; ++i) {
+      const int r = 16 * (4 * i + wave) + 4 * g;
+      if (r < p.R) {
+#pragma unroll
+        for (int k = 0; k < 4; ++k) wsr[2 + r + k] = acc[i][k];
+      }
+    }
+    return;
+  }
+  float M = m, den = l, f = 1.f;
+  if (p.sink) {
+    const float sk = p.sink[h];
+    M = fmaxf(m, sk);
+    f = m == -INFINITY ? 0.f : expf(m - M);
+    den = l * f + expf(sk - M);
+  }
+  const float inv = den > 0.f ? f / den : 0.f;
+  bf16_t* out = (bf16_t*)p.out + ((size_t)h * p.T + t) * p.R;
+#pragma unroll
+  for (int i = 0; i < NOB; ++i) {
+    const int r = 16 * (4 * i + wave) + 4 * g;
+    if (r < p.R) {
+      uint2 w;
+      w.x = pack_bf16x2(acc[i][0] * inv, acc[i][1] * inv);
+      w.y = pack_bf16x2(acc[i][2] * inv, acc[i][3] * inv);
+      *reinterpret_cast<uint2*>(out + r) = w;
+    }
+  }
+}
+
 // out[h, t] from the key splits' (m, l, acc) partials, merged in split order.
 // One wave per (token, head): lane s first turns split s's (m, l) into its
 // weight e^{m_s - M} (M = the largest m, or the sink), then the partial
@@ -491,12 +758,20 @@ extern "C" int loqa_latent_inputs(const void* z, int dt, long ldz, const void* n
   if (T <= 0) return 0;
   if (R <= 0 || Dr < 0 || dims < 0 || dims > Dr || Rq < 0 || (Rq && (!dq || !qw || !cq)))
     return (int)hipErrorInvalidValue;
+  const size_t run = dt == 0 ? 8 : 16;
+  auto runs = [&](const void* a, long lda, const void* w, const void* b, long ldb, int n) {
+    return n % 4 == 0 && lda % 4 == 0 && ldb % 4 == 0 && (size_t)a % run == 0 &&
+           (size_t)b % run == 0 && (size_t)w % 16 == 0;
+  };
   const LatInParams p{z, ldz, (const float*)nw, eps, (const int*)pos, (const float*)cs, max_pos,
                       cache, (long)blk * nblocks, (const int*)slots, R, Dr, dims, dq, lddq,
-                      (const float*)qw, Rq, cq};
+                      (const float*)qw, Rq, cq, runs(z, ldz, nw, cache, R + Dr, R),
+                      Rq ? runs(dq, lddq, qw, cq, Rq, Rq) : 0};
+  // a decode step has few tokens: a token's row spreads over workgroups
+  const dim3 grid(T, T >= 256 ? 1 : (s_n > 0 ? 2 + ceil_div(s_n, 1024) : (Rq ? 2 : 1)));
   const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
-  if (dt == 0) hipLaunchKernelGGL(latent_inputs_kernel<bf16_t>, dim3(T), dim3(128), 0, st, p, side);
-  else hipLaunchKernelGGL(latent_inputs_kernel<float>, dim3(T), dim3(128), 0, st, p, side);
+  if (dt == 0) hipLaunchKernelGGL(latent_inputs_kernel<bf16_t>, grid, dim3(128), 0, st, p, side);
+  else hipLaunchKernelGGL(latent_inputs_kernel<float>, grid, dim3(128), 0, st, p, side);
   return (int)hipGetLastError();
 }
 
@@ -505,7 +780,7 @@ extern "C" int loqa_latent_attention(
     const void* cache, int blk, int nblocks, const void* cu_q, const void* ctx, const void* bt,
     int max_blocks, const void* pos, const void* cs, int max_pos, const void* sink, float scale,
     int B, int H, int T, int R, int Dr, int dims, void* out, int num_splits, void* ws, int window,
-    hipStream_t st) {
+    int mfma, hipStream_t st) {
   if (T <= 0 || H <= 0) return 0;
   if (R > 64 * LAT_MAXR || R <= 0 || B <= 0) return (int)hipErrorInvalidValue;
   if (num_splits > 1 && !ws) return (int)hipErrorInvalidValue;
@@ -519,6 +794,19 @@ extern "C" int loqa_latent_attention(
   p.num_splits = num_splits < 1 ? 1 : num_splits; p.ws = (float*)ws;
   p.window = window;
   const int W = R + Dr, Ws = W | 1;
+  if (mfma) {
+    // 16-byte rows and queries, whole output blocks
+    if (dt != 0 || R % 16 || W % 8 || R > LM_MAXR || W > LM_MAXW || dims % 2 || dims > Dr ||
+        ((size_t)cache & 15))
+      return (int)hipErrorInvalidValue;
+    hipLaunchKernelGGL(latent_attn_mfma_kernel, dim3(T, (H + 15) / 16, p.num_splits), dim3(256),
+                       latent_mfma_lds(W), st, p);
+    int rc = (int)hipGetLastError();
+    if (rc || p.num_splits == 1) return rc;
+    hipLaunchKernelGGL(latent_combine_kernel<bf16_t>, dim3(T, H), dim3(64), 0, st, (const float*)ws,
+                       (const float*)sink, (bf16_t*)out, T, H, R, p.num_splits);
+    return (int)hipGetLastError();
+  }
   if (W % 2 == 0 && R % 2 == 0 && R <= 128 * LAT_MAXP) {
     const size_t esz = dt == 0 ? 2 : 4;
     int KT2 = 32;

@@ -123,7 +123,10 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
     __syncthreads();
     if (kt + LP_TILE < kend) fetch(kt + LP_TILE);
     // a wave whose rows see nothing of this tile only keeps the barriers
-    if (kt > wpos_hi || (p.window > 0 && kt + LP_TILE <= wpos_lo - p.window + 1)) continue;
+    // (a scalar branch: matrix instructions ignore the lane mask)
+    if (__builtin_amdgcn_readfirstlane(
+            kt > wpos_hi || (p.window > 0 && kt + LP_TILE <= wpos_lo - p.window + 1)))
+      continue;
 
     float16v st[2];
 #pragma unroll

@@ -15,7 +15,8 @@
 // mixed batches are one launch. window = 0 with cap = 0 is plain causal
 // attention.
 //
-// qk_prep_append_kernel (one workgroup per token, a wave per head): the first
+// qk_prep_append_kernel (one workgroup per token, several in steps of few tokens,
+// a wave per head): the first
 // `dims` entries of each q and k head rotate pairwise (2i with 2i + 1) by the
 // position's angles, each head is divided by its root mean square (no weight),
 // q is multiplied by the position's temperature; q out, k into its page, and
@@ -162,7 +163,7 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(
   const float* csr = dims ? cs + (size_t)min(max(p, 0), max_pos - 1) * dims : nullptr;
   const float temp = 1.f + coef * logf((float)((p + 1) / every) + 1.f);
   constexpr int NP = 4;                           // pairs per lane (D <= 512)
-  for (int job = wave; job < H + G; job += 4) {
+  for (int job = blockIdx.y * 4 + wave; job < H + G; job += 4 * gridDim.y) {
     const bool isq = job < H;
     const T* src = ur + (size_t)job * D;          // q heads, then k heads
     float a[NP], b[NP];
@@ -228,10 +229,11 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(
     T* vr = vc + (size_t)slot * G * Dv;
     if (vf) {                                      // (1 - lam) v + lam v_first
       const T* fr = vf + (size_t)t * vf_ld;
-      for (int c = threadIdx.x; c < G * Dv; c += blockDim.x)
+      for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < G * Dv; c += gridDim.y * blockDim.x)
         Act<T>::st(vr + c, (1.f - lam) * Act<T>::ld(ur + v_off + c) + lam * Act<T>::ld(fr + c));
     } else {
-      for (int c = threadIdx.x; c < G * Dv; c += blockDim.x) vr[c] = ur[v_off + c];
+      for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < G * Dv; c += gridDim.y * blockDim.x)
+        vr[c] = ur[v_off + c];
     }
   }
   side_relu2<T>(side, t);
@@ -800,8 +802,10 @@ extern "C" int loqa_qk_prep_append(const void* u, int dt, long ldu, int H, int G
     return (int)hipErrorInvalidValue;
   const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
   const long rows = (long)blk * nblocks;
+  // a decode step has few tokens: a token's heads and columns spread over workgroups
+  const int gy = T >= 256 ? 1 : ceil_div(H + G, 4);
 #define GO(TT)                                                                                  \
-  hipLaunchKernelGGL(qk_prep_append_kernel<TT>, dim3(T), dim3(256), 0, st, (const TT*)u, ldu, H, \
+  hipLaunchKernelGGL(qk_prep_append_kernel<TT>, dim3(T, gy), dim3(256), 0, st, (const TT*)u, ldu, H, \
                      G, D, Dv, v_off, (const float*)cs, max_pos, dims, eps, coef, every,        \
                      (const int*)pos, (TT*)kc, (TT*)vc, rows, (const int*)kvslots, (TT*)q,      \
                      (const float*)qn, (const float*)kn, norm, (const TT*)vf, vf_ld, lam, side)

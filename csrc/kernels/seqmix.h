@@ -66,8 +66,9 @@ template <typename T, int N> __device__ __forceinline__ void st_run(T* p, const 
 // reads the same input as the mixer, so its up projection is a column slice of
 // the same matrix product. src [T, src_ld] (the slice's first column) ->
 // dst[t, 0 .. n) = relu(src)^2, and zeros in the columns zero_lo .. 0 (negative
-// offsets: padding before the slice) and n .. zero_hi. One workgroup per token
-// calls it with its row; vec: rows and bases are aligned for runs of four.
+// offsets: padding before the slice) and n .. zero_hi. The workgroups of a token
+// (gridDim.y of them) share its row; vec: rows and bases are aligned for runs of
+// four.
 struct SideCols {
   const void* src; long src_ld;
   void* dst; long dst_ld;
@@ -78,8 +79,10 @@ __device__ __forceinline__ void side_relu2(const SideCols& s, size_t t) {
   if (!s.dst) return;
   const T* a = (const T*)s.src + t * s.src_ld;
   T* o = (T*)s.dst + t * s.dst_ld;
+  const int me = blockIdx.y * blockDim.x + threadIdx.x, all = gridDim.y * blockDim.x;
   if (s.vec) {
-    for (int c = 4 * threadIdx.x; c < s.n; c += 4 * blockDim.x) {
+#pragma unroll 2
+    for (int c = 4 * me; c < s.n; c += 4 * all) {
       float f[4];
       ld_run<T, 4>(a + c, f);
 #pragma unroll
@@ -87,13 +90,13 @@ __device__ __forceinline__ void side_relu2(const SideCols& s, size_t t) {
       st_run<T, 4>(o + c, f);
     }
   } else {
-    for (int c = threadIdx.x; c < s.n; c += blockDim.x) {
+    for (int c = me; c < s.n; c += all) {
       const float f = fmaxf(Act<T>::ld(a + c), 0.f);
       Act<T>::st(o + c, f * f);
     }
   }
-  for (int c = s.zero_lo + (int)threadIdx.x; c < 0; c += blockDim.x) Act<T>::st(o + c, 0.f);
-  for (int c = s.n + (int)threadIdx.x; c < s.zero_hi; c += blockDim.x) Act<T>::st(o + c, 0.f);
+  for (int c = s.zero_lo + me; c < 0; c += all) Act<T>::st(o + c, 0.f);
+  for (int c = s.n + me; c < s.zero_hi; c += all) Act<T>::st(o + c, 0.f);
 }
 
 static inline int ceil_div(long a, long b) { return (int)((a + b - 1) / b); }

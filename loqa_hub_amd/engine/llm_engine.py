@@ -269,19 +269,31 @@ class LLMEngine:
         return max_q, max_ctx, host
 
     def _to_device(self, host: dict, dst: dict | None = None) -> dict:
-        out = {}
-        for k, a in host.items():
-            if not isinstance(a, np.ndarray):      # host-side scalars ride along
-                out[k] = a
-                continue
-            t = torch.from_numpy(a)
-            if self.is_gpu:
-                t = t.pin_memory()
-            if dst is not None:
-                dst[k].copy_(t, non_blocking=True)
-                out[k] = dst[k]
-            else:
-                out[k] = t.to(self.device, non_blocking=True)
+        out = {k: a for k, a in host.items() if not isinstance(a, np.ndarray)}   # host-side scalars
+        arrays = {k: a for k, a in host.items() if isinstance(a, np.ndarray)}
+        if dst is not None or not self.is_gpu:
+            for k, a in arrays.items():
+                t = torch.from_numpy(a)
+                if dst is None:
+                    out[k] = t.to(self.device)
+                else:
+                    dst[k].copy_(t.pin_memory() if self.is_gpu else t, non_blocking=True)
+                    out[k] = dst[k]
+            return out
+        # one pinned buffer and one copy for the step; every array starts on a
+        # 16-byte boundary of it
+        offs, n = {}, 0
+        for k, a in arrays.items():
+            offs[k] = n
+            n += -(-a.nbytes // 16) * 16
+        stage = torch.empty(max(n, 16), dtype=torch.uint8, pin_memory=True)
+        flat = stage.numpy()
+        for k, a in arrays.items():
+            flat[offs[k]:offs[k] + a.nbytes] = a.reshape(-1).view(np.uint8)
+        buf = stage.to(self.device, non_blocking=True)
+        for k, a in arrays.items():
+            t = buf[offs[k]:offs[k] + a.nbytes].view(torch.from_numpy(a[:0].reshape(-1)).dtype)
+            out[k] = t.view(a.shape)
         return out
 
     # ------------------------------------------------------------ forward

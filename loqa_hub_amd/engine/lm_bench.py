@@ -6,10 +6,13 @@ For each size a Pipizen stack (latent attention / lightning mixers, dense and
 mixture-of-experts feed-forwards), a Sodonex stack (chunked sigmoid attention
 with token shift and short convolutions, squared-relu experts) and a Movinex
 stack (a Mamba-2 layer, full and sliding-window softmax attention, GeGLU and
-sigmoid-routed experts) and a Vilulix stack (parallel layers: a matrix memory,
+sigmoid-routed experts), a Vilulix stack (parallel layers: a matrix memory,
 latent attention with a query latent, sliding-window attention with a sink
-beside a gated delta rule, dense SwiGLU) run beside a Llama stack of the same
-width, depth, head count and feed-forward width - the framework's plain decoder. Measured per family:
+beside a gated delta rule, dense SwiGLU) and a Gopopel stack (parallel layers on
+one norm: sliding-window attention with a distance bias, sliding-window latent
+attention, squared-relu feed-forwards) run beside a Llama stack of the same
+width, depth, head count and feed-forward width - the framework's plain decoder.
+Measured per family:
 
 * prefill: one prompt of ``P`` tokens through ``LLMEngine.step_logits``;
 * decode: ``B`` sequences at context ``P`` advancing one token per step
@@ -27,7 +30,7 @@ import numpy as np
 import torch
 
 from ..models.configs import (ChunkAttnConfig, DeltaRuleConfig, FeedForwardConfig,
-                              HybridLayerConfig, LatentAttnConfig, LightningConfig, LlamaConfig,
+                              GopopelConfig, HybridLayerConfig, LatentAttnConfig, LightningConfig, LlamaConfig,
                               LoopConfig, Mamba2Config, MatrixMemoryConfig, MovinexConfig,
                               ParallelMixerConfig, PipizenConfig, RotaryConfig, SodonexConfig,
                               SoftmaxAttnConfig, VilulixConfig)
@@ -113,6 +116,22 @@ def vilulix_stack(name: str, vocab: int = 32000, window: int = 1024) -> VilulixC
     return VilulixConfig(f"vilulix-{name}", vocab, d, 1e-6, 30.0, tuple(layers))
 
 
+def gopopel_stack(name: str, vocab: int = 32000, window: int = 1024) -> GopopelConfig:
+    """Four parallel layers with an ungated squared-relu feed-forward each,
+    alternating sliding-window attention (4 query heads per key/value head,
+    distance bias, sink, value mixing) and sliding-window latent attention with
+    the latent sizes of the Vilulix stack."""
+    d, n, H, D, Dr, R, ff, _, _, _ = SIZES[name]
+    att = SoftmaxAttnConfig(H, max(1, H // 4), D, D, D ** -0.5, window=window, qk_norm="head_weight",
+                            sink=True, alibi=True, v_mix=True)
+    lat = LatentAttnConfig(H, D, Dr, D, R, (D + Dr) ** -0.5, RotaryConfig(Dr, 10000.0),
+                           q_rank=3 * R, gate=True, window=window)
+    mlp = FeedForwardConfig("dense", ff, act="relu2")
+    return GopopelConfig(f"gopopel-{name}", vocab, d, 1e-6, 1.0, tuple(
+        HybridLayerConfig("latent_attention", lat, mlp) if i % 2 else
+        HybridLayerConfig("attention", att, mlp) for i in range(n)))
+
+
 def llama_stack(name: str, vocab: int = 32000) -> LlamaConfig:
     d, n, H, D, _, _, ff, _, _, _ = SIZES[name]
     return LlamaConfig(f"llama-{name}-stack", d, n, H, max(1, H // 4), D, ff, vocab,
@@ -181,7 +200,7 @@ def run(args) -> int:
     sizes = [s for s in args.lm_sizes.split(",") if s]
     for name in sizes:
         fams = {"pipizen": pipizen_stack, "sodonex": sodonex_stack, "movinex": movinex_stack,
-                "vilulix": vilulix_stack, "llama": llama_stack}
+                "vilulix": vilulix_stack, "gopopel": gopopel_stack, "llama": llama_stack}
         for fam in [f for f in args.lm_families.split(",") if f]:
             cfg = fams[fam](name)
             if dev.type == "cpu":      # plumbing run: tiny stacks

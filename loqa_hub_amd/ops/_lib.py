@@ -214,7 +214,7 @@ _SEQMIX_SIGS = {
     "loqa_latent_inputs": [_vp, _i, _l, _vp, _f, _vp, _vp, _i, _vp, _i, _i, _vp, _i, _i, _i, _i,
                            _vp, _l, _vp, _i, _vp, *_SIDE, _vp],
     "loqa_latent_attention": [_vp, _l, _l, _vp, _l, _l, _i, _vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp,
-                              _i, _vp, _f, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _i, _vp],
+                              _i, _vp, _f, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _i, _i, _vp],
     "loqa_latent_gather": [_vp, _i, _vp, _i, _vp, _vp, _i, _i, _i, _i, _vp, _vp, _vp],
     "loqa_latent_kfill": [_vp, _vp, _i, _i, _i, _i, _i, _vp],
     "loqa_rope_pairs": [_vp, _l, _l, _i, _i, _i, _i, _vp, _vp, _i, _vp],

@@ -194,11 +194,16 @@ def latent_inputs(z: torch.Tensor, norm_w: torch.Tensor, eps: float, positions: 
     return cq
 
 
+def latent_mfma_sizes(R: int, Dr: int) -> bool:
+    """Latent sizes the matrix-core form of the folded attention covers."""
+    return R % 16 == 0 and 0 < R <= 512 and (R + Dr) % 8 == 0 and R + Dr <= 640
+
+
 def latent_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, cu_q: torch.Tensor,
                      ctx_lens: torch.Tensor, block_tables: torch.Tensor, positions: torch.Tensor,
                      cos_sin: torch.Tensor, sink: torch.Tensor | None, scale: float, R: int,
                      dims: int, max_ctx: int = 0, out: torch.Tensor | None = None,
-                     window: int = 0) -> torch.Tensor:
+                     window: int = 0, matrix_cores: bool | None = None) -> torch.Tensor:
     """Causal attention over the paged latent cache, all heads sharing each
     cached row: score = (qa . c + rot(qr) . k_rot) * scale; softmax with
     ``sink`` [H] (f32, optional) in the denominator; out = sum_j p_j c_j. With
@@ -222,17 +227,18 @@ def latent_attention(qa: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, cu
         assert sink.numel() == H
     B = ctx_lens.numel()
     assert cu_q.numel() == B + 1 and block_tables.shape[0] == B and positions.numel() >= T
+    mfma = qa.dtype == torch.bfloat16 and latent_mfma_sizes(R, Dr) and matrix_cores is not False
     # few query rows over a long context: split the keys over workgroups
-    hg = (H + 3) // 4
     keys = min(int(max_ctx), window) if window > 0 else int(max_ctx)
-    ns = 1 if T * hg >= 512 else max(1, min(32, -(-keys // 128), 1024 // max(1, T * hg)))
+    wgs = T * ((H + 15) // 16 if mfma else (H + 3) // 4)
+    ns = 1 if wgs >= 512 else max(1, min(32, -(-keys // (64 if mfma else 128)), 1024 // max(1, wgs)))
     ws = torch.empty(ns * T * H * (R + 2), dtype=torch.float32, device=qa.device) if ns > 1 else None
     if T:
         check(kernels().loqa_latent_attention(
             ptr(qa), qa.stride(1), qa.stride(0), ptr(qr), qr.stride(0), qr.stride(1), _dt(qa),
             ptr(cache), cache.shape[1], cache.shape[0], ptr(cu_q), ptr(ctx_lens), ptr(block_tables),
             block_tables.shape[1], ptr(positions), ptr(cos_sin), cos_sin.shape[0], ptr(sink),
-            float(scale), B, H, T, R, Dr, dims, ptr(out), ns, ptr(ws), int(window),
+            float(scale), B, H, T, R, Dr, dims, ptr(out), ns, ptr(ws), int(window), int(mfma),
             stream_ptr(qa)),
             "latent_attention")
     return out

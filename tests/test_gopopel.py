@@ -809,6 +809,49 @@ def test_windowed_latent_prompt_pass(H, D, Dr, Dv, R, window):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("H,R,Dr,dims,window,sink", [(16, 512, 64, 64, 0, True), (4, 96, 32, 32, 70, False),
+                                                     (17, 64, 8, 4, 33, True), (32, 48, 24, 24, 1, False),
+                                                     (3, 16, 0, 0, 129, True), (1, 512, 128, 128, 64, False)])
+def test_folded_latent_attention_matrix_cores(H, R, Dr, dims, window, sink):
+    """The folded form on the matrix cores against float64 and against the
+    vector form: full and partial head groups, one and many key splits, padding
+    rows, lone tokens of short and long contexts beside a portion."""
+    g = torch.Generator().manual_seed(7)
+    lens, feeds, scale = [700, 1, 333, 90, 32], [1, 1, 3, 17, 1], 0.3 / R ** 0.5
+    rows = [torch.randn(n, R + Dr, generator=g).to(torch.bfloat16).float() for n in lens]
+    (pages,), bt = _paged([rows], lens, 16, "cuda", 3)
+    cu, pos = _meta(feeds, [n - f for n, f in zip(lens, feeds)], "cuda")
+    T = sum(feeds)
+    pos = torch.cat([pos, torch.zeros(2, dtype=torch.int32, device="cuda")])
+    qa = (torch.randn(H, T + 2, R, generator=g) * 3).to(torch.bfloat16)
+    qr = torch.randn(T + 2, H, Dr, generator=g).to(torch.bfloat16)
+    cs = seqmix.rope_table_pairs(dims, 700, 100.0, None, "cuda")
+    sk = torch.randn(H, generator=g) if sink else None
+    args = (pages.to(torch.bfloat16), cu, torch.tensor(lens, dtype=torch.int32, device="cuda"), bt, pos,
+            cs, None if sk is None else sk.cuda(), scale, R, dims)
+    want = torch.zeros(H, T, R, dtype=F64)
+    t0 = 0
+    for b, (n, f) in enumerate(zip(lens, feeds)):
+        c = rows[b].double()
+        for t in range(t0, t0 + f):
+            p = n - f + t - t0
+            lo = max(0, p - window + 1) if window else 0
+            q = torch.cat([qa[:, t].double(), O.rotate_pairs(qr[t].double()[None], dims, 100.0,
+                                                             torch.tensor([p]))[0]], -1)
+            s = q @ c[lo:p + 1].T * scale
+            e = torch.exp(s - s.max())
+            den = e.sum(-1) + (torch.exp(sk.double() - s.max()) if sink else 0)
+            want[:, t] = (e / den[:, None]) @ c[lo:p + 1, :R]
+        t0 += f
+    top = float(want.abs().max())
+    for mc in (True, False):
+        for max_ctx in (700, 64):          # many key splits, one
+            got = seqmix.latent_attention(qa.cuda(), qr.cuda(), *args, max_ctx=max_ctx, window=window,
+                                          matrix_cores=mc)
+            assert (got[:, :T].cpu().double() - want).abs().max() < 0.02 * top, (mc, max_ctx)
+
+
+@pytest.mark.gpu
 def test_serving_sizes_bf16():
     """A model with matrix-core head sizes in bfloat16: whole prompt, portions
     and decoding agree with the oracle within 16-bit rounding, and with each
