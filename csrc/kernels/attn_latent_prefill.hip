@@ -142,19 +142,34 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
     bf16x8 pf[2][2];
     {
       float mx = -INFINITY;
+      // a tile that every row of this wave sees whole needs no per-score tests
+      const bool whole = kt + LP_TILE - 1 <= wpos_lo && kt + LP_TILE <= kend &&
+                         (p.window <= 0 || wpos_hi - kt < p.window);
+      if (__builtin_amdgcn_readfirstlane(whole)) {
 #pragma unroll
-      for (int t = 0; t < 2; ++t)
+        for (int t = 0; t < 2; ++t)
 #pragma unroll
-        for (int j = 0; j < 16; ++j) {
-          const int key = kt + 32 * t + (j & 3) + 8 * (j >> 2) + 4 * h;
-          float sv = st[t][j] * p.scale_log2;
-          if (key >= kend || key > qpos || (p.window > 0 && qpos - key >= p.window)) sv = -INFINITY;
-          st[t][j] = sv;
-          mx = fmaxf(mx, sv);
-        }
+          for (int j = 0; j < 16; ++j) {
+            st[t][j] *= p.scale_log2;
+            mx = fmaxf(mx, st[t][j]);
+          }
+      } else {
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int j = 0; j < 16; ++j) {
+            const int key = kt + 32 * t + (j & 3) + 8 * (j >> 2) + 4 * h;
+            float sv = st[t][j] * p.scale_log2;
+            if (key >= kend || key > qpos || (p.window > 0 && qpos - key >= p.window)) sv = -INFINITY;
+            st[t][j] = sv;
+            mx = fmaxf(mx, sv);
+          }
+      }
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
       const float m_new = fmaxf(m_run, mx);
-      const float alpha = exp2f(m_run - m_new);
+      // the hardware's exp2: the arguments are <= 0, and what falls below the
+      // normal range may flush to zero
+      const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
       float ls = 0.f;
 #pragma unroll
       for (int t = 0; t < 2; ++t)
@@ -162,7 +177,7 @@ __global__ __launch_bounds__(LP_THREADS) void latent_prefill_kernel(LatPrefillPa
         for (int s2 = 0; s2 < 2; ++s2)
 #pragma unroll
           for (int j = 0; j < 8; ++j) {
-            const float e = exp2f(st[t][8 * s2 + j] - m_new);
+            const float e = __builtin_amdgcn_exp2f(st[t][8 * s2 + j] - m_new);
             ls += e;
             pf[t][s2][j] = (__bf16)e;
           }

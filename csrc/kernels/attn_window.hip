@@ -129,111 +129,190 @@ __device__ __forceinline__ int wa_seq_of_row(const int* __restrict__ cu_q, int B
 // ------------------------------------------------------------------ q / k rows
 enum { QKN_HEAD = 0, QKN_WHOLE = 1, QKN_HEAD_W = 2 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void qk_prep_append_kernel(
-    const T* __restrict__ u, long ldu, int H, int G, int D, int Dv, int v_off,
-    const float* __restrict__ cs, int max_pos, int dims, float eps, float coef, int every,
-    const int* __restrict__ pos, T* __restrict__ kc, T* __restrict__ vc, long cache_rows,
-    const int* __restrict__ kvslots, T* __restrict__ q, const float* __restrict__ qn,
-    const float* __restrict__ kn, int norm, const T* __restrict__ vf, long vf_ld, float lam,
-    SideCols side) {
+// NP: pairs of neighbouring entries per lane (D <= 128 NP). PAIR: heads are even
+// and rows aligned, so a pair is one access (and the value rows go in runs of
+// four); else entry by entry.
+template <typename T> struct Two;
+template <> struct Two<bf16_t> {
+  static __device__ __forceinline__ void ld(const bf16_t* p, float& a, float& b) {
+    const uint32_t w = *reinterpret_cast<const uint32_t*>(p);
+    a = __uint_as_float(w << 16);
+    b = __uint_as_float(w & 0xffff0000u);
+  }
+  static __device__ __forceinline__ void st(bf16_t* p, float a, float b) {
+    *reinterpret_cast<uint32_t*>(p) = pack_bf16x2(a, b);
+  }
+};
+template <> struct Two<float> {
+  static __device__ __forceinline__ void ld(const float* p, float& a, float& b) {
+    const float2 w = *reinterpret_cast<const float2*>(p);
+    a = w.x;
+    b = w.y;
+  }
+  static __device__ __forceinline__ void st(float* p, float a, float b) {
+    *reinterpret_cast<float2*>(p) = make_float2(a, b);
+  }
+};
+template <typename T, bool PAIR>
+__device__ __forceinline__ void ld_two(const T* p, bool two, float& a, float& b) {
+  if constexpr (PAIR) {
+    Two<T>::ld(p, a, b);
+  } else {
+    a = Act<T>::ld(p);
+    b = two ? Act<T>::ld(p + 1) : 0.f;
+  }
+}
+template <typename T, bool PAIR>
+__device__ __forceinline__ void st_two(T* p, bool two, float a, float b) {
+  if constexpr (PAIR) {
+    Two<T>::st(p, a, b);
+  } else {
+    Act<T>::st(p, a);
+    if (two) Act<T>::st(p + 1, b);
+  }
+}
+
+template <typename T> struct QkPrepParams {
+  const T* u; long ldu; int H, G, D, Dv, v_off;
+  const float* cs; int max_pos, dims; float eps, coef; int every;
+  const int* pos; T* kc; T* vc; long cache_rows; const int* kvslots; T* q;
+  const float* qn; const float* kn; int norm;
+  const T* vf; long vf_ld; float lam;      // values blended with another layer's, or null
+  int vruns;                               // value rows can be accessed in runs of four
+};
+
+template <typename T, int NP, bool PAIR>
+__global__ __launch_bounds__(256) void qk_prep_append_kernel(QkPrepParams<T> p, SideCols side) {
   __shared__ float wsum[2][4];
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int p = pos[t];
-  const long slot = kvslots[t];
-  const bool store = slot >= 0 && slot < cache_rows;
-  const T* ur = u + (size_t)t * ldu;
+  const int H = p.H, G = p.G, D = p.D, Dv = p.Dv;
+  const int pos = p.pos[t];
+  const long slot = p.kvslots[t];
+  const bool store = slot >= 0 && slot < p.cache_rows;
+  const T* ur = p.u + (size_t)t * p.ldu;
   // norm: QKN_HEAD divides each head by its root mean square after the rotation;
   // QKN_WHOLE is an RMS norm over the whole q and the whole k projection and
   // QKN_HEAD_W one per head with weights shared by the heads, both before it
   float invq = 1.f, invk = 1.f;
-  if (norm == QKN_WHOLE) {
+  if (p.norm == QKN_WHOLE) {
     float sq = 0.f, sk = 0.f;
-    for (int c = threadIdx.x; c < (H + G) * D; c += blockDim.x) {
-      const float v = Act<T>::ld(ur + c);
-      if (c < H * D) sq += v * v; else sk += v * v;
+    if constexpr (PAIR) {
+      for (int c = 2 * threadIdx.x; c < (H + G) * D; c += 2 * blockDim.x) {
+        float a, b;
+        Two<T>::ld(ur + c, a, b);
+        if (c < H * D) sq += a * a + b * b; else sk += a * a + b * b;
+      }
+    } else {
+      for (int c = threadIdx.x; c < (H + G) * D; c += blockDim.x) {
+        const float v = Act<T>::ld(ur + c);
+        if (c < H * D) sq += v * v; else sk += v * v;
+      }
     }
-    sq = wave_sum(sq);
-    sk = wave_sum(sk);
+    sq = wa_group_sum(sq, 64);
+    sk = wa_group_sum(sk, 64);
     if (lane == 0) { wsum[0][wave] = sq; wsum[1][wave] = sk; }
     __syncthreads();
-    invq = 1.f / sqrtf((wsum[0][0] + wsum[0][1] + wsum[0][2] + wsum[0][3]) / (float)(H * D) + eps);
-    invk = 1.f / sqrtf((wsum[1][0] + wsum[1][1] + wsum[1][2] + wsum[1][3]) / (float)(G * D) + eps);
+    invq = 1.f / sqrtf((wsum[0][0] + wsum[0][1] + wsum[0][2] + wsum[0][3]) / (float)(H * D) + p.eps);
+    invk = 1.f / sqrtf((wsum[1][0] + wsum[1][1] + wsum[1][2] + wsum[1][3]) / (float)(G * D) + p.eps);
   }
-  const float* csr = dims ? cs + (size_t)min(max(p, 0), max_pos - 1) * dims : nullptr;
-  const float temp = 1.f + coef * logf((float)((p + 1) / every) + 1.f);
-  constexpr int NP = 4;                           // pairs per lane (D <= 512)
+  const float* csr = p.dims ? p.cs + (size_t)min(max(pos, 0), p.max_pos - 1) * p.dims : nullptr;
+  const float temp = p.coef == 0.f ? 1.f : 1.f + p.coef * logf((float)((pos + 1) / p.every) + 1.f);
   for (int job = blockIdx.y * 4 + wave; job < H + G; job += 4 * gridDim.y) {
     const bool isq = job < H;
     const T* src = ur + (size_t)job * D;          // q heads, then k heads
     float a[NP], b[NP];
-    float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < NP; ++i) {
       const int e = 2 * (lane + 64 * i);
       a[i] = b[i] = 0.f;
-      if (e < D) {
-        const bool two = e + 1 < D;
-        a[i] = Act<T>::ld(src + e);
-        if (two) b[i] = Act<T>::ld(src + e + 1);
-        if (!isq && v_off < 0 && store) {         // the values are the keys as projected
-          T* vr = vc + (size_t)slot * G * Dv + (size_t)(job - H) * Dv + e;
-          Act<T>::st(vr, a[i]);
-          if (two) Act<T>::st(vr + 1, b[i]);
-        }
-        ss += a[i] * a[i] + b[i] * b[i];
-      }
+      if (e < D) ld_two<T, PAIR>(src + e, e + 1 < D, a[i], b[i]);
     }
-    float inv = 1.f;
-    if (norm == QKN_HEAD_W) inv = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
-    ss = 0.f;
+    if (!isq && p.v_off < 0 && store) {           // the values are the keys as projected
 #pragma unroll
-    for (int i = 0; i < NP; ++i) {
-      const int e = 2 * (lane + 64 * i);
-      if (e < D) {
-        if (norm == QKN_WHOLE) {
-          const float* wn = isq ? qn + (size_t)job * D + e : kn + (size_t)(job - H) * D + e;
-          const float iv = isq ? invq : invk;
-          a[i] *= iv * wn[0];
-          if (e + 1 < D) b[i] *= iv * wn[1];
-        } else if (norm == QKN_HEAD_W) {
-          const float* wn = (isq ? qn : kn) + e;
-          a[i] *= inv * wn[0];
-          if (e + 1 < D) b[i] *= inv * wn[1];
-        }
-        if (e < dims) {
-          const float c = csr[e], s = csr[e + 1];
-          const float x = a[i] * c - b[i] * s, y = b[i] * c + a[i] * s;
-          a[i] = x;
-          b[i] = y;
-        }
-        ss += a[i] * a[i] + b[i] * b[i];
+      for (int i = 0; i < NP; ++i) {
+        const int e = 2 * (lane + 64 * i);
+        if (e < D)
+          st_two<T, PAIR>(p.vc + (size_t)slot * G * Dv + (size_t)(job - H) * Dv + e, e + 1 < D, a[i],
+                          b[i]);
       }
     }
-    inv = norm == QKN_HEAD ? 1.f / sqrtf(wave_sum(ss) / (float)D + eps) : 1.f;
-    if (isq) inv *= temp;
-    T* dst = isq ? q + (size_t)t * H * D + (size_t)job * D
-                 : (store ? kc + (size_t)slot * G * D + (size_t)(job - H) * D : nullptr);
-    if (dst) {
+    if (p.norm != QKN_HEAD) {
+      float inv;
+      const float* wn;
+      if (p.norm == QKN_HEAD_W) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NP; ++i) ss += a[i] * a[i] + b[i] * b[i];
+        inv = 1.f / sqrtf(wa_group_sum(ss, 64) / (float)D + p.eps);
+        wn = isq ? p.qn : p.kn;
+      } else {
+        inv = isq ? invq : invk;
+        wn = isq ? p.qn + (size_t)job * D : p.kn + (size_t)(job - H) * D;
+      }
 #pragma unroll
       for (int i = 0; i < NP; ++i) {
         const int e = 2 * (lane + 64 * i);
         if (e < D) {
-          Act<T>::st(dst + e, a[i] * inv);
-          if (e + 1 < D) Act<T>::st(dst + e + 1, b[i] * inv);
+          float w0, w1;
+          ld_two<float, PAIR>(wn + e, e + 1 < D, w0, w1);
+          a[i] *= inv * w0;
+          b[i] *= inv * w1;
         }
       }
     }
+    if (p.dims) {
+#pragma unroll
+      for (int i = 0; i < NP; ++i) {
+        const int e = 2 * (lane + 64 * i);
+        if (e < p.dims) {
+          float c, s;
+          ld_two<float, true>(csr + e, true, c, s);
+          const float x = a[i] * c - b[i] * s, y = b[i] * c + a[i] * s;
+          a[i] = x;
+          b[i] = y;
+        }
+      }
+    }
+    float inv = isq ? temp : 1.f;
+    if (p.norm == QKN_HEAD) {
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < NP; ++i) ss += a[i] * a[i] + b[i] * b[i];
+      inv /= sqrtf(wa_group_sum(ss, 64) / (float)D + p.eps);
+    }
+    T* dst = isq ? p.q + (size_t)t * H * D + (size_t)job * D
+                 : (store ? p.kc + (size_t)slot * G * D + (size_t)(job - H) * D : nullptr);
+    if (dst) {
+#pragma unroll
+      for (int i = 0; i < NP; ++i) {
+        const int e = 2 * (lane + 64 * i);
+        if (e < D) st_two<T, PAIR>(dst + e, e + 1 < D, a[i] * inv, b[i] * inv);
+      }
+    }
   }
-  if (v_off >= 0 && store) {
-    T* vr = vc + (size_t)slot * G * Dv;
-    if (vf) {                                      // (1 - lam) v + lam v_first
-      const T* fr = vf + (size_t)t * vf_ld;
-      for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < G * Dv; c += gridDim.y * blockDim.x)
-        Act<T>::st(vr + c, (1.f - lam) * Act<T>::ld(ur + v_off + c) + lam * Act<T>::ld(fr + c));
+  if (p.v_off >= 0 && store) {
+    T* vr = p.vc + (size_t)slot * G * Dv;
+    const T* vs = ur + p.v_off;
+    const T* fr = p.vf ? p.vf + (size_t)t * p.vf_ld : nullptr;
+    const int me = blockIdx.y * blockDim.x + threadIdx.x, all = gridDim.y * blockDim.x;
+    if (p.vruns) {
+      for (int c = 4 * me; c < G * Dv; c += 4 * all) {
+        float v[4];
+        ld_run<T, 4>(vs + c, v);
+        if (fr) {                                  // (1 - lam) v + lam v_first
+          float f[4];
+          ld_run<T, 4>(fr + c, f);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) v[i] = (1.f - p.lam) * v[i] + p.lam * f[i];
+        }
+        st_run<T, 4>(vr + c, v);
+      }
     } else {
-      for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < G * Dv; c += gridDim.y * blockDim.x)
-        vr[c] = ur[v_off + c];
+      for (int c = me; c < G * Dv; c += all) {
+        float v = Act<T>::ld(vs + c);
+        if (fr) v = (1.f - p.lam) * v + p.lam * Act<T>::ld(fr + c);
+        Act<T>::st(vr + c, v);
+      }
     }
   }
   side_relu2<T>(side, t);
@@ -801,15 +880,33 @@ extern "C" int loqa_qk_prep_append(const void* u, int dt, long ldu, int H, int G
       norm > QKN_HEAD_W || (norm != QKN_HEAD && (!qn || !kn)) || (vf && v_off < 0))
     return (int)hipErrorInvalidValue;
   const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
-  const long rows = (long)blk * nblocks;
   // a decode step has few tokens: a token's heads and columns spread over workgroups
-  const int gy = T >= 256 ? 1 : ceil_div(H + G, 4);
-#define GO(TT)                                                                                  \
-  hipLaunchKernelGGL(qk_prep_append_kernel<TT>, dim3(T, gy), dim3(256), 0, st, (const TT*)u, ldu, H, \
-                     G, D, Dv, v_off, (const float*)cs, max_pos, dims, eps, coef, every,        \
-                     (const int*)pos, (TT*)kc, (TT*)vc, rows, (const int*)kvslots, (TT*)q,      \
-                     (const float*)qn, (const float*)kn, norm, (const TT*)vf, vf_ld, lam, side)
-  if (dt == 0) GO(bf16_t); else GO(float);
+  const dim3 grid(T, T >= 256 ? 1 : ceil_div(H + G, 4));
+  const size_t esz = dt == 0 ? 2 : 4;
+  auto aligned = [&](const void* a, size_t run) { return (size_t)a % run == 0; };
+  const bool pair = D % 2 == 0 && Dv % 2 == 0 && ldu % 2 == 0 && aligned(u, 2 * esz) &&
+                    aligned(q, 2 * esz) && aligned(kc, 2 * esz) && aligned(vc, 2 * esz) &&
+                    aligned(qn, 8) && aligned(kn, 8) && aligned(cs, 8);
+  const bool vruns = v_off >= 0 && G * Dv % 4 == 0 && ldu % 4 == 0 && v_off % 4 == 0 &&
+                     aligned(u, 4 * esz) && aligned(vc, 4 * esz) &&
+                     (!vf || (vf_ld % 4 == 0 && aligned(vf, 4 * esz)));
+#define GO(TT, NP, PR)                                                                         \
+  do {                                                                                         \
+    const QkPrepParams<TT> p{(const TT*)u, ldu, H, G, D, Dv, v_off, (const float*)cs, max_pos, \
+                             dims, eps, coef, every, (const int*)pos, (TT*)kc, (TT*)vc,        \
+                             (long)blk * nblocks, (const int*)kvslots, (TT*)q,                 \
+                             (const float*)qn, (const float*)kn, norm, (const TT*)vf, vf_ld,   \
+                             lam, vruns};                                                      \
+    hipLaunchKernelGGL((qk_prep_append_kernel<TT, NP, PR>), grid, dim3(256), 0, st, p, side);  \
+  } while (0)
+#define BY_D(TT)                                                                               \
+  do {                                                                                         \
+    if (!pair) GO(TT, 4, false);                                                               \
+    else if (D <= 128) GO(TT, 1, true); else if (D <= 256) GO(TT, 2, true);                    \
+    else GO(TT, 4, true);                                                                      \
+  } while (0)
+  if (dt == 0) BY_D(bf16_t); else BY_D(float);
+#undef BY_D
 #undef GO
   return (int)hipGetLastError();
 }
