@@ -23,7 +23,7 @@
 // the value row (its own projection columns, or the k columns as projected)
 // into its page. Statistics, angles and temperature are f32. Options: a norm
 // over the whole projection, or per head, both with weights and before the
-// rotation; values blended with another layer's value rows of the same tokens;
+// rotation; no norm at all; values blended with another layer's value rows of the same tokens;
 // side columns of a parallel layer (seqmix.h).
 //
 // window_attn_keys_kernel (any dtype, any head size up to 512; decode steps,
@@ -45,7 +45,7 @@
 // contexts the windows are also dealt out to several workgroups per row, whose
 // partial triples a small combine launch merges.
 //
-// window_attn_mfma_kernel (bf16, D up to 256 and Dv up to 128 in multiples of 8,
+// window_attn_mfma_kernel (bf16, D and Dv up to 256 in multiples of 8,
 // padded with zeros in LDS to the next built size; prompt portions): a
 // workgroup per (64, 128 or 256 query rows of one sequence, query head); each
 // wave owns 32 rows. The block-table entries of the key range go to LDS once.
@@ -127,7 +127,7 @@ __device__ __forceinline__ int wa_seq_of_row(const int* __restrict__ cu_q, int B
 }
 
 // ------------------------------------------------------------------ q / k rows
-enum { QKN_HEAD = 0, QKN_WHOLE = 1, QKN_HEAD_W = 2 };
+enum { QKN_HEAD = 0, QKN_WHOLE = 1, QKN_HEAD_W = 2, QKN_NONE = 3 };
 
 // NP: pairs of neighbouring entries per lane (D <= 128 NP). PAIR: heads are even
 // and rows aligned, so a pair is one access (and the value rows go in runs of
@@ -236,7 +236,7 @@ __global__ __launch_bounds__(256) void qk_prep_append_kernel(QkPrepParams<T> p, 
                           b[i]);
       }
     }
-    if (p.norm != QKN_HEAD) {
+    if (p.norm == QKN_WHOLE || p.norm == QKN_HEAD_W) {
       float inv;
       const float* wn;
       if (p.norm == QKN_HEAD_W) {
@@ -850,6 +850,21 @@ int window_attention_mfma(const WinAttnParams& p, int max_q, hipStream_t st) {
   }
   GO(64, 64) GO(128, 64) GO(64, 128) GO(128, 128)
 #undef GO
+  // values of more than 128 entries: the accumulators alone take half the
+  // registers of a wave that has its SIMD for itself (4 waves per workgroup)
+#define GO(A, C, PADDED)                                                                      \
+  do {                                                                                        \
+    hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 4, PADDED>),                            \
+                       dim3((max_q + 127) / 128, p.H, p.B), dim3(256), 0, st, p);             \
+    return (int)hipGetLastError();                                                            \
+  } while (0)
+  if (p.Dv > 128) {
+    if (p.D == 128 && p.Dv == 256) GO(128, 256, false);
+    else if (p.D <= 128 && p.Dv <= 256) GO(128, 256, true);
+    else if (p.D <= 256 && p.Dv <= 256) GO(256, 256, true);
+    return (int)hipErrorInvalidValue;
+  }
+#undef GO
   // other sizes: the next built size, in two block widths
   const dim3 grid_p = waves == 8 ? grid : dim3((max_q + 63) / 64, p.H, p.B);
 #define GO(A, C)                                                                              \
@@ -877,7 +892,8 @@ extern "C" int loqa_qk_prep_append(const void* u, int dt, long ldu, int H, int G
   if (T <= 0) return 0;
   if (D <= 0 || D > 512 || dims < 0 || dims > D || dims % 2 || every < 1 ||
       (dims > 0 && (!cs || max_pos <= 0)) || H <= 0 || G <= 0 || norm < QKN_HEAD ||
-      norm > QKN_HEAD_W || (norm != QKN_HEAD && (!qn || !kn)) || (vf && v_off < 0))
+      norm > QKN_NONE || ((norm == QKN_WHOLE || norm == QKN_HEAD_W) && (!qn || !kn)) ||
+      (vf && v_off < 0))
     return (int)hipErrorInvalidValue;
   const SideCols side{s_src, s_src_ld, s_dst, s_dst_ld, s_n, s_lo, s_hi, s_vec};
   // a decode step has few tokens: a token's heads and columns spread over workgroups
@@ -933,7 +949,7 @@ extern "C" int loqa_window_attention(const void* q, int dt, const void* kc, cons
   // the matrix-core form reads the gate and writes the output in 8-byte runs
   const bool runs_ok = (!gate || (gate_ld % 4 == 0 && ((size_t)gate & 7) == 0)) && o_ld % 4 == 0 &&
                        ((size_t)o & 7) == 0;
-  if (mfma && dt == 0 && D % 8 == 0 && D <= 256 && Dv % 8 == 0 && Dv <= 128 && runs_ok)
+  if (mfma && dt == 0 && D % 8 == 0 && D <= 256 && Dv % 8 == 0 && Dv <= 256 && runs_ok)
     return window_attention_mfma(p, max_q, st);
   const int rep = H / G;
   // value layout: whole rows in 16-byte runs when Dv / (elements per run) is a
@@ -944,13 +960,14 @@ extern "C" int loqa_window_attention(const void* q, int dt, const void* kc, cons
   int R = rep >= 8 ? 8 : (rep >= 4 ? 4 : (rep >= 2 ? 2 : 1));
   if (nv == 8 && R > 4) R = 4;
   if (ns > 1 && part) { p.ns = ns; p.part = (float*)part; }
-  const dim3 grid(T, G, (rep + R - 1) / R * p.ns);
   // few workgroups (decode steps): 16 waves share a row's keys, else 4
   auto lds_of = [&](int nw) {
     const size_t a = (size_t)(R * D + nw * (R + 1) * 64) * 4;
     const size_t b = (size_t)(2 * nw * R + nw * R * Dv) * 4;
     return a > b ? a : b;
   };
+  while (R > 1 && lds_of(4) > 64 * 1024) R /= 2;     // wide heads: fewer of them per workgroup
+  const dim3 grid(T, G, (rep + R - 1) / R * p.ns);
   int nw = rows && R <= 2 && p.ns == 1 && (long)grid.x * grid.y * grid.z < 256 ? 16 : 4;
   if (lds_of(nw) > 64 * 1024) nw = 4;
   const size_t lds = lds_of(nw);

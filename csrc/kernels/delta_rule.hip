@@ -3,6 +3,9 @@
 //
 //   S <- g_t S;   u = beta_t (v_t - S^T k_t);   S <- S + k_t u^T;   o_t = S^T q_t
 //
+// g_t is one number per head, or (CHAN) one per head and key channel, acting on
+// the rows of S.
+//
 // delta_prep_kernel: the input stage, a wave per (token, run of D channels). The
 // q | k | v columns of the projected row pass a causal convolution per channel
 // (weights tap-major, the last tap is the current token's, no bias; rows before
@@ -10,7 +13,8 @@
 // slot needs no clearing) and SiLU; a run that is a q or k head is made a unit
 // vector x / sqrt(sum x^2 + 1e-6) by one wave reduction (q also times D^(-1/2)).
 // The gate rows give beta = sigmoid(z) and g = exp(a_neg softplus(z + dt_bias)).
-// Everything it writes is f32.
+// With a decay per key channel beta comes from a column of the projected row and
+// the H x D decays follow the token's q | k | v in act. Everything it writes is f32.
 //
 // delta_scan_kernel: one workgroup per (sequence, head, EC value columns). A
 // column of S never meets another column: u_e depends on column e of S only.
@@ -27,7 +31,9 @@
 // which is the definition with the read-out folded in (S_new^T q = g S^T q + u
 // k . q). c is the same for every column: it is computed once per token group.
 // The decayed state g S is formed while the sum for r is under way, so that one
-// multiply-add per row follows it. The state is stored with a column's rows side by side ([slots, H, Dv,
+// multiply-add per row follows it. With a decay per channel the products are S^T
+// (g k) and S^T (g q), the scaled k and q being formed off the chain from token to
+// token, and the rest is unchanged. The state is stored with a column's rows side by side ([slots, H, Dv,
 // D]), so a wave reads and writes 4 D contiguous floats. The step's tokens are
 // staged TC at a time in LDS (rows zero-padded to 16 MAXD), the next group's
 // values already in flight in registers. The recurrence runs token by token
@@ -72,9 +78,33 @@ template <int LPC> __device__ __forceinline__ float dr_lane_sum(float v) {
   return v;
 }
 
-template <typename TU>
+// The gates of one token: (g, beta) per head from gz = [beta | decay] pre-
+// activations, or (CHAN) beta from ub [H] of the projected row and the decays [H,
+// D] from gz [H D]. The token's workgroups share the work.
+template <bool CHAN, typename TU>
+__device__ __forceinline__ void dr_gates(const TU* ub, const float* gz, int H, int D,
+                                         const float* a_neg, const float* dt_bias, float* tok,
+                                         float* g) {
+  if constexpr (CHAN) {
+    for (int i = blockIdx.y * 64 + threadIdx.x; i < H * D; i += 64 * gridDim.y)
+      g[i] = expf(a_neg[i / D] * dr_softplus(gz[i] + dt_bias[i]));
+    if (blockIdx.y == 0)
+      for (int h = threadIdx.x; h < H; h += 64) {
+        tok[2 * h] = 1.f;
+        tok[2 * h + 1] = sigmoid_f(Act<TU>::ld(ub + h));
+      }
+  } else if (blockIdx.y == 0) {
+    for (int h = threadIdx.x; h < H; h += 64) {
+      tok[2 * h] = expf(a_neg[h] * dr_softplus(gz[H + h] + dt_bias[h]));
+      tok[2 * h + 1] = sigmoid_f(gz[h]);
+    }
+  }
+}
+
+template <typename TU, bool CHAN>
 __global__ __launch_bounds__(64) void delta_prep_kernel(
-    const TU* __restrict__ u, long ldu, const float* __restrict__ gz, int G, int D, int H, int Dv,
+    const TU* __restrict__ u, long ldu, const float* __restrict__ gz, long ldz, int b_off, long lda,
+    int G, int D, int H, int Dv,
     const float* __restrict__ cw, int taps, const float* __restrict__ tail, int nslots,
     const float* __restrict__ a_neg, const float* __restrict__ dt_bias,
     const int* __restrict__ sslots, const int* __restrict__ cu_q, const int* __restrict__ pos,
@@ -85,12 +115,8 @@ __global__ __launch_bounds__(64) void delta_prep_kernel(
   const int i = t - cu_q[b], p = pos[t], keep = taps - 1;
   const int QK = 2 * G * D, C = QK + H * Dv;
   const float* ts = tail + (size_t)min(max(sslots[b], 0), nslots - 1) * keep * C;
-  if (blockIdx.y == 0)
-    for (int h = lane; h < H; h += 64) {
-      const float* z = gz + (size_t)t * 2 * H;
-      tok[((size_t)t * H + h) * 2] = expf(a_neg[h] * dr_softplus(z[H + h] + dt_bias[h]));
-      tok[((size_t)t * H + h) * 2 + 1] = sigmoid_f(z[h]);
-    }
+  dr_gates<CHAN>(u + (size_t)t * ldu + b_off, gz + (size_t)t * (CHAN ? ldz : 2 * H), H, D, a_neg,
+                 dt_bias, tok + (size_t)t * 2 * H, act + (size_t)t * lda + C);
   const float qscale = 1.f / sqrtf((float)D);
   const int units = (C + D - 1) / D;            // runs of D channels: the q heads, the k heads, then v
   constexpr int NC = 8;                         // channels per lane (D <= 512)
@@ -122,7 +148,7 @@ __global__ __launch_bounds__(64) void delta_prep_kernel(
     }
 #pragma unroll
     for (int k = 0; k < NC; ++k)
-      if (lane + 64 * k < n) act[(size_t)t * C + c0 + lane + 64 * k] = y[k] * mul;
+      if (lane + 64 * k < n) act[(size_t)t * lda + c0 + lane + 64 * k] = y[k] * mul;
   }
 }
 
@@ -140,8 +166,10 @@ __device__ __forceinline__ float dr_group_sum(float v, int gs) {
   return v;
 }
 
+template <bool CHAN>
 __global__ __launch_bounds__(64) void delta_prep_v8_kernel(
-    const bf16_t* __restrict__ u, long ldu, const float* __restrict__ gz, int G, int D, int H, int Dv,
+    const bf16_t* __restrict__ u, long ldu, const float* __restrict__ gz, long ldz, int b_off,
+    long lda, int G, int D, int H, int Dv,
     const float* __restrict__ cw, int taps, const float* __restrict__ tail, int nslots,
     const float* __restrict__ a_neg, const float* __restrict__ dt_bias,
     const int* __restrict__ sslots, const int* __restrict__ cu_q, const int* __restrict__ pos,
@@ -152,12 +180,8 @@ __global__ __launch_bounds__(64) void delta_prep_v8_kernel(
   const int i = t - cu_q[b], p = pos[t], keep = taps - 1;
   const int QK = 2 * G * D, C = QK + H * Dv;
   const float* ts = tail + (size_t)min(max(sslots[b], 0), nslots - 1) * keep * C;
-  if (blockIdx.y == 0)
-    for (int h = lane; h < H; h += 64) {
-      const float* z = gz + (size_t)t * 2 * H;
-      tok[((size_t)t * H + h) * 2] = expf(a_neg[h] * dr_softplus(z[H + h] + dt_bias[h]));
-      tok[((size_t)t * H + h) * 2 + 1] = sigmoid_f(z[h]);
-    }
+  dr_gates<CHAN>(u + (size_t)t * ldu + b_off, gz + (size_t)t * (CHAN ? ldz : 2 * H), H, D, a_neg,
+                 dt_bias, tok + (size_t)t * 2 * H, act + (size_t)t * lda + C);
   const float qscale = 1.f / sqrtf((float)D);
   const int lpg = D / 8;                              // lanes per head
   for (int c = 8 * (blockIdx.y * 64 + lane); c - 8 * lane < C; c += 8 * 64 * gridDim.y) {
@@ -193,7 +217,7 @@ __global__ __launch_bounds__(64) void delta_prep_v8_kernel(
     float mul = 1.f;
     if (c < QK) mul = (c < G * D ? qscale : 1.f) / sqrtf(ss + 1e-6f);
     if (ok) {
-      float* o = act + (size_t)t * C + c;
+      float* o = act + (size_t)t * lda + c;
       *reinterpret_cast<float4*>(o) =
           make_float4(acc[0] * mul, acc[1] * mul, acc[2] * mul, acc[3] * mul);
       *reinterpret_cast<float4*>(o + 4) =
@@ -202,10 +226,10 @@ __global__ __launch_bounds__(64) void delta_prep_v8_kernel(
   }
 }
 
-template <int MAXD, int TC, int EC, int LPC>   // LPC lanes per column, D <= LPC * MAXD
+template <int MAXD, int TC, int EC, int LPC, bool CHAN>   // LPC lanes per column, D <= LPC * MAXD
 __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
     const float* __restrict__ act, long ld, int H, int D, int Dv, int q_off, int k_off, int v_off,
-    int hpg, float* __restrict__ state, const int* __restrict__ state_slots,
+    int g_off, int hpg, float* __restrict__ state, const int* __restrict__ state_slots,
     const int* __restrict__ cu_q, const int* __restrict__ positions, const float* __restrict__ tok,
     float* __restrict__ o) {
   constexpr int NTH = EC * LPC;
@@ -214,6 +238,7 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
   constexpr int NVT = (TC * EC + NTH - 1) / NTH;
   __shared__ __attribute__((aligned(16))) float qs[TC * DPAD];
   __shared__ __attribute__((aligned(16))) float ks[TC * DPAD];
+  __shared__ __attribute__((aligned(16))) float gv[CHAN ? TC * DPAD : 1];   // the channels' decays
   __shared__ float vs[TC * EC];
   __shared__ float os[TC * EC];
   __shared__ float gs[TC], bs[TC], cs[TC];
@@ -242,7 +267,8 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
   const size_t qoff = (size_t)q_off + (size_t)(h / hpg) * D;
   const size_t koff = (size_t)k_off + (size_t)(h / hpg) * D;
   const size_t voff = (size_t)v_off + (size_t)h * Dv + e0;
-  float rq[NPT], rk[NPT], rv[NVT], rg = 1.f, rb = 0.f;
+  const size_t goff = (size_t)g_off + (size_t)h * D;
+  float rq[NPT], rk[NPT], rgv[CHAN ? NPT : 1], rv[NVT], rg = 1.f, rb = 0.f;
   auto fetch = [&](int t0) {               // the values of tokens t0 .. t0 + TC into registers
     if (tid < TC) {
       const bool ok = t0 + tid < q1;
@@ -256,6 +282,7 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
       const float* row = act + (size_t)(ok ? t0 + tt : q0) * ld;
       rq[j] = ok ? row[qoff + d] : 0.f;
       rk[j] = ok ? row[koff + d] : 0.f;
+      if constexpr (CHAN) rgv[j] = ok ? row[goff + d] : 0.f;
     }
 #pragma unroll
     for (int j = 0; j < NVT; ++j) {
@@ -272,6 +299,7 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
     for (int j = 0; j < NPT; ++j) {
       qs[tid + NTH * j] = rq[j];
       ks[tid + NTH * j] = rk[j];
+      if constexpr (CHAN) gv[tid + NTH * j] = rgv[j];
     }
 #pragma unroll
     for (int j = 0; j < NVT; ++j)
@@ -293,17 +321,27 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
     }
     __syncthreads();
     for (int tt = 0; tt < nt; ++tt) {
-      float4 kc[MAXD / 4], qc[MAXD / 4];
+      float4 kc[MAXD / 4], qc[MAXD / 4], gc[MAXD / 4], kd[MAXD / 4];
       const float4* k4 = reinterpret_cast<const float4*>(ks + tt * DPAD + dp * MAXD);
       const float4* q4 = reinterpret_cast<const float4*>(qs + tt * DPAD + dp * MAXD);
 #pragma unroll
-      for (int i = 0; i < MAXD / 4; ++i) { kc[i] = k4[i]; qc[i] = q4[i]; }
+      for (int i = 0; i < MAXD / 4; ++i) { kc[i] = k4[i]; qc[i] = q4[i]; kd[i] = kc[i]; }
+      if constexpr (CHAN) {
+        const float4* g4 = reinterpret_cast<const float4*>(gv + tt * DPAD + dp * MAXD);
+#pragma unroll
+        for (int i = 0; i < MAXD / 4; ++i) {
+          const float4 w = g4[i];
+          gc[i] = w;
+          kd[i] = make_float4(w.x * kc[i].x, w.y * kc[i].y, w.z * kc[i].z, w.w * kc[i].w);
+          qc[i] = make_float4(w.x * qc[i].x, w.y * qc[i].y, w.z * qc[i].z, w.w * qc[i].w);
+        }
+      }
       const float g = gs[tt], bt = bs[tt], vv = vs[tt * EC + e], kq = cs[tt];
       float r0 = 0.f, r1 = 0.f, s0 = 0.f, s1 = 0.f;
 #pragma unroll
       for (int i = 0; i < MAXD / 4; ++i) {
-        r0 += S[4 * i] * kc[i].x;     r1 += S[4 * i + 1] * kc[i].y;
-        r0 += S[4 * i + 2] * kc[i].z; r1 += S[4 * i + 3] * kc[i].w;
+        r0 += S[4 * i] * kd[i].x;     r1 += S[4 * i + 1] * kd[i].y;
+        r0 += S[4 * i + 2] * kd[i].z; r1 += S[4 * i + 3] * kd[i].w;
       }
       // the decayed state and the second product are formed while the lane sum
       // of the first is under way
@@ -313,8 +351,16 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
         s0 += S[4 * i + 2] * qc[i].z; s1 += S[4 * i + 3] * qc[i].w;
       }
       const float r = dr_lane_sum<LPC>(r0 + r1);
+      if constexpr (CHAN) {
 #pragma unroll
-      for (int i = 0; i < MAXD; ++i) S[i] *= g;
+        for (int i = 0; i < MAXD / 4; ++i) {
+          S[4 * i] *= gc[i].x;     S[4 * i + 1] *= gc[i].y;
+          S[4 * i + 2] *= gc[i].z; S[4 * i + 3] *= gc[i].w;
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < MAXD; ++i) S[i] *= g;
+      }
       const float uu = bt * (vv - g * r);
 #pragma unroll
       for (int i = 0; i < MAXD / 4; ++i) {
@@ -343,42 +389,57 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
   }
 }
 
-extern "C" int loqa_delta_prep(const void* u, int u_dt, long ldu, const void* gz, int G, int D,
-                               int H, int Dv, const void* cw, int taps, const void* tail,
-                               int nslots, const void* a_neg, const void* dt_bias,
-                               const void* sslots, const void* cu_q, const void* pos, int B, int T,
-                               void* act, void* tok, hipStream_t st) {
+// za null: gz [T, 2 H] holds the beta and decay pre-activations of the heads. Else
+// a decay per key channel: za f32 [T, ldz] (H D columns), a_neg [H], dt_bias [H D],
+// beta from the columns b_off .. b_off + H of u, and act's rows are C + H D wide.
+extern "C" int loqa_delta_prep(const void* u, int u_dt, long ldu, const void* gz, const void* za,
+                               long ldz, int b_off, int G, int D, int H, int Dv, const void* cw,
+                               int taps, const void* tail, int nslots, const void* a_neg,
+                               const void* dt_bias, const void* sslots, const void* cu_q,
+                               const void* pos, int B, int T, void* act, void* tok,
+                               hipStream_t st) {
   if (T <= 0) return 0;
-  if (B <= 0 || taps < 1 || nslots <= 0 || G <= 0 || D <= 0 || D > 512 || H <= 0 || Dv <= 0)
+  if (B <= 0 || taps < 1 || nslots <= 0 || G <= 0 || D <= 0 || D > 512 || H <= 0 || Dv <= 0 ||
+      (!gz) == (!za) || (za && (ldz < (long)H * D || b_off < 0 || b_off + H > ldu)))
     return (int)hipErrorInvalidValue;
   const int C = 2 * G * D + H * Dv, lpg = D / 8;
+  const long lda = za ? C + (long)H * D : C;
+#define ARGS(TU)                                                                                 \
+  (const TU*)u, ldu, (const float*)(za ? za : gz), ldz, b_off, lda, G, D, H, Dv, (const float*)cw, \
+      taps, (const float*)tail, nslots, (const float*)a_neg, (const float*)dt_bias,               \
+      (const int*)sslots, (const int*)cu_q, (const int*)pos, B, (float*)act, (float*)tok
   if (u_dt == 0 && D % 8 == 0 && lpg <= 64 && (lpg & (lpg - 1)) == 0 && C % 8 == 0 &&
       ldu % 8 == 0 && ((size_t)u & 15) == 0) {
     const int per = (C + 511) / 512;
-    hipLaunchKernelGGL(delta_prep_v8_kernel, dim3(T, T >= 2048 ? (per + 1) / 2 : per), dim3(64), 0,
-                       st, (const bf16_t*)u, ldu, (const float*)gz, G, D, H, Dv, (const float*)cw,
-                       taps, (const float*)tail, nslots, (const float*)a_neg,
-                       (const float*)dt_bias, (const int*)sslots, (const int*)cu_q,
-                       (const int*)pos, B, (float*)act, (float*)tok);
+    const dim3 grid(T, T >= 2048 ? (per + 1) / 2 : per);
+    if (za)
+      hipLaunchKernelGGL((delta_prep_v8_kernel<true>), grid, dim3(64), 0, st, ARGS(bf16_t));
+    else
+      hipLaunchKernelGGL((delta_prep_v8_kernel<false>), grid, dim3(64), 0, st, ARGS(bf16_t));
     return (int)hipGetLastError();
   }
   const int units = (C + D - 1) / D;
   // many rows: a wave walks several runs
   const dim3 grid(T, T >= 4096 ? (units + 3) / 4 : units);
 #define GO(TU)                                                                                   \
-  hipLaunchKernelGGL(delta_prep_kernel<TU>, grid, dim3(64), 0, st, (const TU*)u, ldu,            \
-                     (const float*)gz, G, D, H, Dv, (const float*)cw, taps, (const float*)tail,  \
-                     nslots, (const float*)a_neg, (const float*)dt_bias, (const int*)sslots,     \
-                     (const int*)cu_q, (const int*)pos, B, (float*)act, (float*)tok)
+  do {                                                                                           \
+    if (za)                                                                                      \
+      hipLaunchKernelGGL((delta_prep_kernel<TU, true>), grid, dim3(64), 0, st, ARGS(TU));        \
+    else                                                                                         \
+      hipLaunchKernelGGL((delta_prep_kernel<TU, false>), grid, dim3(64), 0, st, ARGS(TU));       \
+  } while (0)
   if (u_dt == 0) GO(bf16_t); else GO(float);
 #undef GO
+#undef ARGS
   return (int)hipGetLastError();
 }
 
 // act: f32 [T, ld]; head h reads q at q_off + (h / hpg) D, k at k_off + (h / hpg) D,
-// v at v_off + h Dv; tok [T, H, 2] = (decay, beta); state [slots, H, Dv, D].
+// v at v_off + h Dv; tok [T, H, 2] = (decay, beta); g_off >= 0: the head's D
+// decays, one per key channel, at g_off + h D (tok's are not read); state [slots,
+// H, Dv, D].
 extern "C" int loqa_delta_scan(const void* act, long ld, int H, int D, int Dv, int q_off, int k_off,
-                               int v_off, int hpg, void* state, int nslots,
+                               int v_off, int g_off, int hpg, void* state, int nslots,
                                const void* state_slots, const void* cu_q, const void* positions,
                                const void* tok, void* o, int B, int T, hipStream_t st) {
   if (T <= 0 || B <= 0) return 0;
@@ -392,11 +453,15 @@ extern "C" int loqa_delta_scan(const void* act, long ld, int H, int D, int Dv, i
   // columns: 648 us with 8 columns, 549 us with 16, 586 us with 32) - and the
   // denser grid leaves compute units to whatever runs on the other stream.
   const int ec = Dv > 8 ? 16 : (Dv > 4 ? 8 : 4);
-#define GOL(MD, TCC, ECC, LL)                                                                     \
-  hipLaunchKernelGGL((delta_scan_kernel<MD, TCC, ECC, LL>), dim3(B, H, (Dv + ECC - 1) / ECC),     \
+#define GOC(MD, TCC, ECC, LL, CH)                                                                 \
+  hipLaunchKernelGGL((delta_scan_kernel<MD, TCC, ECC, LL, CH>), dim3(B, H, (Dv + ECC - 1) / ECC), \
                      dim3(ECC * LL), 0, st, (const float*)act, ld, H, D, Dv, q_off, k_off,        \
-                     v_off, hpg, (float*)state, (const int*)state_slots, (const int*)cu_q,        \
+                     v_off, g_off, hpg, (float*)state, (const int*)state_slots, (const int*)cu_q, \
                      (const int*)positions, (const float*)tok, (float*)o)
+#define GOL(MD, TCC, ECC, LL)                                                                     \
+  do {                                                                                            \
+    if (g_off >= 0) GOC(MD, TCC, ECC, LL, true); else GOC(MD, TCC, ECC, LL, false);               \
+  } while (0)
 #define GO(MD, TCC, ECC) GOL(MD, TCC, ECC, 16)
 #define GOE(MD, TCC)                                                                              \
   do {                                                                                            \
@@ -412,5 +477,6 @@ extern "C" int loqa_delta_scan(const void* act, long ld, int H, int D, int Dv, i
 #undef GOE
 #undef GO
 #undef GOL
+#undef GOC
   return (int)hipGetLastError();
 }

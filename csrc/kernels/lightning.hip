@@ -13,6 +13,10 @@
 // lightning_prep_kernel: act = SiLU of the q | k | v projection columns, f32,
 // once per step (every column block of a head reads the same q and k).
 //
+// retention_prep_kernel: the same for retention (a fixed decay per head, no
+// SiLU): q and k rotate pairwise by the position's angles, k times D^(-1/2), v as
+// projected, all f32.
+//
 // state_scan_kernel: one workgroup per (sequence, head, EC value columns).
 // The columns of S evolve independently, so the grid splits Dv freely: EC is
 // 32 when the batch alone fills the GPU and 16 or 8 for a lone prompt. A
@@ -38,6 +42,43 @@ __global__ __launch_bounds__(256) void lightning_prep_kernel(const T* __restrict
   const size_t r = blockIdx.x;
   for (int c = blockIdx.y * blockDim.x + threadIdx.x; c < n; c += gridDim.y * blockDim.x)
     act[r * n + c] = silu_f(Act<T>::ld(qkv + r * ld + c));
+}
+
+// N = 4: head sizes, column offsets and addresses allow runs of four (two pairs)
+template <typename T, int N>
+__global__ __launch_bounds__(256) void retention_prep_kernel(
+    const T* __restrict__ u, long ld, int H, int D, int Dv, const float* __restrict__ cs,
+    int max_pos, int dims, const int* __restrict__ pos, float* __restrict__ act) {
+  const size_t t = blockIdx.x;
+  const int HD = H * D, n = 2 * HD + H * Dv;
+  const T* ur = u + t * ld;
+  const float* cr = dims ? cs + (size_t)min(max(pos[t], 0), max_pos - 1) * dims : nullptr;
+  const float ks = 1.f / sqrtf((float)D);
+  for (int c = N * (blockIdx.y * blockDim.x + threadIdx.x); c < n; c += N * gridDim.y * blockDim.x) {
+    float v[N];
+    ld_run<T, N>(ur + c, v);
+    if (c < 2 * HD) {
+      const int e = c % D;
+      if constexpr (N == 4) {
+#pragma unroll
+        for (int k = 0; k < 4; k += 2)
+          if (e + k < dims) {
+            const float2 a = *reinterpret_cast<const float2*>(cr + e + k);
+            const float x = v[k] * a.x - v[k + 1] * a.y;
+            v[k + 1] = v[k + 1] * a.x + v[k] * a.y;
+            v[k] = x;
+          }
+      } else if (e < dims) {
+        const int e0 = e & ~1;                       // entries 2i and 2i + 1 turn together
+        const float w = Act<T>::ld(ur + c + (e == e0 ? 1 : -1));
+        v[0] = e == e0 ? v[0] * cr[e0] - w * cr[e0 + 1] : v[0] * cr[e0] + w * cr[e0 + 1];
+      }
+      if (c >= HD)
+#pragma unroll
+        for (int k = 0; k < N; ++k) v[k] *= ks;
+    }
+    st_run<float, N>(act + t * n + c, v);
+  }
 }
 
 template <int MAXD, int TC, int EC>   // D <= LS_DP * MAXD
@@ -207,6 +248,60 @@ __global__ __launch_bounds__(256) void gated_rmsnorm_kernel(
   }
 }
 
+// The same for parts of up to 512 entries: a wave per (row, part), four parts per
+// workgroup, the part in registers between the sum and the output.
+template <typename TG, typename TO>
+__global__ __launch_bounds__(256) void gated_rmsnorm_wave_kernel(
+    const float* __restrict__ o, const float* __restrict__ w, const TG* __restrict__ gate, long ldg,
+    float eps, TO* __restrict__ y, int n, int groups, int mode) {
+  const size_t r = blockIdx.x;
+  const int part = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (part >= groups) return;
+  const int per = n / groups, c0 = part * per;
+  const bool silu_first = mode == 1;
+  constexpr int NV = 8;
+  float v[NV], g[NV], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = lane + 64 * i;
+    v[i] = g[i] = 0.f;
+    if (c < per) {
+      v[i] = o[r * n + c0 + c];
+      const float z = Act<TG>::ld(gate + r * ldg + c0 + c);
+      g[i] = mode == 0 ? sigmoid_f(z) : silu_f(z);
+      if (silu_first) v[i] *= g[i];
+      ss += v[i] * v[i];
+    }
+  }
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)per + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = lane + 64 * i;
+    if (c < per)
+      Act<TO>::st(y + r * n + c0 + c, v[i] * inv * w[c0 + c] * (silu_first ? 1.f : g[i]));
+  }
+}
+
+extern "C" int loqa_retention_prep(const void* u, int dt, long ld, int H, int D, int Dv,
+                                   const void* cs, int max_pos, int dims, const void* pos, void* act,
+                                   int T, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (H <= 0 || D <= 0 || Dv <= 0 || dims < 0 || dims > D || dims % 2 ||
+      (dims > 0 && (!cs || max_pos <= 0)))
+    return (int)hipErrorInvalidValue;
+  const int n = 2 * H * D + H * Dv;
+  const bool v4 = D % 4 == 0 && Dv % 4 == 0 && ld % 4 == 0 && (size_t)u % (dt == 0 ? 8 : 16) == 0 &&
+                  (size_t)cs % 8 == 0;
+  const dim3 grid(T, T >= 512 ? 1 : ceil_div(n, v4 ? 1024 : 256));
+#define GO(TT, N)                                                                              \
+  hipLaunchKernelGGL((retention_prep_kernel<TT, N>), grid, dim3(256), 0, st, (const TT*)u, ld, \
+                     H, D, Dv, (const float*)cs, max_pos, dims, (const int*)pos, (float*)act)
+  if (dt == 0) { if (v4) GO(bf16_t, 4); else GO(bf16_t, 1); }
+  else { if (v4) GO(float, 4); else GO(float, 1); }
+#undef GO
+  return (int)hipGetLastError();
+}
+
 extern "C" int loqa_lightning_prep(const void* qkv, int dt, long ld, int T, int n, void* act,
                                    hipStream_t st) {
   if (T <= 0 || n <= 0) return 0;
@@ -261,10 +356,18 @@ extern "C" int loqa_gated_rmsnorm(const void* o, const void* w, const void* gate
                                   int mode, hipStream_t st) {
   if (T <= 0) return 0;
   if (groups <= 0 || n % groups) return (int)hipErrorInvalidValue;
-#define GO(TG, TO)                                                                            \
-  hipLaunchKernelGGL((gated_rmsnorm_kernel<TG, TO>), dim3(T, groups), dim3(256), 0, st,        \
-                     (const float*)o, (const float*)w, (const TG*)gate, ldg, eps, (TO*)y, n,   \
-                     groups, mode)
+  const bool wave = n / groups <= 512;
+#define GO(TG, TO)                                                                              \
+  do {                                                                                          \
+    if (wave)                                                                                   \
+      hipLaunchKernelGGL((gated_rmsnorm_wave_kernel<TG, TO>), dim3(T, (groups + 3) / 4),         \
+                         dim3(256), 0, st, (const float*)o, (const float*)w, (const TG*)gate,   \
+                         ldg, eps, (TO*)y, n, groups, mode);                                    \
+    else                                                                                        \
+      hipLaunchKernelGGL((gated_rmsnorm_kernel<TG, TO>), dim3(T, groups), dim3(256), 0, st,      \
+                         (const float*)o, (const float*)w, (const TG*)gate, ldg, eps, (TO*)y, n, \
+                         groups, mode);                                                         \
+  } while (0)
   if (g_dt == 0 && y_dt == 0) GO(bf16_t, bf16_t);
   else if (g_dt == 0) GO(bf16_t, float);
   else if (y_dt == 0) GO(float, bf16_t);

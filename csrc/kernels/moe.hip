@@ -9,7 +9,8 @@
 //   the choice is by the logit itself (+ bias) and the weights are the softmax
 //   over the chosen logits only. Mode 2: scores = sigmoid(z) instead of the
 //   softmax. With `grank` n > 1 a group ranks by the sum of its n best choice
-//   scores.
+//   scores. With `renorm` the chosen weights are divided by their sum (+ 1e-20);
+//   `wscale` multiplies them.
 // moe_plan_kernel (one workgroup): (token, k) pairs bucketed by expert without
 //   a host round trip: offsets[E + 2], perm[P] (pair ids in expert order; the
 //   identity bucket E last), pos[P] (where each pair sits).
@@ -18,7 +19,9 @@
 //   pair's result does not depend on which other pairs share its tile). Mode
 //   1 gathers A rows by token and applies the SwiGLU epilogue to the (gate,
 //   up) weight row pairs; mode 2 gathers A rows by token and squares the relu
-//   of a single (up) weight set; mode 0 reads the sorted activation rows.
+//   of a single (up) weight set; mode 3 is mode 1 with the clamped gate
+//   g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, +-limit);
+//   mode 0 reads the sorted activation rows.
 // moe_combine_kernel: out[t] = sum_k weight * (expert output | the input
 //   itself for an identity expert), f32.
 #include "seqmix.h"
@@ -36,8 +39,8 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
 
 __global__ __launch_bounds__(64) void moe_route_kernel(
     const float* __restrict__ z, const float* __restrict__ corr, const float* __restrict__ bias,
-    int mode, int E, int G, int keep, int grank, int top, int* __restrict__ idx,
-    float* __restrict__ wt) {
+    int mode, int E, int G, int keep, int grank, int top, int renorm, float wscale,
+    int* __restrict__ idx, float* __restrict__ wt) {
   const int top_softmax = mode == 1;
   __shared__ float sc[MOE_MAX_E], ch[MOE_MAX_E], gs[MOE_MAX_E];
   const int t = blockIdx.x, lane = threadIdx.x;
@@ -109,6 +112,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(
       if (gs[e / per] != INFINITY) ch[e] = -INFINITY;
     __syncthreads();
   }
+  float tot = 0.f;
   for (int k = 0; k < top; ++k) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
@@ -121,15 +125,14 @@ __global__ __launch_bounds__(64) void moe_route_kernel(
     if (lane == 0) {
       idx[(size_t)t * top + k] = bi;
       wt[(size_t)t * top + k] = sc[bi];
+      tot += sc[bi];
       ch[bi] = INFINITY;                      // taken
     }
     __syncthreads();
   }
-  if (top_softmax && lane == 0) {
-    // softmax over the chosen logits: exp(z - max) of the chosen ones over their sum
-    float tot = 0.f;
-    for (int k = 0; k < top; ++k) tot += wt[(size_t)t * top + k];
-    const float r = 1.f / tot;
+  if ((top_softmax || renorm || wscale != 1.f) && lane == 0) {
+    // top_softmax: exp(z - max) of the chosen logits over their sum
+    const float r = top_softmax ? wscale / tot : renorm ? wscale / (tot + 1e-20f) : wscale;
     for (int k = 0; k < top; ++k) wt[(size_t)t * top + k] *= r;
   }
 }
@@ -170,12 +173,23 @@ __global__ __launch_bounds__(256) void moe_plan_kernel(const int* __restrict__ i
 #define GG_K 16
 
 __device__ __forceinline__ float relu2_f(float z) { const float r = fmaxf(z, 0.f); return r * r; }
+__device__ __forceinline__ float clamped_glu_f(float g, float u, float limit) {
+  g = fminf(g, limit);
+  return g * sigmoid_f(1.702f * g) * (fminf(fmaxf(u, -limit), limit) + 1.f);
+}
+// the up product's epilogue (a: gate or the only product, u: up)
+template <int MODE> __device__ __forceinline__ float moe_epilogue(float a, float u, float limit) {
+  if constexpr (MODE == 1) return silu_f(a) * u;
+  else if constexpr (MODE == 2) return relu2_f(a);
+  else if constexpr (MODE == 3) return clamped_glu_f(a, u, limit);
+  else return a;
+}
 
 template <typename T, int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_gemm_kernel(
     const T* __restrict__ A, const T* __restrict__ Wt, const int* __restrict__ plan, int P, int E,
-    int top, int K, int N, T* __restrict__ out) {
-  constexpr int SWIGLU = MODE == 1;
+    int top, int K, int N, float limit, T* __restrict__ out) {
+  constexpr int SWIGLU = MODE == 1 || MODE == 3;    // gate and up rows
   constexpr bool GATHER = MODE != 0;
   __shared__ float As[GG_K][GG_T + 1], Bs[GG_K][GG_T + 1], Bu[SWIGLU ? GG_K : 1][GG_T + 1];
   const int* offsets = plan;
@@ -244,8 +258,8 @@ __global__ __launch_bounds__(256) void moe_grouped_gemm_kernel(
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n < N)
-        Act<T>::st(out + (size_t)r * N + n, SWIGLU ? silu_f(acc[i][j]) * accu[i][j]
-                                                   : MODE == 2 ? relu2_f(acc[i][j]) : acc[i][j]);
+        Act<T>::st(out + (size_t)r * N + n,
+                   moe_epilogue<MODE>(acc[i][j], accu[SWIGLU ? i : 0][j], limit));
     }
   }
 }
@@ -262,8 +276,8 @@ __global__ __launch_bounds__(256) void moe_grouped_gemm_kernel(
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_gemm_mfma_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wt, const int* __restrict__ plan, int P,
-    int E, int top, int K, int N, bf16_t* __restrict__ out) {
-  constexpr int SWIGLU = MODE == 1;
+    int E, int top, int K, int N, float limit, bf16_t* __restrict__ out) {
+  constexpr int SWIGLU = MODE == 1 || MODE == 3;    // gate and up rows
   constexpr bool GATHER = MODE != 0;
   const int* offsets = plan;
   const int* perm = plan + E + 2;
@@ -319,9 +333,8 @@ __global__ __launch_bounds__(256) void moe_grouped_gemm_mfma_kernel(
     for (int i = 0; i < 4; ++i) {
       const int n = nb + 4 * fq + i;
       if (n < N) {
-        const float v = SWIGLU ? silu_f(acc[j][i]) * accu[j][i]
-                               : MODE == 2 ? relu2_f(acc[j][i]) : acc[j][i];
-        out[(size_t)r * N + n] = f2bf(v);
+        out[(size_t)r * N + n] =
+            f2bf(moe_epilogue<MODE>(acc[j][i], accu[SWIGLU ? j : 0][i], limit));
       }
     }
   }
@@ -342,8 +355,8 @@ __global__ __launch_bounds__(256) void moe_grouped_gemm_mfma_kernel(
 template <int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_gemm_mfma2_kernel(
     const bf16_t* __restrict__ A, const bf16_t* __restrict__ Wt, const int* __restrict__ plan, int P,
-    int E, int top, int K, int N, bf16_t* __restrict__ out) {
-  constexpr int SWIGLU = MODE == 1;
+    int E, int top, int K, int N, float limit, bf16_t* __restrict__ out) {
+  constexpr int SWIGLU = MODE == 1 || MODE == 3;    // gate and up rows
   constexpr bool GATHER = MODE != 0;
   __shared__ __attribute__((aligned(16))) bf16_t rows[GG_R2][GG_KC + 8];
   const int* offsets = plan;
@@ -458,9 +471,8 @@ __global__ __launch_bounds__(256) void moe_grouped_gemm_mfma2_kernel(
       for (int i = 0; i < 4; ++i) {
         const int n = nb + 16 * f + 4 * fq + i;
         if (n < N) {
-          const float v = SWIGLU ? silu_f(acc[f][j][i]) * accu[f][j][i]
-                                 : MODE == 2 ? relu2_f(acc[f][j][i]) : acc[f][j][i];
-          out[(size_t)r * N + n] = f2bf(v);
+          out[(size_t)r * N + n] = f2bf(
+              moe_epilogue<MODE>(acc[f][j][i], accu[SWIGLU ? f : 0][SWIGLU ? j : 0][i], limit));
         }
       }
     }
@@ -501,6 +513,66 @@ __global__ __launch_bounds__(256) void act_mul_any_kernel(const T* __restrict__ 
   }
 }
 
+// relu(x)^2 entry by entry, in place or out of place
+template <typename T, int N>
+__global__ __launch_bounds__(256) void relu2_any_kernel(const T* x, long n, T* y) {
+  for (long i = N * ((long)blockIdx.x * 256 + threadIdx.x); i < n; i += N * 256L * gridDim.x) {
+    float f[N];
+    ld_run<T, N>(x + i, f);
+#pragma unroll
+    for (int k = 0; k < N; ++k) f[k] = relu2_f(f[k]);
+    st_run<T, N>(y + i, f);
+  }
+}
+
+extern "C" int loqa_relu2_any(const void* x, int dt, long n, void* y, hipStream_t st) {
+  if (n <= 0) return 0;
+  const size_t esz = dt == 0 ? 2 : 4;
+  const bool v4 = n % 4 == 0 && (size_t)x % (4 * esz) == 0 && (size_t)y % (4 * esz) == 0;
+  const long units = (n / (v4 ? 4 : 1) + 255) / 256;
+  const dim3 grid((int)(units < 8192 ? units : 8192));
+#define GO(TT, NN)                                                                            \
+  hipLaunchKernelGGL((relu2_any_kernel<TT, NN>), grid, dim3(256), 0, st, (const TT*)x, n, (TT*)y)
+  if (dt == 0) { if (v4) GO(bf16_t, 4); else GO(bf16_t, 1); }
+  else { if (v4) GO(float, 4); else GO(float, 1); }
+#undef GO
+  return (int)hipGetLastError();
+}
+
+// y[t, c] = gelu_tanh(z[t, c]) * table[tokens[t], off + c]: a gate on the rows of
+// a per-token table. TE: the table's dtype.
+template <typename T, typename TE>
+__global__ __launch_bounds__(256) void token_gate_kernel(const T* __restrict__ z, long ldz,
+                                                         const TE* __restrict__ table, long ldt,
+                                                         const int* __restrict__ tokens, int vocab,
+                                                         int off, int n, T* __restrict__ y, int T_) {
+  const long total = (long)T_ * n;
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < total; i += 256L * gridDim.x) {
+    const int t = (int)(i / n), c = (int)(i - (long)t * n);
+    const int tok = min(max(tokens[t], 0), vocab - 1);
+    Act<T>::st(y + i, gelu_tanh_f(Act<T>::ld(z + (size_t)t * ldz + c)) *
+                          Act<TE>::ld(table + (size_t)tok * ldt + off + c));
+  }
+}
+
+extern "C" int loqa_token_gate(const void* z, int dt, long ldz, const void* table, int t_dt, long ldt,
+                               const void* tokens, int vocab, int off, int n, void* y, int T,
+                               hipStream_t st) {
+  if (T <= 0 || n <= 0) return 0;
+  if (vocab <= 0 || off < 0 || off + n > ldt || ldz < n) return (int)hipErrorInvalidValue;
+  const long units = ((long)T * n + 255) / 256;
+  const dim3 grid((int)(units < 8192 ? units : 8192));
+#define GO(TT, TE)                                                                            \
+  hipLaunchKernelGGL((token_gate_kernel<TT, TE>), grid, dim3(256), 0, st, (const TT*)z, ldz,   \
+                     (const TE*)table, ldt, (const int*)tokens, vocab, off, n, (TT*)y, T)
+  if (dt == 0 && t_dt == 0) GO(bf16_t, bf16_t);
+  else if (dt == 0) GO(bf16_t, float);
+  else if (t_dt == 0) GO(float, bf16_t);
+  else GO(float, float);
+#undef GO
+  return (int)hipGetLastError();
+}
+
 extern "C" int loqa_act_mul_any(const void* x, int dt, int T, int F, int act, void* y,
                                 hipStream_t st) {
   if (T <= 0) return 0;
@@ -517,13 +589,14 @@ extern "C" int loqa_act_mul_any(const void* x, int dt, int T, int F, int act, vo
 }
 
 extern "C" int loqa_moe_route(const void* z, const void* corr, const void* bias, int mode,
-                              int E, int G, int keep, int grank, int top, void* idx, void* wt,
-                              int T, hipStream_t st) {
+                              int E, int G, int keep, int grank, int top, int renorm, float wscale,
+                              void* idx, void* wt, int T, hipStream_t st) {
   if (T <= 0) return 0;
   if (E > MOE_MAX_E || E <= 0 || G <= 0 || E % G || top <= 0 || top > E || mode < 0 || mode > 2)
     return (int)hipErrorInvalidValue;
   hipLaunchKernelGGL(moe_route_kernel, dim3(T), dim3(64), 0, st, (const float*)z, (const float*)corr,
-                     (const float*)bias, mode, E, G, keep, grank, top, (int*)idx, (float*)wt);
+                     (const float*)bias, mode, E, G, keep, grank, top, renorm, wscale, (int*)idx,
+                     (float*)wt);
   return (int)hipGetLastError();
 }
 
@@ -534,22 +607,20 @@ extern "C" int loqa_moe_plan(const void* idx, int P, int E, void* plan, hipStrea
 }
 
 extern "C" int loqa_moe_grouped_gemm(const void* A, int dt, const void* W, const void* plan, int P,
-                                     int E, int top, int K, int N, int mode, void* out,
+                                     int E, int top, int K, int N, int mode, float limit, void* out,
                                      hipStream_t st) {
   if (P <= 0) return 0;
-  if (mode < 0 || mode > 2) return (int)hipErrorInvalidValue;
+  if (mode < 0 || mode > 3) return (int)hipErrorInvalidValue;
   const dim3 grid((P + GG_T - 1) / GG_T + E, (N + GG_T - 1) / GG_T);
+#define GO_MODE(M, KERNEL, GRID, TT)                                                             \
+  hipLaunchKernelGGL(KERNEL(M), GRID, dim3(256), 0, st, (const TT*)A, (const TT*)W,             \
+                     (const int*)plan, P, E, top, K, N, limit, (TT*)out)
 #define BY_MODE(KERNEL, GRID, TT)                                                               \
   do {                                                                                          \
-    if (mode == 1)                                                                              \
-      hipLaunchKernelGGL(KERNEL(1), GRID, dim3(256), 0, st, (const TT*)A, (const TT*)W,         \
-                         (const int*)plan, P, E, top, K, N, (TT*)out);                          \
-    else if (mode == 2)                                                                         \
-      hipLaunchKernelGGL(KERNEL(2), GRID, dim3(256), 0, st, (const TT*)A, (const TT*)W,         \
-                         (const int*)plan, P, E, top, K, N, (TT*)out);                          \
-    else                                                                                        \
-      hipLaunchKernelGGL(KERNEL(0), GRID, dim3(256), 0, st, (const TT*)A, (const TT*)W,         \
-                         (const int*)plan, P, E, top, K, N, (TT*)out);                          \
+    if (mode == 1) GO_MODE(1, KERNEL, GRID, TT);                                                \
+    else if (mode == 2) GO_MODE(2, KERNEL, GRID, TT);                                           \
+    else if (mode == 3) GO_MODE(3, KERNEL, GRID, TT);                                           \
+    else GO_MODE(0, KERNEL, GRID, TT);                                                          \
   } while (0)
 #define K_MFMA2(M) (moe_grouped_gemm_mfma2_kernel<M>)
 #define K_MFMA(M) (moe_grouped_gemm_mfma_kernel<M>)
@@ -571,6 +642,7 @@ extern "C" int loqa_moe_grouped_gemm(const void* A, int dt, const void* W, const
 #undef K_BF16
 #undef K_F32
 #undef BY_MODE
+#undef GO_MODE
   return (int)hipGetLastError();
 }
 

@@ -15,9 +15,10 @@ Two kinds of per-sequence memory share one sequence table:
   ``BlockPool``);
 * **state slots**: one slot per live sequence (the last slot is the write
   target of padding rows) in every per-layer state tensor: a recurrent layer's
-  matrix state [slots + 1, H, D, Dv] f32 (``state``), or named f32 rows of any
+  matrix state [slots + 1, H, D, Dv] f32 (``state``), named f32 rows of any
   shape [slots + 1, ...] (``rows``: a previous token's activations, the tail
-  of a short convolution). A slot is taken when a sequence is added and
+  of a short convolution), or named int32 values (``ints``: a previous token's
+  id). A slot is taken when a sequence is added and
   returned with its pages when the sequence is freed; the kernels treat the
   state of a sequence at position 0 as zero, so a reused slot needs no
   clearing.
@@ -117,7 +118,11 @@ class HybridCache:
         self.rows = {li: {name: torch.zeros(max_seqs + 1, *shape, dtype=torch.float32, device=dev)
                           for name, shape in named.items()}
                      for li, named in spec.get("rows", {}).items()}
-        self.slots = SlotPool(max_seqs) if (self.state or self.rows) else None
+        # named per-sequence integers
+        self.ints = {key: {name: torch.zeros(max_seqs + 1, *shape, dtype=torch.int32, device=dev)
+                           for name, shape in named.items()}
+                     for key, named in spec.get("ints", {}).items()}
+        self.slots = SlotPool(max_seqs) if (self.state or self.rows or self.ints) else None
         self.pool = _SeqPool(make_block_pool(num_blocks, block_size,
                                              require_native=dev.type == "cuda"), self.slots)
 
@@ -134,5 +139,6 @@ class HybridCache:
     def nbytes(self) -> int:
         ts = [*self.latent.values(), *self.state.values()]
         ts += [t for pair in (*self.kv.values(), *self.kv_rows.values()) for t in pair]
-        ts += [t for named in self.rows.values() for t in named.values()]
+        ts += [t for group in (self.rows, self.ints) for named in group.values()
+               for t in named.values()]
         return sum(t.numel() * t.element_size() for t in ts)

@@ -263,7 +263,9 @@ class FeedForwardConfig:
     groups: int = 1
     keep: int = 1
     shared_ff: int = 0              # 0: no shared expert
-    # "swiglu": down(silu(gate x) * (up x)); "relu2": down(relu(up x)^2), no gate
+    # "swiglu": down(silu(gate x) * (up x)); "relu2": down(relu(up x)^2), no gate;
+    # "clamped_glu": down(g sigmoid(1.702 g) (u + 1)), g = min(gate x, limit), u =
+    # clamp(up x, -limit, limit)
     act: str = "swiglu"
     # "swiglu" / "geglu" (the tanh form of GELU on the gate) for dense layers
     # router: "softmax_all" scores every output and weighs by the plain score;
@@ -273,6 +275,9 @@ class FeedForwardConfig:
     router: str = "softmax_all"
     # a group of experts ranks by the sum of its ``group_rank`` best scores
     group_rank: int = 1
+    limit: float = 0.0              # of "clamped_glu"
+    renorm: bool = False            # the chosen weights are divided by their sum
+    weight_scale: float = 1.0       # ... and multiplied by this
 
 
 @dataclass(frozen=True)
@@ -440,7 +445,8 @@ class SoftmaxAttnConfig:
     # "head": q and k divided by their root mean square per head after rotation,
     # no weight; "whole": RMS norm over the whole q (and k) projection with a
     # weight vector of that size, before rotation; "head_weight": RMS norm per
-    # head with a weight of the head's size shared by the heads, before rotation
+    # head with a weight of the head's size shared by the heads, before rotation;
+    # "none": no norm
     qk_norm: str = "head"
     zero_sink: bool = False         # the softmax denominator holds one more term exp(0)
     sink: bool = False              # ... one more term exp(sink_h), learned per head
@@ -594,6 +600,9 @@ class DeltaRuleConfig:
     dim: int
     vdim: int
     taps: int                       # short causal convolution on q, k and v
+    # the decay: one per head, or one per head and key channel (a low-rank
+    # projection, as the output gate's then is)
+    channel_decay: bool = False
 
     @property
     def conv_channels(self) -> int:
@@ -601,11 +610,21 @@ class DeltaRuleConfig:
 
 
 @dataclass(frozen=True)
+class RetentionConfig:
+    heads: int
+    dim: int                        # query / key size per head
+    vdim: int
+    decay: tuple                    # fixed, one per head
+    rot: RotaryConfig
+
+
+@dataclass(frozen=True)
 class ParallelMixerConfig:
     left: SoftmaxAttnConfig
-    right: DeltaRuleConfig
+    right: object                   # DeltaRuleConfig | RetentionConfig
     left_scale: float
     right_scale: float
+    out_norms: bool = False         # each output RMS-normed over the width, with a weight
 
 
 @dataclass(frozen=True)
@@ -765,3 +784,113 @@ def gopopel_config_from_json(d: dict, name: str = "gopopel") -> GopopelConfig:
                              f"{mix[0][0]}, which they are mixed with")
     return GopopelConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]),
                          float((d.get("embedding") or {}).get("scale", 1.0)), tuple(layers))
+
+
+# --------------------------------------------------------------------------
+# Vodalorn: a pre-norm decoder with layer norms (weight and bias), a constant on
+# every residual addition, an embedding that adds a row hashed from the token
+# pair, and after every layer's feed-forward a gated per-token side input. A
+# stretch of layers may run several times in a row with the same weights, each
+# pass entered through a projection of [x ; embedding output] plus a learned
+# vector of its own. Mixers: sliding-window softmax attention beside retention
+# (both outputs RMS-normed, half their sum), and a gated delta rule with a decay
+# per key channel. Feed-forwards: dense squared relu, or experts with a clamped
+# gated unit behind a softmax router with renormalised weights. Every size and
+# constant comes from config.json or a tensor's shape.
+@dataclass(frozen=True)
+class BigramConfig:
+    buckets: int
+    mul_prev: int
+    mul_cur: int                    # row (previous * mul_prev + current * mul_cur) mod buckets
+
+
+@dataclass(frozen=True)
+class VodalornConfig:
+    name: str
+    vocab_size: int
+    d_model: int
+    norm_eps: float
+    residual_mult: float
+    layers: tuple
+    bigram: BigramConfig | None = None
+    side_dim: int = 0               # width of a layer's per-token side input; 0: none
+    loop: LoopConfig | None = None
+
+    @property
+    def n_layers(self) -> int:
+        return len(self.layers)
+
+    def runs(self) -> list[tuple[int, int | None]]:
+        """The layers in execution order as (layer index, the number of the pass
+        when the run opens a pass of the repeated stretch, else None); every run
+        has a cache or state of its own."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None) for i in range(n)]
+        lp = self.loop
+        out = [(i, None) for i in range(lp.start)]
+        for t in range(lp.times):
+            out += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
+        return out + [(i, None) for i in range(lp.stop, n)]
+
+
+def vodalorn_config_from_json(d: dict, name: str = "vodalorn") -> VodalornConfig:
+    layers = []
+    for i, L in enumerate(d["layers"]):
+        m, kind = L["mixer"], L["type"]
+        if kind == "channel_delta":
+            mixer = DeltaRuleConfig(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]),
+                                    int(m["vdim"]), int(m["conv"]), channel_decay=True)
+            if mixer.heads % mixer.kv_heads or mixer.taps < 1:
+                raise ValueError(f"layer {i}: heads or conv taps do not fit")
+        elif kind == "parallel":
+            a, r = m["left"], m["right"]
+            left = SoftmaxAttnConfig(int(a["heads"]), int(a["kv_heads"]), int(a["dim"]),
+                                     int(a["vdim"]), float(a["scale"]), bias=True,
+                                     rot=_rot_half(a["rot"], int(a["dim"]), f"layer {i}"),
+                                     window=int(a["mask"]["size"]), qk_norm="none")
+            right = RetentionConfig(int(r["heads"]), int(r["dim"]), int(r["vdim"]),
+                                    tuple(float(v) for v in r["decay"]),
+                                    _rot_half(r["rot"], int(r["dim"]), f"layer {i}"))
+            if left.heads % left.kv_heads or left.window < 1:
+                raise ValueError(f"layer {i}: heads or mask size do not fit")
+            if len(right.decay) != right.heads:
+                raise ValueError(f"layer {i}: one decay per head expected")
+            mixer = ParallelMixerConfig(left, right, 0.5, 0.5, out_norms=True)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        f = L.get("mlp")
+        if not f:
+            mlp = None
+        elif f["kind"] == "dense":
+            mlp = FeedForwardConfig("dense", int(f["ff"]), act="relu2")
+        elif f["kind"] == "moe":
+            r, e = f["router"], f["expert"]
+            g = r.get("groups") or {}
+            mlp = FeedForwardConfig("moe", int(e["ff"]), int(r["experts"]), 0, int(r["top"]),
+                                    int(g.get("count", 1)), int(g.get("keep", g.get("count", 1))),
+                                    act="clamped_glu", limit=float(e["limit"]), renorm=True,
+                                    weight_scale=float(r.get("scale", 1.0)))
+            if mlp.experts % mlp.groups or not 0 < mlp.keep <= mlp.groups:
+                raise ValueError(f"layer {i}: {mlp.experts} experts do not split into "
+                                 f"{mlp.groups} groups")
+            if not 0 < mlp.top <= mlp.keep * (mlp.experts // mlp.groups):
+                raise ValueError(f"layer {i}: top {mlp.top} exceeds the eligible experts")
+        else:
+            raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+        layers.append(HybridLayerConfig(kind, mixer, mlp))
+    lp = d.get("loop")
+    loop = None
+    if lp:
+        loop = LoopConfig(int(lp["start"]), int(lp["stop"]), int(lp["times"]))
+        if not 0 <= loop.start <= loop.stop <= len(layers) or loop.times < 1:
+            raise ValueError("loop: start, stop and times do not fit the layer list")
+        if loop.start == loop.stop:
+            loop = None
+    b = (d.get("embedding") or {}).get("bigram")
+    bigram = BigramConfig(int(b["buckets"]), int(b["mul_prev"]), int(b["mul_cur"])) if b else None
+    if bigram is not None and bigram.buckets < 1:
+        raise ValueError("bigram: buckets must be positive")
+    return VodalornConfig(name, int(d["vocab"]), int(d["width"]), float(d["norm"]["eps"]),
+                          float(d.get("residual_mult", 1.0)), tuple(layers), bigram,
+                          int((d.get("token_side") or {}).get("dim", 0)), loop)

@@ -4,9 +4,10 @@ own naming, told apart by ``"architecture"``: the hybrid Pipizen (latent /
 lightning mixers), Sodonex (chunked sigmoid attention with row state) and
 Movinex (windowed softmax attention, Mamba-2 layers, a repeated stretch of
 layers), Vilulix (parallel layers; matrix memory, latent attention, windowed
-attention beside a gated delta rule) and Gopopel (parallel layers on one norm;
+attention beside a gated delta rule), Gopopel (parallel layers on one norm;
 windowed attention with a distance bias and value mixing, windowed latent
-attention). A family knows how to read its config, load or seed its weights and
+attention) and Vodalorn (windowed attention beside retention, a delta rule with a
+decay per key channel, token-pair embedding, per-token side inputs). A family knows how to read its config, load or seed its weights and
 build its step function; the engine, the scheduler and the command line go
 through this table only.
 """
@@ -18,9 +19,10 @@ from typing import Callable
 import torch
 
 from .configs import (GopopelConfig, LlamaConfig, MovinexConfig, PipizenConfig, SodonexConfig,
-                      VilulixConfig, checkpoint_config, gopopel_config_from_json,
+                      VilulixConfig, VodalornConfig, checkpoint_config, gopopel_config_from_json,
                       llama_config_from_hf, movinex_config_from_json, pipizen_config_from_json,
-                      sodonex_config_from_json, vilulix_config_from_json)
+                      sodonex_config_from_json, vilulix_config_from_json,
+                      vodalorn_config_from_json)
 
 
 @dataclass(frozen=True)
@@ -52,6 +54,10 @@ def _is_gopopel(d: dict) -> bool:
     return str(d.get("architecture", "")).lower() == "gopopel"
 
 
+def _is_vodalorn(d: dict) -> bool:
+    return str(d.get("architecture", "")).lower() == "vodalorn"
+
+
 def _is_llama(d: dict) -> bool:
     arch = " ".join(d.get("architectures") or []) + " " + str(d.get("model_type", ""))
     return "num_attention_heads" in d and ("llama" in arch.lower() or "hidden_size" in d)
@@ -63,6 +69,7 @@ FAMILIES = (
     Family("movinex", MovinexConfig, _is_movinex, movinex_config_from_json, True),
     Family("vilulix", VilulixConfig, _is_vilulix, vilulix_config_from_json, True),
     Family("gopopel", GopopelConfig, _is_gopopel, gopopel_config_from_json, True),
+    Family("vodalorn", VodalornConfig, _is_vodalorn, vodalorn_config_from_json, True),
     Family("llama", LlamaConfig, _is_llama, llama_config_from_hf, False),
 )
 
@@ -109,6 +116,8 @@ def load_lm_weights(cfg, path: str, device, *, dtype=torch.bfloat16, tp=None,
         return loader.load_vilulix(cfg, path, device, dtype, max_positions)
     if fam.name == "gopopel":
         return loader.load_gopopel(cfg, path, device, dtype, max_positions)
+    if fam.name == "vodalorn":
+        return loader.load_vodalorn(cfg, path, device, dtype, max_positions)
     return loader.load_pipizen(cfg, path, device, dtype, max_positions)
 
 
@@ -130,6 +139,9 @@ def random_lm_weights(cfg, device, *, seed: int = 0, dtype=torch.bfloat16, tp=No
     if fam.name == "gopopel":
         from .gopopel import GopopelWeights
         return GopopelWeights.random(cfg, device, seed, dtype, max_positions)
+    if fam.name == "vodalorn":
+        from .vodalorn import VodalornWeights
+        return VodalornWeights.random(cfg, device, seed, dtype, max_positions)
     from .pipizen import PipizenWeights
     return PipizenWeights.random(cfg, device, seed, dtype, max_positions)
 
@@ -150,5 +162,8 @@ def build_model(weights):
     from .gopopel import GopopelModel, GopopelWeights
     if isinstance(weights, GopopelWeights):
         return GopopelModel(weights)
+    from .vodalorn import VodalornModel, VodalornWeights
+    if isinstance(weights, VodalornWeights):
+        return VodalornModel(weights)
     from .pipizen import PipizenModel
     return PipizenModel(weights)

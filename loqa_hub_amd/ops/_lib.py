@@ -225,9 +225,11 @@ _SEQMIX_SIGS = {
                         _vp, _i, _i, _i, _vp],
     "loqa_gated_rmsnorm": [_vp, _vp, _vp, _i, _l, _f, _vp, _i, _i, _i, _i, _i, _vp],
     "loqa_act_mul_any": [_vp, _i, _i, _i, _i, _vp, _vp],
-    "loqa_moe_route": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _vp],
+    "loqa_moe_route": [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _f, _vp, _vp, _i, _vp],
     "loqa_moe_plan": [_vp, _i, _i, _vp, _vp],
-    "loqa_moe_grouped_gemm": [_vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _vp],
+    "loqa_moe_grouped_gemm": [_vp, _i, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _vp, _vp],
+    "loqa_relu2_any": [_vp, _i, _l, _vp, _vp],
+    "loqa_token_gate": [_vp, _i, _l, _vp, _i, _l, _vp, _i, _i, _i, _vp, _i, _vp],
     "loqa_moe_combine": [_vp, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _i, _vp, _vp],
     "loqa_token_shift": [_vp, _vp, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _vp, _i, _vp],
     "loqa_seq_state_save": [_vp, _i, _vp, _i, _i, _vp, _vp, _i, _i, _i, _vp, _vp, _vp, _i, _vp],
@@ -255,10 +257,15 @@ _SEQMIX_SIGS = {
     "loqa_exp_gate_scan": [_vp, _i, _vp, _vp, _f, _vp, _i, _vp, _vp, _vp, _i, _i, _vp, _vp, _vp],
     "loqa_matrix_memory_inputs": [_vp, _i, _l, _i, _i, _i, _vp, _i, _vp],
     "loqa_normalized_gated_rmsnorm": [_vp, _vp, _vp, _vp, _i, _l, _f, _vp, _i, _i, _i, _i, _vp],
-    "loqa_delta_prep": [_vp, _i, _l, _vp, _i, _i, _i, _i, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp,
+    "loqa_delta_prep": [_vp, _i, _l, _vp, _vp, _l, _i, _i, _i, _i, _i, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp,
                         _vp, _i, _i, _vp, _vp, _vp],
-    "loqa_delta_scan": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i,
+    "loqa_delta_scan": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i,
                         _i, _vp],
+    "loqa_retention_prep": [_vp, _i, _l, _i, _i, _i, _vp, _i, _i, _vp, _vp, _i, _vp],
+    "loqa_residual_ln": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _f, _vp, _vp, _vp, _f, _vp, _i, _l, _i,
+                         _i, _vp],
+    "loqa_bigram_embed": [_vp, _vp, _vp, _i, _i, _l, _l, _l, _vp, _i, _vp, _vp, _vp, _i, _i, _vp,
+                          _vp, _i, _l, _i, _i, _vp],
 }
 _seqmix = None
 

@@ -800,7 +800,8 @@ def gated_rmsnorm(o, w, gate, eps: float, out_dtype, groups: int = 1, silu_first
 
 
 def moe_route(z, correction, n_groups: int, keep: int, top: int, bias=None,
-              top_softmax: bool = False, sigmoid: bool = False, group_rank: int = 1):
+              top_softmax: bool = False, sigmoid: bool = False, group_rank: int = 1,
+              renorm: bool = False, weight_scale: float = 1.0):
     """z f32 [T, E] router logits (+ ``bias`` [E]) -> (expert index int32 [T, top],
     weight f32 [T, top]). Default: scores are softmax(z); experts are chosen by
     score + correction among the ``keep`` best of ``n_groups`` equal groups of
@@ -808,11 +809,12 @@ def moe_route(z, correction, n_groups: int, keep: int, top: int, bias=None,
     plain scores. ``top_softmax``: the ``top`` largest logits are chosen and the
     weights are the softmax over the chosen logits only. ``sigmoid``: the scores
     are sigmoid(z) instead of the softmax. ``group_rank`` n: a group ranks by the
-    sum of its n best choice scores."""
+    sum of its n best choice scores. ``renorm``: the weights are divided by their
+    sum (+ 1e-20); ``weight_scale`` multiplies them last."""
     z = z.float() if bias is None else z.float() + bias.float()
     if top_softmax:
         best = z.topk(top, dim=-1)
-        return best.indices.to(torch.int32), torch.softmax(best.values, dim=-1)
+        return best.indices.to(torch.int32), torch.softmax(best.values, dim=-1) * weight_scale
     s = torch.sigmoid(z) if sigmoid else torch.softmax(z, dim=-1)
     choice = s if correction is None else s + correction.float()
     if n_groups > 1 and keep < n_groups:
@@ -823,13 +825,17 @@ def moe_route(z, correction, n_groups: int, keep: int, top: int, bias=None,
         ok = torch.zeros(T, n_groups, dtype=torch.bool, device=z.device).scatter_(1, kept, True)
         choice = choice.masked_fill(~ok.repeat_interleave(per, dim=1), float("-inf"))
     idx = choice.topk(top, dim=-1).indices
-    return idx.to(torch.int32), s.gather(1, idx)
+    wt = s.gather(1, idx)
+    if renorm:
+        wt = wt / (wt.sum(-1, keepdim=True) + 1e-20)
+    return idx.to(torch.int32), wt * weight_scale
 
 
-def moe_experts(h, idx, wt, w_gate_up, w_down, out_dtype, gated: bool = True):
+def moe_experts(h, idx, wt, w_gate_up, w_down, out_dtype, gated: bool = True, limit=None):
     """Weighted sum of each token's chosen experts: expert e < E is a
     feed-forward - gated: down(silu(gate x) * (up x)) with w_gate_up [E, 2F, d]
-    = gate | up rows; not gated: down(relu(up x)^2) with w_gate_up [E, F, d] -
+    = gate | up rows (with ``limit``: g sigmoid(1.702 g) (u + 1) with g = min(gate,
+    limit), u = clamp(up, -limit, limit)); not gated: down(relu(up x)^2) with w_gate_up [E, F, d] -
     and w_down [E, d, F]; an index >= E is an identity expert (its output is
     h). Returns f32 [T, d]; the expert outputs are rounded to ``out_dtype``
     first, as GEMM outputs."""
@@ -845,7 +851,11 @@ def moe_experts(h, idx, wt, w_gate_up, w_down, out_dtype, gated: bool = True):
             rows = (e == ee).nonzero()[:, 0]
             x = h[rows].to(out_dtype)
             gu = torch.nn.functional.linear(x, w_gate_up[ee])
-            if gated:
+            if limit is not None:
+                g = gu[:, :F].float().clamp(max=limit)
+                u = gu[:, F:].float().clamp(-limit, limit)
+                a = (g * torch.sigmoid(1.702 * g) * (u + 1.0)).to(out_dtype)
+            elif gated:
                 a = (torch.nn.functional.silu(gu[:, :F].float()) * gu[:, F:].float()).to(out_dtype)
             else:
                 a = torch.relu(gu.float()).pow(2).to(out_dtype)
@@ -1031,7 +1041,7 @@ def scaled_add_rms1p(resid, y, ls, nxt, eps: float, out_dtype):
 
 def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims: int, eps: float,
                    q_temp, positions, k_cache, v_cache, slots, out_dtype, q_norm=None, k_norm=None,
-                   v_mix=None, side=None):
+                   v_mix=None, side=None, norm: bool = True):
     """u [T, >= H D + G D (+ G Dv)]: projected q | k (| v) rows. Per head: the
     first ``dims`` entries of q and k rotate pairwise (2i with 2i + 1) by the
     position's angles, then each head's q and k is divided by its root mean
@@ -1044,7 +1054,7 @@ def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims
     are RMS-normed over their whole projection with these weights BEFORE the
     rotation, and no per-head division follows; with both [D] per head with
     shared weights, also before it. ``v_mix`` = (v_first [T, G Dv], lam): the
-    values stored are (1 - lam) v + lam v_first."""
+    values stored are (1 - lam) v + lam v_first. ``norm`` False: no norm at all."""
     T = u.shape[0]
     uf = u.float()
     q = uf[:, :H * D].reshape(T, H, D)
@@ -1064,7 +1074,7 @@ def qk_prep_append(u, H: int, G: int, D: int, Dv: int, v_off: int, cos_sin, dims
     if dims:
         cs = cos_sin[pos]
         q, k = rotate_pairs(q, cs, dims), rotate_pairs(k, cs, dims)
-    if q_norm is None:
+    if q_norm is None and norm:
         q = q * torch.rsqrt(q.pow(2).mean(-1, keepdim=True) + eps)
         k = k * torch.rsqrt(k.pow(2).mean(-1, keepdim=True) + eps)
     if q_temp is not None:
@@ -1253,7 +1263,7 @@ def normalized_gated_rmsnorm(o, floor, w, gate, eps: float, out_dtype, H: int, D
 
 
 def delta_prep(u, gz, G: int, D: int, H: int, Dv: int, conv_w, tail, a_neg, dt_bias, state_slots,
-               cu_q, positions):
+               cu_q, positions, chan=None):
     """The input stage of a gated delta rule over a flat token batch. u [T, >=
     C], C = 2 G D + H Dv: the projected q | k | v rows pass a causal
     convolution per channel (weights tap-major [taps, C], the last tap is the
@@ -1261,7 +1271,9 @@ def delta_prep(u, gz, G: int, D: int, H: int, Dv: int, conv_w, tail, a_neg, dt_b
     before position 0) and SiLU; every q and k head becomes a unit vector x /
     sqrt(sum x^2 + 1e-6), q also times D^(-1/2) -> f32 [T, C]. gz f32 [T, 2 H]:
     the first H columns give beta = sigmoid(z), the others the decay exp(a_neg
-    softplus(z + dt_bias)) -> f32 [T, H, 2] = (decay, beta)."""
+    softplus(z + dt_bias)) -> f32 [T, H, 2] = (decay, beta). ``chan`` = (za f32 [T,
+    H D], b_off): a decay per head and key channel from za, beta from the columns
+    at b_off of u; the H D decays follow the C inputs of a token."""
     T = u.shape[0]
     taps, C = conv_w.shape
     cu = cu_q.tolist()
@@ -1286,6 +1298,12 @@ def delta_prep(u, gz, G: int, D: int, H: int, Dv: int, conv_w, tail, a_neg, dt_b
     qk = qk * torch.rsqrt(qk.pow(2).sum(-1, keepdim=True) + 1e-6)
     qk[:, :G] *= D ** -0.5
     act = torch.cat([qk.reshape(T, 2 * G * D), y[:, 2 * G * D:]], dim=1).contiguous()
+    if chan is not None:
+        za, b_off = chan
+        beta = torch.sigmoid(u[:, b_off:b_off + H].float())
+        g = torch.exp(a_neg.float()[None, :, None] * torch.nn.functional.softplus(
+            za.float() + dt_bias.float()).view(T, H, D)).view(T, H * D)
+        return torch.cat([act, g], dim=1), torch.stack([torch.ones_like(beta), beta], -1).contiguous()
     z = gz.float()
     beta = torch.sigmoid(z[:, :H])
     decay = torch.exp(a_neg.float() * torch.nn.functional.softplus(z[:, H:] + dt_bias.float()))
@@ -1293,12 +1311,13 @@ def delta_prep(u, gz, G: int, D: int, H: int, Dv: int, conv_w, tail, a_neg, dt_b
 
 
 def delta_scan(act, H: int, D: int, Dv: int, q_off: int, k_off: int, v_off: int, hpg: int, state,
-               state_slots, cu_q, positions, tok):
+               state_slots, cu_q, positions, tok, g_off=None):
     """The gated delta rule, token by token in f32, per sequence and head:
 
         S <- g S;   u = beta (v - S^T k);   S <- S + k u^T;   o = S^T q
 
-    with (g, beta) = ``tok[t, h]``. ``act`` f32 [T, W]: head h reads q at
+    with (g, beta) = ``tok[t, h]``, or g a vector over the rows of S, the D columns
+    at ``g_off + h D``. ``act`` f32 [T, W]: head h reads q at
     ``q_off + (h // hpg) D``, k at ``k_off + (h // hpg) D`` and v at ``v_off +
     h Dv``. The state is kept with a column's rows side by side, [slots, H, Dv,
     D]; it is read at the sequence's slot (zero when the step's first position
@@ -1320,10 +1339,83 @@ def delta_scan(act, H: int, D: int, Dv: int, q_off: int, k_off: int, v_off: int,
         S = torch.zeros(H, D, Dv, dtype=torch.float32, device=act.device) \
             if int(positions[q0]) == 0 else state[slot].transpose(1, 2).clone()
         for t in range(q0, q1):
-            S = tok[t, :, 0].float()[:, None, None] * S
+            S = S * (tok[t, :, 0].float()[:, None, None] if g_off is None else
+                     a[t, g_off:g_off + H * D].view(H, D, 1))
             r = torch.einsum("hde,hd->he", S, k[t])
             uu = tok[t, :, 1].float()[:, None] * (v[t] - r)
             S = S + k[t][:, :, None] * uu[:, None, :]
             o[t] = torch.einsum("hde,hd->he", S, q[t])
         state[slot] = S.transpose(1, 2)
     return o.view(T, H * Dv)
+
+
+# ---------------------------------------------------------------------------
+# Layer norm on the residual step, token-pair embedding, per-token side inputs,
+# retention inputs
+def layer_norm(x, w, b, eps: float):
+    """(x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b over rows, f32."""
+    c = x.float() - x.float().mean(-1, keepdim=True)
+    return c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * w.float() + b.float()
+
+
+def residual_ln(resid, addends, scale: float, nxt, eps: float, out, vec=None, row_idx=None):
+    """resid (f32, in place) += scale * sum of the addends (y, w), each y / rms(y) *
+    w where it has a weight, + ``vec``; ``out`` takes layer_norm(resid; nxt = (w,
+    b)), or resid itself without ``nxt`` (rows ``row_idx`` of it)."""
+    s = None
+    for y, w in addends:
+        y = y.float()
+        if w is not None:
+            y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+        s = y if s is None else s + y
+    if s is not None:
+        resid.add_(s * float(scale))
+    if vec is not None:
+        resid.add_(vec.float())
+    if out is not None:
+        x = resid if row_idx is None else resid[row_idx]
+        out.copy_(x if nxt is None else layer_norm(x, *nxt, eps))
+    return out
+
+
+def bigram_embed(tokens, embed, pairs, mul_prev: int, mul_cur: int, prev, state_slots, cu_q,
+                 positions, out2=None):
+    """embed[token] + pairs[hash of (previous token, token)], the pair table's last
+    row at position 0; the token before a feed comes from ``prev[slot]``, which
+    becomes the feed's last token."""
+    toks, pos, cu = tokens.tolist(), positions.tolist(), cu_q.tolist()
+    buckets = pairs.shape[0] - 1
+    rows = [buckets] * len(toks)
+    for b in range(len(cu) - 1):
+        if cu[b + 1] == cu[b]:
+            continue
+        slot = int(state_slots[b])
+        before = int(prev[slot])
+        for t in range(cu[b], cu[b + 1]):
+            if pos[t] > 0:
+                rows[t] = (before * int(mul_prev) + toks[t] * int(mul_cur)) % buckets
+            before = toks[t]
+        prev[slot] = before
+    x = embed[tokens.long()].float() + pairs[torch.tensor(rows, device=pairs.device)].float()
+    if out2 is not None:
+        out2.copy_(x.repeat(1, out2.shape[1] // x.shape[1]))
+    return x
+
+
+def token_gate(z, table, tokens, off: int):
+    """gelu_tanh(z) * table[tokens, off : off + n]."""
+    g = torch.nn.functional.gelu(z.float(), approximate="tanh")
+    return (g * table[tokens.long(), off:off + z.shape[1]].float()).to(z.dtype)
+
+
+def retention_prep(u, H: int, D: int, Dv: int, cos_sin, dims: int, positions):
+    """q | k | v of retention in f32: q and k rotated pairwise on the first ``dims``
+    entries of each head, k times D^(-1/2), v as projected."""
+    T = u.shape[0]
+    q = u[:, :H * D].float().reshape(T, H, D)
+    k = u[:, H * D:2 * H * D].float().reshape(T, H, D)
+    if dims:
+        cs = cos_sin[positions[:T].long()]
+        q, k = rotate_pairs(q, cs, dims), rotate_pairs(k, cs, dims)
+    return torch.cat([q.reshape(T, H * D), k.reshape(T, H * D) * D ** -0.5,
+                      u[:, 2 * H * D:2 * H * D + H * Dv].float()], dim=1).contiguous()

@@ -5,12 +5,15 @@ grouped top-k expert router with its expert feed-forward; further down the
 row-state ops and sigmoid attention of the Sodonex family, and the pre-norm /
 layer-scale residual step, windowed softmax attention over paged K / V and the
 Mamba-2 input stage of the Movinex family (whose recurrence is ``state_scan``,
-the generalised lightning scan).
+the generalised lightning scan); the layer norm on the residual step, the
+token-pair embedding, per-token side inputs and the retention input stage of the
+Vodalorn family come last.
 
 As everywhere in ``ops``: GPU tensors run the HIP kernels
 (``csrc/kernels/norm_dyt.hip``, ``attn_latent.hip``, ``lightning.hip``,
 ``moe.hip``, ``seq_rows.hip``, ``attn_sigmoid.hip``, ``norm_scalar.hip``,
-``norm_rms1p.hip``, ``attn_window.hip``, ``mamba2.hip``), CPU tensors the f32
+``norm_rms1p.hip``, ``attn_window.hip``, ``mamba2.hip``, ``matrix_memory.hip``,
+``delta_rule.hip``, ``norm_layer.hip``), CPU tensors the f32
 PyTorch references (the CPU test tier and the numerics oracle of the GPU
 tests). Activations are bfloat16 or float32
 (``_DT``); the residual stream, scores, softmax, recurrent state, router and
@@ -459,7 +462,8 @@ def silu_mul_any(x: torch.Tensor) -> torch.Tensor:
 
 def moe_route(z: torch.Tensor, correction: torch.Tensor | None, n_groups: int, keep: int,
               top: int, bias: torch.Tensor | None = None, top_softmax: bool = False,
-              sigmoid: bool = False, group_rank: int = 1) -> tuple[torch.Tensor, torch.Tensor]:
+              sigmoid: bool = False, group_rank: int = 1, renorm: bool = False,
+              weight_scale: float = 1.0) -> tuple[torch.Tensor, torch.Tensor]:
     """Router decisions from f32 logits z [T, E] (+ ``bias`` [E]). Default:
     softmax scores, choice by score + ``correction`` limited to the ``keep``
     best of ``n_groups`` groups of neighbouring experts, weights = the plain
@@ -467,10 +471,11 @@ def moe_route(z: torch.Tensor, correction: torch.Tensor | None, n_groups: int, k
     chosen and weighed by the softmax over the chosen logits only. ``sigmoid``:
     the scores are sigmoid(z) instead of the softmax. ``group_rank`` n: a group
     ranks by the sum of its n best choice scores instead of its best one.
-    Returns (idx int32 [T, top], weight f32 [T, top])."""
+    ``renorm``: the chosen weights are divided by their sum (+ 1e-20);
+    ``weight_scale`` multiplies them last. Returns (idx int32 [T, top], weight f32 [T, top])."""
     if not z.is_cuda:
         return ref.moe_route(z, correction, n_groups, keep, top, bias, top_softmax, sigmoid,
-                             group_rank)
+                             group_rank, renorm, weight_scale)
     assert not (top_softmax and sigmoid)
     _f32c(z, "z")
     T, E = z.shape
@@ -485,22 +490,25 @@ def moe_route(z: torch.Tensor, correction: torch.Tensor | None, n_groups: int, k
         check(kernels().loqa_moe_route(ptr(z), ptr(correction), ptr(bias),
                                        1 if top_softmax else (2 if sigmoid else 0), E,
                                        max(1, n_groups), min(keep, max(1, n_groups)),
-                                       max(1, group_rank), top, ptr(idx), ptr(wt), T,
+                                       max(1, group_rank), top, int(renorm), float(weight_scale),
+                                       ptr(idx), ptr(wt), T,
                                        stream_ptr(z)), "moe_route")
     return idx, wt
 
 
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, wt: torch.Tensor, w_gate_up: torch.Tensor,
-                w_down: torch.Tensor, gated: bool = True) -> torch.Tensor:
+                w_down: torch.Tensor, gated: bool = True, limit: float | None = None) -> torch.Tensor:
     """Weighted sum of every token's chosen experts, f32 [T, d]. Experts below
     E = w_gate_up.shape[0] are feed-forwards: gated (w_gate_up [E, 2F, d] with
-    gate rows then up rows, SwiGLU) or not (w_gate_up [E, F, d], the square of
-    relu), w_down [E, d, F]; an index >= E is an identity expert. On the GPU: a
+    gate rows then up rows, SwiGLU; with ``limit`` the clamped gate g sigmoid(1.702
+    g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)) or not
+    (w_gate_up [E, F, d], the square of relu), w_down [E, d, F]; an index >= E is an identity expert. On the GPU: a
     device-side plan (tokens grouped by expert, no host round trip), a grouped
     up GEMM with the activation as its epilogue, a grouped down GEMM, and a
     combine launch that applies the weights in f32."""
     if not h.is_cuda:
-        return ref.moe_experts(h, idx, wt, w_gate_up, w_down, h.dtype, gated)
+        return ref.moe_experts(h, idx, wt, w_gate_up, w_down, h.dtype, gated, limit)
+    assert gated or limit is None
     T, d = h.shape
     E, F2, _ = w_gate_up.shape
     F = F2 // 2 if gated else F2
@@ -522,8 +530,9 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wt: torch.Tensor, w_gate_up:
     k, st = kernels(), stream_ptr(h)
     check(k.loqa_moe_plan(ptr(idx), P, E, ptr(plan), st), "moe_plan")
     check(k.loqa_moe_grouped_gemm(ptr(h), _dt(h), ptr(w_gate_up), ptr(plan), P, E, top, d, F,
-                                  1 if gated else 2, ptr(act), st), "moe_up")
-    check(k.loqa_moe_grouped_gemm(ptr(act), _dt(h), ptr(w_down), ptr(plan), P, E, top, F, d, 0,
+                                  (1 if limit is None else 3) if gated else 2, limit or 0.0,
+                                  ptr(act), st), "moe_up")
+    check(k.loqa_moe_grouped_gemm(ptr(act), _dt(h), ptr(w_down), ptr(plan), P, E, top, F, d, 0, 0.0,
                                   ptr(y), st), "moe_down")
     check(k.loqa_moe_combine(ptr(h), ptr(y), _dt(h), ptr(idx), ptr(wt), ptr(plan), T, top, E, d,
                              ptr(out), st), "moe_combine")
@@ -770,7 +779,7 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
                    positions: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                    slots: torch.Tensor, out_dtype, q_norm: torch.Tensor | None = None,
                    k_norm: torch.Tensor | None = None, v_mix: tuple | None = None,
-                   side: SideCols | None = None) -> torch.Tensor:
+                   side: SideCols | None = None, norm: bool = True) -> torch.Tensor:
     """One launch between the fused q | k (| v) projection u [T, W] and
     attention: per head the first ``dims`` entries of q and k rotate pairwise
     (interleaved layout, table ``cos_sin`` [positions, dims / 2, 2]), then q and
@@ -786,16 +795,17 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
     RMS-normed per head with weights shared by the heads, also before it (sizes
     that fit both readings, H = G = 1, mean the same). ``v_mix`` = (v_first [T,
     G Dv], lam): the stored values are (1 - lam) v + lam v_first. ``side``: see
-    :class:`SideCols`."""
-    assert (q_norm is None) == (k_norm is None)
+    :class:`SideCols`. ``norm`` False: no division or norm of any kind."""
+    assert (q_norm is None) == (k_norm is None) and (norm or q_norm is None)
     if not u.is_cuda:
         return ref.qk_prep_append(u, H, G, D, Dv, v_off, cos_sin, dims, eps, q_temp, positions,
-                                  k_cache, v_cache, slots, out_dtype, q_norm, k_norm, v_mix, side)
-    norm = 0
+                                  k_cache, v_cache, slots, out_dtype, q_norm, k_norm, v_mix, side,
+                                  norm)
+    mode = 0 if norm else 3
     if q_norm is not None:
         _f32c(q_norm, "q_norm"); _f32c(k_norm, "k_norm")
-        norm = 2 if q_norm.numel() == k_norm.numel() == D else 1
-        assert norm == 2 or (q_norm.numel() == H * D and k_norm.numel() == G * D)
+        mode = 2 if q_norm.numel() == k_norm.numel() == D else 1
+        assert mode == 2 or (q_norm.numel() == H * D and k_norm.numel() == G * D)
     vf, lam = None, 0.0
     if v_mix is not None:
         vf, lam = v_mix
@@ -822,16 +832,16 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
             ptr(u), _dt(u), u.stride(0), H, G, D, Dv, int(v_off), ptr(cos_sin) if dims else None,
             cos_sin.shape[0] if dims else 0, dims, float(eps), coef, every, ptr(positions),
             ptr(k_cache), ptr(v_cache), k_cache.shape[1], k_cache.shape[0], ptr(slots), ptr(q), T,
-            ptr(q_norm), ptr(k_norm), norm, ptr(vf), vf.stride(0) if vf is not None else 0,
+            ptr(q_norm), ptr(k_norm), mode, ptr(vf), vf.stride(0) if vf is not None else 0,
             float(lam), *(side.args() if side is not None else _NO_SIDE), stream_ptr(u)),
             "qk_prep_append")
     return q
 
 
 def window_mfma_sizes(D: int, Dv: int) -> bool:
-    """Head sizes the matrix-core form covers (built for 64 / 128 / 256 and 64 /
-    128; multiples of 8 in between are padded with zeros in LDS)."""
-    return D % 8 == 0 and 0 < D <= 256 and Dv % 8 == 0 and 0 < Dv <= 128
+    """Head sizes the matrix-core form covers (built for 64 / 128 / 256 both ways;
+    multiples of 8 in between are padded with zeros in LDS)."""
+    return D % 8 == 0 and 0 < D <= 256 and Dv % 8 == 0 and 0 < Dv <= 256
 
 
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
@@ -1108,7 +1118,8 @@ def normalized_gated_rmsnorm(o: torch.Tensor, floor: torch.Tensor, w: torch.Tens
 def delta_prep(u: torch.Tensor, gz: torch.Tensor, G: int, D: int, H: int, Dv: int,
                conv_w: torch.Tensor, tail: torch.Tensor, a_neg: torch.Tensor,
                dt_bias: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
-               positions: torch.Tensor) -> tuple[torch.Tensor, torch.Tensor]:
+               positions: torch.Tensor, chan: tuple | None = None
+               ) -> tuple[torch.Tensor, torch.Tensor]:
     """The input stage of a gated delta rule, one launch over a flat token
     batch. The first C = 2 G D + H Dv columns of the projected rows u [T, W] (q
     | k | v) pass a causal convolution per channel (f32 weights tap-major [taps,
@@ -1118,24 +1129,35 @@ def delta_prep(u: torch.Tensor, gz: torch.Tensor, G: int, D: int, H: int, Dv: in
     times D^(-1/2) -> f32 [T, C]. gz f32 [T, 2 H]: the first H columns give the
     write strengths beta = sigmoid(z), the others the decays exp(a_neg
     softplus(z + dt_bias)) -> f32 [T, H, 2] = (decay, beta). ``tail`` is not
-    written here (:func:`seq_state_save` does, after every reader)."""
+    written here (:func:`seq_state_save` does, after every reader).
+
+    ``chan`` = (za, b_off): a decay per head and key channel. za f32 [T, H D] are
+    the decays' pre-activations, ``dt_bias`` [H D], ``a_neg`` [H], beta comes from
+    the columns b_off .. b_off + H of u and ``gz`` is None; the decays follow the
+    token's inputs, so the first result is f32 [T, C + H D]."""
     if not u.is_cuda:
         return ref.delta_prep(u, gz, G, D, H, Dv, conv_w, tail, a_neg, dt_bias, state_slots, cu_q,
-                              positions)
+                              positions, chan)
     T, W = u.shape
     taps, C = conv_w.shape
     assert C == 2 * G * D + H * Dv and u.stride(1) == 1 and C <= W
+    za, b_off = chan if chan is not None else (None, 0)
+    assert (gz is None) == (za is not None) and 0 <= b_off <= W - H
+    if za is not None:
+        assert za.dtype == torch.float32 and za.shape == (T, H * D) and za.stride(1) == 1
     for t, name, n in ((conv_w, "conv_w", None), (tail, "tail", None), (a_neg, "a_neg", H),
-                       (dt_bias, "dt_bias", H), (gz, "gz", T * 2 * H)):
+                       (dt_bias, "dt_bias", H if za is None else H * D),
+                       *(((gz, "gz", T * 2 * H),) if za is None else ())):
         _f32c(t, name)
         assert n is None or t.numel() == n
     assert tail.shape[1:] == (taps - 1, C)
     B = _seq_args(state_slots, cu_q, positions, T)
-    act = torch.empty(T, C, dtype=torch.float32, device=u.device)
+    act = torch.empty(T, C + (H * D if za is not None else 0), dtype=torch.float32, device=u.device)
     tok = torch.empty(T, H, 2, dtype=torch.float32, device=u.device)
     if T:
         check(kernels().loqa_delta_prep(
-            ptr(u), _dt(u), u.stride(0), ptr(gz), G, D, H, Dv, ptr(conv_w), taps, ptr(tail),
+            ptr(u), _dt(u), u.stride(0), ptr(gz), ptr(za), za.stride(0) if za is not None else 0,
+            b_off, G, D, H, Dv, ptr(conv_w), taps, ptr(tail),
             tail.shape[0], ptr(a_neg), ptr(dt_bias), ptr(state_slots), ptr(cu_q), ptr(positions), B,
             T, ptr(act), ptr(tok), stream_ptr(u)), "delta_prep")
     return act, tok
@@ -1143,10 +1165,12 @@ def delta_prep(u: torch.Tensor, gz: torch.Tensor, G: int, D: int, H: int, Dv: in
 
 def delta_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: int, v_off: int,
                hpg: int, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
-               positions: torch.Tensor, tok: torch.Tensor) -> torch.Tensor:
+               positions: torch.Tensor, tok: torch.Tensor, g_off: int | None = None
+               ) -> torch.Tensor:
     """The gated delta rule with a carried matrix state, per sequence and head,
     token by token in f32:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;
-    o = S^T q, with (g, beta) = ``tok[t, h]``. ``act`` f32 [T, W]: head h reads
+    o = S^T q, with (g, beta) = ``tok[t, h]``; with ``g_off`` g is a vector over the
+    rows of S, the D columns at ``g_off + h D`` of ``act``. ``act`` f32 [T, W]: head h reads
     q at ``q_off + (h // hpg) D``, k at ``k_off + (h // hpg) D`` and v at
     ``v_off + h Dv``. ``state`` [slots, H, Dv, D] f32 (a column's rows side by
     side) carries S between steps (zero when the step's first position is 0).
@@ -1154,16 +1178,167 @@ def delta_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     tokens."""
     if not act.is_cuda:
         return ref.delta_scan(act, H, D, Dv, q_off, k_off, v_off, hpg, state, state_slots, cu_q,
-                              positions, tok)
+                              positions, tok, g_off)
     T, W = act.shape
     _f32c(act, "act"); _f32c(state, "state"); _f32c(tok, "tok")
+    assert g_off is None or 0 <= g_off and g_off + H * D <= W
     assert state.shape[1:] == (H, Dv, D) and hpg >= 1 and H % hpg == 0 and tok.shape == (T, H, 2)
     G = H // hpg
     assert min(q_off, k_off, v_off) >= 0 and max(q_off, k_off) + G * D <= W and v_off + H * Dv <= W
     B = _seq_args(state_slots, cu_q, positions, T)
     o = torch.empty(T, H * Dv, dtype=torch.float32, device=act.device)
     if T:
-        check(kernels().loqa_delta_scan(ptr(act), W, H, D, Dv, q_off, k_off, v_off, hpg, ptr(state),
+        check(kernels().loqa_delta_scan(ptr(act), W, H, D, Dv, q_off, k_off, v_off,
+                                        -1 if g_off is None else g_off, hpg, ptr(state),
                                         state.shape[0], ptr(state_slots), ptr(cu_q), ptr(positions),
                                         ptr(tok), ptr(o), B, T, stream_ptr(act)), "delta_scan")
     return o
+
+
+# ---------------------------------------------------------------------------
+# Layer norm on the residual step, token-pair embedding, per-token side inputs,
+# retention inputs (csrc/kernels/norm_layer.hip, moe.hip, lightning.hip)
+class LnParams:
+    """A layer norm's f32 weight and bias."""
+    __slots__ = ("w", "b")
+
+    def __init__(self, w: torch.Tensor, b: torch.Tensor):
+        self.w, self.b = w.float().contiguous(), b.float().contiguous()
+
+    def tup(self):
+        return self.w, self.b
+
+
+def residual_ln(resid: torch.Tensor, addends: list, scale: float, nxt: "LnParams | None",
+                eps: float, out: torch.Tensor | None, vec: torch.Tensor | None = None,
+                row_idx: torch.Tensor | None = None) -> torch.Tensor | None:
+    """The residual step of a pre-norm layer with layer norms: resid (f32, in
+    place) += ``scale`` * sum_i n_i(y_i) + ``vec``, over up to two ``addends`` (y
+    [rows, d] in one activation dtype, w f32 [d] or None), n_i(y) = y / sqrt(mean
+    y^2 + eps) * w with a weight and y itself without; ``vec`` f32 [d]. The same
+    launch writes to ``out`` [rows, d] (any activation dtype; may be a column slice
+    of a wider row) the layer norm of the sum, (resid - mean) / sqrt(var + eps) * w
+    + b, or with ``nxt`` None the sum itself; ``out`` None: nothing. Without
+    addends and ``vec`` it is the norm alone; ``row_idx`` (int64) gathers rows of
+    resid then."""
+    if not resid.is_cuda:
+        return ref.residual_ln(resid, addends, scale, None if nxt is None else nxt.tup(), eps, out,
+                               vec, row_idx)
+    _f32c(resid, "resid")
+    d = resid.shape[1]
+    rows = resid.shape[0]
+    if row_idx is not None:
+        assert row_idx.dtype == torch.int64 and row_idx.is_contiguous() and not addends
+        assert vec is None and out is not None
+        rows = row_idx.numel()
+    assert len(addends) <= 2 and (nxt is None or out is not None)
+    ys, ws = [None, None], [None, None]
+    for i, (y, w) in enumerate(addends):
+        assert y.shape == resid.shape and y.is_contiguous() and y.dtype == addends[0][0].dtype
+        ys[i], ws[i] = y, w
+        if w is not None:
+            _f32c(w, "addend weight")
+            assert w.numel() == d
+    if vec is not None:
+        assert vec.dtype == torch.float32 and vec.is_contiguous() and vec.numel() == d
+    if nxt is not None:
+        assert nxt.w.numel() == d and nxt.b.numel() == d
+    if out is not None:
+        assert out.shape == (rows, d) and out.stride(1) == 1
+    if rows:
+        check(kernels().loqa_residual_ln(
+            ptr(resid), ptr(row_idx), ptr(ys[0]), ptr(ws[0]), ptr(ys[1]), ptr(ws[1]),
+            _dt(ys[0]) if addends else 0, float(scale), ptr(vec), ptr(nxt.w) if nxt else None,
+            ptr(nxt.b) if nxt else None, float(eps), ptr(out), _dt(out) if out is not None else 0,
+            out.stride(0) if out is not None else d, rows, d, stream_ptr(resid)), "residual_ln")
+    return out
+
+
+def bigram_embed(tokens: torch.Tensor, embed: torch.Tensor, pairs: torch.Tensor, mul_prev: int,
+                 mul_cur: int, prev: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
+                 positions: torch.Tensor, out2: torch.Tensor | None = None) -> torch.Tensor:
+    """x = embed[token] + pairs[row], f32 [T, d]: row = (previous token * mul_prev +
+    token * mul_cur) mod buckets, for a sequence's first token the table's last row
+    (``pairs`` [buckets + 1, d]). The token before a feed is ``prev[slot]`` int32
+    [slots], which is set to the feed's last token. ``out2`` [T, n d] (activation
+    dtype) receives n copies of x side by side."""
+    if not tokens.is_cuda:
+        return ref.bigram_embed(tokens, embed, pairs, mul_prev, mul_cur, prev, state_slots, cu_q,
+                                positions, out2)
+    T, d = tokens.numel(), embed.shape[1]
+    _i32c(tokens, "tokens"); _i32c(prev, "prev")
+    assert embed.is_contiguous() and pairs.is_contiguous() and embed.dtype == pairs.dtype
+    assert pairs.shape[1] == d and pairs.shape[0] > 1
+    B = _seq_args(state_slots, cu_q, positions, T)
+    x = torch.empty(T, d, dtype=torch.float32, device=tokens.device)
+    n = 0
+    if out2 is not None:
+        n = out2.shape[1] // d
+        assert out2.shape == (T, n * d) and out2.stride(1) == 1
+    if T:
+        check(kernels().loqa_bigram_embed(
+            ptr(tokens), ptr(embed), ptr(pairs), _dt(embed), embed.shape[0], pairs.shape[0] - 1,
+            int(mul_prev), int(mul_cur), ptr(prev), prev.numel(), ptr(state_slots), ptr(cu_q),
+            ptr(positions), B, T, ptr(x), ptr(out2), _dt(out2) if out2 is not None else 0,
+            out2.stride(0) if out2 is not None else 0, n, d, stream_ptr(tokens)), "bigram_embed")
+    return x
+
+
+def token_gate(z: torch.Tensor, table: torch.Tensor, tokens: torch.Tensor, off: int) -> torch.Tensor:
+    """gelu_tanh(z) * table[tokens, off : off + n] for z [T, n] (may be a column
+    slice) and a per-token table [vocab, W] in bf16 or f32 -> [T, n]."""
+    if not z.is_cuda:
+        return ref.token_gate(z, table, tokens, off)
+    T, n = z.shape
+    _i32c(tokens, "tokens")
+    assert z.stride(1) == 1 and table.is_contiguous() and off + n <= table.shape[1]
+    assert tokens.numel() == T
+    y = torch.empty(T, n, dtype=z.dtype, device=z.device)
+    if T:
+        check(kernels().loqa_token_gate(ptr(z), _dt(z), z.stride(0), ptr(table), _dt(table),
+                                        table.shape[1], ptr(tokens), table.shape[0], int(off), n,
+                                        ptr(y), T, stream_ptr(z)), "token_gate")
+    return y
+
+
+def relu2_(x: torch.Tensor) -> torch.Tensor:
+    """x <- relu(x)^2 in place over a contiguous bf16 or f32 tensor."""
+    if not x.is_cuda:
+        return x.copy_(x.float().relu().square())
+    assert x.is_contiguous()
+    if x.numel():
+        check(kernels().loqa_relu2_any(ptr(x), _dt(x), x.numel(), ptr(x), stream_ptr(x)), "relu2_any")
+    return x
+
+
+def retention_prep(u: torch.Tensor, H: int, D: int, Dv: int, cos_sin: torch.Tensor | None, dims: int,
+                   positions: torch.Tensor) -> torch.Tensor:
+    """The recurrence inputs of retention from the projected rows u [T, >= 2 H D +
+    H Dv] (q | k | v): q and k rotate pairwise (interleaved layout, the first
+    ``dims`` entries of each head), k also times D^(-1/2) -> f32 [T, 2 H D + H Dv]."""
+    if not u.is_cuda:
+        return ref.retention_prep(u, H, D, Dv, cos_sin, dims, positions)
+    T, n = u.shape[0], 2 * H * D + H * Dv
+    assert u.stride(1) == 1 and u.shape[1] >= n and dims % 2 == 0 and 0 <= dims <= D
+    _i32c(positions, "positions")
+    assert positions.numel() >= T
+    if dims:
+        _f32c(cos_sin, "cos_sin")
+        assert cos_sin.shape[1] * 2 == dims
+    act = torch.empty(T, n, dtype=torch.float32, device=u.device)
+    if T:
+        check(kernels().loqa_retention_prep(
+            ptr(u), _dt(u), u.stride(0), H, D, Dv, ptr(cos_sin) if dims else None,
+            cos_sin.shape[0] if dims else 0, dims, ptr(positions), ptr(act), T, stream_ptr(u)),
+            "retention_prep")
+    return act
+
+
+def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """x W^T with the accumulator's f32 result for operands in either activation
+    dtype (a product that is a residual stream or enters a recurrence)."""
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, w)
+    if not x.is_cuda:
+        return torch.nn.functional.linear(x.float(), w.float())
+    return torch.mm(x, w.t(), out_dtype=torch.float32)
