@@ -10,7 +10,9 @@ sigmoid-routed experts), a Vilulix stack (parallel layers: a matrix memory,
 latent attention with a query latent, sliding-window attention with a sink
 beside a gated delta rule, dense SwiGLU) and a Gopopel stack (parallel layers on
 one norm: sliding-window attention with a distance bias, sliding-window latent
-attention, squared-relu feed-forwards) run beside a Llama stack of the same
+attention, squared-relu feed-forwards) and a Vodalorn stack (a delta rule with a
+decay per key channel, sliding-window attention beside retention, squared-relu
+feed-forwards and clamped experts, per-token side inputs) run beside a Llama stack of the same
 width, depth, head count and feed-forward width - the framework's plain decoder.
 Measured per family:
 
@@ -29,11 +31,11 @@ import time
 import numpy as np
 import torch
 
-from ..models.configs import (ChunkAttnConfig, DeltaRuleConfig, FeedForwardConfig,
+from ..models.configs import (BigramConfig, ChunkAttnConfig, DeltaRuleConfig, FeedForwardConfig,
                               GopopelConfig, HybridLayerConfig, LatentAttnConfig, LightningConfig, LlamaConfig,
                               LoopConfig, Mamba2Config, MatrixMemoryConfig, MovinexConfig,
-                              ParallelMixerConfig, PipizenConfig, RotaryConfig, SodonexConfig,
-                              SoftmaxAttnConfig, VilulixConfig)
+                              ParallelMixerConfig, PipizenConfig, RetentionConfig, RotaryConfig,
+                              SodonexConfig, SoftmaxAttnConfig, VilulixConfig, VodalornConfig)
 
 SIZES = {
     # name: (width, layers, heads, head_dim, rot_dim, kv_rank, ff, experts, expert_ff, top)
@@ -132,6 +134,31 @@ def gopopel_stack(name: str, vocab: int = 32000, window: int = 1024) -> GopopelC
         HybridLayerConfig("attention", att, mlp) for i in range(n)))
 
 
+def vodalorn_stack(name: str, vocab: int = 32000, window: int = 1024) -> VodalornConfig:
+    """Four layers: twice a delta rule with a decay per key channel (the Vilulix
+    stack's heads and taps, low ranks of one head) with a dense squared relu, then
+    sliding-window attention (4 query heads per key/value head, rotary on half a
+    head, biases) beside retention (as many heads as the Llama stack) with clamped
+    experts of the other stacks' sizes; a side input of 256 entries a layer. Layers
+    1 - 2 are entered through the [x ; embedding] projection of a repeated stretch
+    (one pass, so the stack stays four layer runs deep)."""
+    d, n, H, D, Dr, _, ff, E, eff, top = SIZES[name]
+    G = max(1, H // 4)
+    rule = DeltaRuleConfig(H, G, D, D, 4, channel_decay=True)
+    left = SoftmaxAttnConfig(H, G, D, D, D ** -0.5, bias=True, rot=RotaryConfig(Dr, 10000.0, half=True),
+                             window=window, qk_norm="none")
+    ret = RetentionConfig(H, D, D, tuple(1.0 - 2.0 ** (-5.0 - 4.0 * h / H) for h in range(H)),
+                          RotaryConfig(D, 10000.0, half=True))
+    par = ParallelMixerConfig(left, ret, 0.5, 0.5, out_norms=True)
+    dense = FeedForwardConfig("dense", ff, act="relu2")
+    moe = FeedForwardConfig("moe", eff, E, 0, top, 4, 2, act="clamped_glu", limit=7.0, renorm=True,
+                            weight_scale=2.5)
+    return VodalornConfig(f"vodalorn-{name}", vocab, d, 1e-6, 0.5, tuple(
+        HybridLayerConfig("parallel", par, moe) if i % 2 else
+        HybridLayerConfig("channel_delta", rule, dense) for i in range(n)),
+        BigramConfig(16381, 31, 7), 256 if d >= 512 else 8, LoopConfig(1, min(3, n), 1))
+
+
 def llama_stack(name: str, vocab: int = 32000) -> LlamaConfig:
     d, n, H, D, _, _, ff, _, _, _ = SIZES[name]
     return LlamaConfig(f"llama-{name}-stack", d, n, H, max(1, H // 4), D, ff, vocab,
@@ -200,7 +227,8 @@ def run(args) -> int:
     sizes = [s for s in args.lm_sizes.split(",") if s]
     for name in sizes:
         fams = {"pipizen": pipizen_stack, "sodonex": sodonex_stack, "movinex": movinex_stack,
-                "vilulix": vilulix_stack, "gopopel": gopopel_stack, "llama": llama_stack}
+                "vilulix": vilulix_stack, "gopopel": gopopel_stack, "vodalorn": vodalorn_stack,
+                "llama": llama_stack}
         for fam in [f for f in args.lm_families.split(",") if f]:
             cfg = fams[fam](name)
             if dev.type == "cpu":      # plumbing run: tiny stacks
