@@ -349,7 +349,7 @@ class PipizenModel:
         H, D, Dv = m.heads, m.dim, m.vdim
         qkvg = ops.linear(h, L["wqkvg"])
         o = seqmix.lightning_scan(qkvg, H, D, Dv, cache.state[i], meta.state_slots, meta.cu_q,
-                                  meta.positions, L["decay"])
+                                  meta.positions, L["decay"], meta.max_q)
         y = seqmix.gated_rmsnorm(o, L["norm"], qkvg[:, 2 * H * D + H * Dv:], self.cfg.norm_eps,
                                  self.w.dtype)
         return ops.linear(y, L["wo"])

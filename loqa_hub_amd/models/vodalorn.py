@@ -466,7 +466,8 @@ class VodalornModel:
         act = seqmix.retention_prep(u[:, off:off + 2 * H * D + H * Dv], H, D, Dv, L["r_cos_sin"],
                                     m.rot.dims, meta.positions)
         o = seqmix.state_scan(act, H, D, Dv, 0, H * D, 2 * H * D, 1, cache.state[r],
-                              meta.state_slots, meta.cu_q, meta.positions, decay=L["r_decay"])
+                              meta.state_slots, meta.cu_q, meta.positions, decay=L["r_decay"],
+                              max_q=meta.max_q)
         y = seqmix.gated_rmsnorm(o, L["r_norm"], u[:, g_off:g_off + H * Dv], self.cfg.norm_eps,
                                  self.w.dtype, groups=H, gate_act="silu")
         return ops.linear(y, L["r_wo"])

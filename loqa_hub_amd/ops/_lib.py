@@ -261,6 +261,8 @@ _SEQMIX_SIGS = {
                         _vp, _i, _i, _vp, _vp, _vp],
     "loqa_delta_scan": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i,
                         _i, _vp],
+    "loqa_linear_chunks": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
+                           _i, _i, _vp],
     "loqa_retention_prep": [_vp, _i, _l, _i, _i, _i, _vp, _i, _i, _vp, _vp, _i, _vp],
     "loqa_residual_ln": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _f, _vp, _vp, _vp, _f, _vp, _i, _l, _i,
                          _i, _vp],

@@ -340,14 +340,13 @@ def latent_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, cu_q: torc
 
 def lightning_scan(qkv: torch.Tensor, H: int, D: int, Dv: int, state: torch.Tensor,
                    state_slots: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor,
-                   decay: torch.Tensor) -> torch.Tensor:
+                   decay: torch.Tensor, max_q: int = 0) -> torch.Tensor:
     """Decayed linear attention over a flat token batch: per sequence and head
     S <- decay_h S + k v^T, o = S^T q, token by token in f32, with q, k, v the
     SiLU of the first columns of ``qkv`` [T, >= 2 H D + H Dv]. ``state`` [slots,
     H, D, Dv] f32 carries S between steps (a sequence whose first position in
-    this step is 0 starts from zero). Returns o f32 [T, H Dv]. Prompt portions
-    and single decode tokens take the same kernel and the same order of
-    operations, so the result does not depend on how a prompt was cut."""
+    this step is 0 starts from zero). Returns o f32 [T, H Dv]. ``max_q``: see
+    :func:`state_scan`."""
     if not qkv.is_cuda:
         return ref.lightning_scan(qkv, H, D, Dv, state, state_slots, cu_q, positions, decay)
     T = qkv.shape[0]
@@ -365,14 +364,17 @@ def lightning_scan(qkv: torch.Tensor, H: int, D: int, Dv: int, state: torch.Tens
     check(kernels().loqa_lightning_prep(ptr(qkv), _dt(qkv), qkv.stride(0), T, n, ptr(act),
                                         stream_ptr(qkv)), "lightning_prep")
     return state_scan(act, H, D, Dv, 0, H * D, 2 * H * D, 1, state, state_slots, cu_q, positions,
-                      decay=decay)
+                      decay=decay, max_q=max_q)
+
+
+LINEAR_CHUNK = 64        # tokens per chunk of the chunked recurrence (linear_chunks.hip)
 
 
 def state_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: int, v_off: int,
                hpg: int, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
                positions: torch.Tensor, decay: torch.Tensor | None = None,
                tok: torch.Tensor | None = None, skip: torch.Tensor | None = None,
-               col_block: int = 0) -> torch.Tensor:
+               col_block: int = 0, max_q: int = 0, chunked: bool | None = None) -> torch.Tensor:
     """The linear recurrence with a carried matrix state that decayed linear
     attention and Mamba-2 layers share, per sequence and head, token by token
     in f32:  S <- a S + k (c v)^T,  o = S^T q + skip_h v,  with a = ``decay[h]``
@@ -383,7 +385,12 @@ def state_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     one order of operations for prompt portions and single tokens.
     ``col_block`` (8, 16 or 32; 0: chosen from the batch) sets the value columns
     per workgroup: a caller that runs other work beside the scan asks for the
-    denser grid. The result does not depend on it."""
+    denser grid. The result does not depend on it.
+
+    With a constant decay and no skip, steps whose longest feed (``max_q``; 0: not
+    known) has at least two chunks and whose feeds are long on average go chunk by
+    chunk on the f32 matrix cores instead: the same f32 sums in another order.
+    ``chunked`` forces either form."""
     if not act.is_cuda:
         return ref.state_scan(act, H, D, Dv, q_off, k_off, v_off, hpg, state, state_slots, cu_q,
                               positions, decay, tok, skip)
@@ -406,6 +413,14 @@ def state_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     B = state_slots.numel()
     assert cu_q.numel() == B + 1 and positions.numel() >= T
     o = torch.empty(T, H * Dv, dtype=torch.float32, device=act.device)
+    if chunked is None:
+        chunked = max_q >= 2 * LINEAR_CHUNK and T >= 32 * B
+    if chunked and decay is not None and skip is None and T:
+        ws = torch.empty(T // LINEAR_CHUNK + B, H, D, Dv, dtype=torch.float32, device=act.device)
+        check(kernels().loqa_linear_chunks(ptr(act), W, H, D, Dv, q_off, k_off, v_off, hpg, ptr(state),
+                                           ptr(state_slots), ptr(cu_q), ptr(positions), ptr(decay),
+                                           ptr(ws), ptr(o), B, T, stream_ptr(act)), "linear_chunks")
+        return o
     if T:
         check(kernels().loqa_state_scan(ptr(act), W, H, D, Dv, q_off, k_off, v_off, hpg, ptr(state),
                                         state.shape[0], ptr(state_slots), ptr(cu_q), ptr(positions),

@@ -438,6 +438,72 @@ def test_retention_mixer(device, m, cuts):
         close(a, b, 3e-4)
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,hpg,D,Dv,decay", [
+    (3, 1, 8, 10, [0.0, 0.9, 1.0]), (2, 2, 128, 64, [0.97, 0.9995]), (4, 2, 36, 130, [0.5, 0.99, 0.9, 1.0]),
+    (1, 1, 5, 3, [0.93]), (2, 1, 256, 33, [0.99, 0.2]), (1, 1, 72, 256, [0.999])])
+@pytest.mark.parametrize("starts", [(0, 0, 0, 0, 0), (77, 1, 0, 64, 300)])
+def test_chunked_recurrence(H, hpg, D, Dv, decay, starts):
+    """The chunked form on feeds that end on, before and after a chunk's edge (one
+    of them empty, one a single token), from a fresh and from a carried state,
+    against the oracle and the token-by-token kernel; then both go on one token."""
+    lens = (200, 1, 0, 128, 65)
+    B, T, G = len(lens), sum(lens), H // hpg
+    g = torch.Generator().manual_seed(D)
+    q, k = (torch.randn(T, G, D, generator=g) for _ in range(2))
+    v = torch.randn(T, H, Dv, generator=g)
+    act = torch.cat([q.reshape(T, -1), torch.zeros(T, 4), k.reshape(T, -1), v.reshape(T, -1)], 1).cuda()
+    ko = G * D + 4
+    vo = ko + G * D
+    cu, pos = _meta(list(lens), list(starts), "cuda")
+    slots = torch.tensor([4, 0, 5, 2, 1], dtype=torch.int32, device="cuda")
+    state0 = torch.randn(7, H, D, Dv, generator=g)
+    lam = torch.tensor(decay, device="cuda")
+    one = torch.randn(B, act.shape[1], generator=g).cuda()
+    outs = []
+    for chunked in (True, False):
+        st = state0.cuda()
+        o = seqmix.state_scan(act, H, D, Dv, 0, ko, vo, hpg, st, slots, cu, pos, decay=lam,
+                              chunked=chunked)
+        cu1, pos1 = _meta([1] * B, [s + n for s, n in zip(starts, lens)], "cuda")
+        o1 = seqmix.state_scan(one, H, D, Dv, 0, ko, vo, hpg, st, slots, cu1, pos1, decay=lam,
+                               chunked=chunked)
+        outs.append((o, o1, st))
+    a, b = outs
+    for x, y in zip(a, b):
+        close(x, y.double().cpu(), 2e-5)
+    o0 = 0
+    for b_, n in enumerate(lens):
+        S0 = torch.zeros(H, D, Dv, dtype=F64) if starts[b_] == 0 else \
+            state0[int(slots[b_])].double()
+        want = O.retention_scan(q[o0:o0 + n].repeat_interleave(hpg, 1).double(),
+                                k[o0:o0 + n].repeat_interleave(hpg, 1).double(),
+                                v[o0:o0 + n].double(), decay)
+        for t in range(n):
+            for h in range(H):
+                want[t, h] += decay[h] ** (t + 1) * (S0[h].T @ q[o0 + t, h // hpg].double())
+        close(a[0][o0:o0 + n].view(n, H, Dv), want, 2e-5) if n else None
+        o0 += n
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_prompt_takes_the_chunked_form(dtype):
+    """A model whose prompts are long enough for the chunked recurrence."""
+    layers = [(O.parallel(O.window(size=30), O.retention(heads=2, dim=16, vdim=24, rot_dims=16,
+                                                         decay=[0.97, 0.998])), O.dense_ff())]
+    cfg = O.make_config(layers, loop=(0, 1, 2))
+    sd = O.make_weights(cfg, 15)
+    toks = tokens(330, cfg["vocab"], 22)
+    want = O.forward(cfg, sd, toks)
+    eng = engine(cfg, sd, "cuda", dtype, max_tokens=336)
+    for cuts in ([330], [150, 1, 2, 140], [129, 1, 1, 200]):
+        s = eng.open_sequence()
+        got = feed(eng, s, toks, cuts)
+        eng.close_sequence(s)
+        assert rel_err(got, want, 1.0 if dtype == torch.float32 else 0.9) < 2 * TOL[dtype], cuts
+
+
 @pytest.mark.parametrize("device", DEVICES)
 def test_retention_remembers_one_far_key(device):
     """A single key written hundreds of tokens ago, every other key orthogonal to
