@@ -336,7 +336,7 @@ __global__ __launch_bounds__(EC * LPC) void delta_scan_kernel(
           qc[i] = make_float4(w.x * qc[i].x, w.y * qc[i].y, w.z * qc[i].z, w.w * qc[i].w);
         }
       }
-      const float g = gs[tt], bt = bs[tt], vv = vs[tt * EC + e], kq = cs[tt];
+      const float g = CHAN ? 1.f : gs[tt], bt = bs[tt], vv = vs[tt * EC + e], kq = cs[tt];
       float r0 = 0.f, r1 = 0.f, s0 = 0.f, s1 = 0.f;
 #pragma unroll
       for (int i = 0; i < MAXD / 4; ++i) {

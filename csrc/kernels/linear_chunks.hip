@@ -35,34 +35,6 @@ __device__ __forceinline__ float lc_pow(float x, int n) {
   return r;
 }
 
-// The chunk numbered i over all feeds: its sequence, first token and length. All
-// lanes of the wave must be active; false past the last chunk.
-__device__ __forceinline__ bool lc_chunk(const int* __restrict__ cu_q, int B, int i, int& b, int& t0,
-                                         int& n) {
-  const int lane = threadIdx.x & 63;
-  for (int base = 0; base < B; base += 64) {
-    const int s = base + lane;
-    const int lo = s < B ? cu_q[s] : 0, hi = s < B ? cu_q[s + 1] : 0;
-    const int nc = (hi - lo + LC_C - 1) / LC_C;
-    int end = nc;                                    // inclusive prefix sum over the lanes
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const int v = __shfl_up(end, o, 64);
-      if (lane >= o) end += v;
-    }
-    const unsigned long long past = __ballot(end > i);
-    if (past) {
-      const int w = __ffsll(past) - 1;
-      b = base + w;
-      t0 = __shfl(lo, w, 64) + (i - __shfl(end - nc, w, 64)) * LC_C;
-      n = min(LC_C, __shfl(hi, w, 64) - t0);
-      return true;
-    }
-    i -= __shfl(end, 63, 64);
-  }
-  return false;
-}
-
 struct LcParams {
   const float* act; long ld; int H, D, Dv, q_off, k_off, v_off, hpg;
   float* state; const int* slots; const int* cu_q; const int* pos; const float* decay;
@@ -78,10 +50,10 @@ __device__ __forceinline__ float16v lc_zero() {
 // the row of accumulator register r in lane half h
 __device__ __forceinline__ int lc_row(int r, int h) { return (r & 3) + 8 * (r >> 2) + 4 * h; }
 
-__global__ __launch_bounds__(256) void lc_local_kernel(LcParams p) {
+__global__ __launch_bounds__(256, 2) void lc_local_kernel(LcParams p) {
   __shared__ float pw[LC_C];
   int b, t0, n;
-  if (!lc_chunk(p.cu_q, p.B, blockIdx.x, b, t0, n)) return;
+  if (!seq_chunk<LC_C>(p.cu_q, p.B, blockIdx.x, b, t0, n)) return;
   const int h = blockIdx.y, wave = threadIdx.x >> 6, l = threadIdx.x & 31, hf = (threadIdx.x >> 5) & 1;
   if (threadIdx.x < LC_C) pw[threadIdx.x] = lc_pow(p.decay[h], threadIdx.x);
   __syncthreads();
@@ -119,13 +91,10 @@ __global__ __launch_bounds__(256) void lc_local_kernel(LcParams p) {
 
 template <int N>
 __global__ __launch_bounds__(256) void lc_pass_kernel(LcParams p) {
-  const int b = blockIdx.x, h = blockIdx.y, lane = threadIdx.x & 63;
+  const int b = blockIdx.x, h = blockIdx.y;
   const int q0 = p.cu_q[b], len = p.cu_q[b + 1] - q0;
   if (len <= 0) return;
-  int before = 0;                                    // chunks of the sequences before this one
-  for (int s = lane; s < b; s += 64) before += (p.cu_q[s + 1] - p.cu_q[s] + LC_C - 1) / LC_C;
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1) before += __shfl_xor(before, o, 64);
+  const int before = seq_chunks_before<LC_C>(p.cu_q, b);
   const size_t n = (size_t)p.D * p.Dv, i = N * ((size_t)blockIdx.z * 256 + threadIdx.x);
   if (i >= n) return;
   const int nc = (len + LC_C - 1) / LC_C;
@@ -166,13 +135,13 @@ __global__ __launch_bounds__(256) void lc_pass_kernel(LcParams p) {
 #define LC_K 32
 
 template <bool VEC>
-__global__ __launch_bounds__(256) void lc_out_kernel(LcParams p) {
+__global__ __launch_bounds__(256, 2) void lc_out_kernel(LcParams p) {
   constexpr int LD = LC_K + 4;
   __shared__ __attribute__((aligned(16))) float qs[LC_C][LD], ks[LC_C][LD];
   __shared__ __attribute__((aligned(16))) float P[LC_C][LC_C + 4];
   __shared__ float pw[LC_C + 1];
   int b, t0, n;
-  if (!lc_chunk(p.cu_q, p.B, blockIdx.x, b, t0, n)) return;
+  if (!seq_chunk<LC_C>(p.cu_q, p.B, blockIdx.x, b, t0, n)) return;
   const int h = blockIdx.y, wave = threadIdx.x >> 6, l = threadIdx.x & 31, hf = (threadIdx.x >> 5) & 1;
   const int ti = wave >> 1, tj = wave & 1;
   if (threadIdx.x <= LC_C) pw[threadIdx.x] = lc_pow(p.decay[h], threadIdx.x);

@@ -99,4 +99,43 @@ __device__ __forceinline__ void side_relu2(const SideCols& s, size_t t) {
   for (int c = s.n + me; c < s.zero_hi; c += all) Act<T>::st(o + c, 0.f);
 }
 
+// Feeds cut into chunks of C tokens counted from their first one. The chunk
+// numbered i over all feeds: its sequence, first token and length; false past the
+// last chunk. All lanes of the wave must be active.
+template <int C>
+__device__ __forceinline__ bool seq_chunk(const int* __restrict__ cu_q, int B, int i, int& b, int& t0,
+                                          int& n) {
+  const int lane = threadIdx.x & 63;
+  for (int base = 0; base < B; base += 64) {
+    const int s = base + lane;
+    const int lo = s < B ? cu_q[s] : 0, hi = s < B ? cu_q[s + 1] : 0;
+    const int nc = (hi - lo + C - 1) / C;
+    int end = nc;                                    // inclusive prefix sum over the lanes
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int v = __shfl_up(end, o, 64);
+      if (lane >= o) end += v;
+    }
+    const unsigned long long past = __ballot(end > i);
+    if (past) {
+      const int w = __ffsll(past) - 1;
+      b = base + w;
+      t0 = __shfl(lo, w, 64) + (i - __shfl(end - nc, w, 64)) * C;
+      n = min(C, __shfl(hi, w, 64) - t0);
+      return true;
+    }
+    i -= __shfl(end, 63, 64);
+  }
+  return false;
+}
+// the number of chunks of the sequences before b (all lanes active)
+template <int C>
+__device__ __forceinline__ int seq_chunks_before(const int* __restrict__ cu_q, int b) {
+  int c = 0;
+  for (int s = threadIdx.x & 63; s < b; s += 64) c += (cu_q[s + 1] - cu_q[s] + C - 1) / C;
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) c += __shfl_xor(c, o, 64);
+  return c;
+}
+
 static inline int ceil_div(long a, long b) { return (int)((a + b - 1) / b); }

@@ -87,7 +87,8 @@ def _build_lib(name: str, sources: list[str], headers: list[str], flags: list[st
 SEQMIX_SOURCES = ("norm_dyt.hip", "attn_latent.hip", "attn_latent_prefill.hip", "lightning.hip",
                   "moe.hip", "seq_rows.hip", "norm_scalar.hip", "attn_sigmoid.hip",
                   "norm_rms1p.hip", "attn_window.hip", "mamba2.hip", "matrix_memory.hip",
-                  "delta_rule.hip", "norm_layer.hip", "linear_chunks.hip")
+                  "delta_rule.hip", "norm_layer.hip", "linear_chunks.hip",
+                  "delta_chunks.hip")
 
 # hipcc may not form packed-f32 VALU instructions from scalar float code
 NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]

@@ -483,7 +483,8 @@ class VilulixModel:
             # every reader of this step's tail is done: store the new rows
             seqmix.seq_state_save(None, u, None, tail, meta.state_slots, meta.cu_q, meta.positions)
         o = seqmix.delta_scan(act, H, D, Dv, 0, G * D, 2 * G * D, H // G, cache.state[r],
-                              meta.state_slots, meta.cu_q, meta.positions, tok)
+                              meta.state_slots, meta.cu_q, meta.positions, tok,
+                              max_q=meta.max_q)
         y = seqmix.gated_rmsnorm(o, L["r_norm"], u[:, C:C + H * Dv], self.cfg.norm_eps,
                                  self.w.dtype, groups=H, gate_act="silu")
         return ops.linear(y, L["r_wo"])

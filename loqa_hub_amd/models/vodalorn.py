@@ -429,7 +429,8 @@ class VodalornModel:
             # every reader of this step's tail is done: store the new rows
             seqmix.seq_state_save(None, u, None, tail, meta.state_slots, meta.cu_q, meta.positions)
         o = seqmix.delta_scan(act, H, D, Dv, 0, G * D, 2 * G * D, H // G, cache.state[r],
-                              meta.state_slots, meta.cu_q, meta.positions, tok, g_off=C)
+                              meta.state_slots, meta.cu_q, meta.positions, tok, g_off=C,
+                              max_q=meta.max_q)
         y = seqmix.gated_rmsnorm(o, L["norm"], gate, self.cfg.norm_eps, self.w.dtype, groups=H)
         return [(ops.linear(y, L["wo"]), None)]
 

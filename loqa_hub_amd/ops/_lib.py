@@ -263,6 +263,8 @@ _SEQMIX_SIGS = {
                         _i, _vp],
     "loqa_linear_chunks": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
                            _i, _i, _vp],
+    "loqa_delta_chunks": [_vp, _l, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _vp,
+                          _vp, _i, _i, _vp],
     "loqa_retention_prep": [_vp, _i, _l, _i, _i, _i, _vp, _i, _i, _vp, _vp, _i, _vp],
     "loqa_residual_ln": [_vp, _vp, _vp, _vp, _vp, _vp, _i, _f, _vp, _vp, _vp, _f, _vp, _i, _l, _i,
                          _i, _vp],
@@ -319,7 +321,7 @@ class _Kernels:
     ``libloqa_kernels.so`` (loaded only when one of its kernels is called)."""
 
     def __getattr__(self, name: str):
-        if name in _SEQMIX_SIGS:
+        if name in _SEQMIX_SIGS or name == "loqa_delta_chunks_ws":
             fn = getattr(seqmix(), name)
         else:
             fn = getattr(_main_kernels(), name)
@@ -337,6 +339,8 @@ def seqmix() -> ctypes.CDLL:
                     f = getattr(lib, fn)
                     f.argtypes = sig
                     f.restype = c_int
+                lib.loqa_delta_chunks_ws.argtypes = [c_int] * 5
+                lib.loqa_delta_chunks_ws.restype = c_ll
                 _seqmix = lib
     return _seqmix
 

@@ -1178,10 +1178,13 @@ def delta_prep(u: torch.Tensor, gz: torch.Tensor, G: int, D: int, H: int, Dv: in
     return act, tok
 
 
+DELTA_CHUNK = 16         # tokens per chunk of the chunked delta rule (delta_chunks.hip)
+
+
 def delta_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: int, v_off: int,
                hpg: int, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
-               positions: torch.Tensor, tok: torch.Tensor, g_off: int | None = None
-               ) -> torch.Tensor:
+               positions: torch.Tensor, tok: torch.Tensor, g_off: int | None = None,
+               max_q: int = 0, chunked: bool | None = None) -> torch.Tensor:
     """The gated delta rule with a carried matrix state, per sequence and head,
     token by token in f32:  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;
     o = S^T q, with (g, beta) = ``tok[t, h]``; with ``g_off`` g is a vector over the
@@ -1189,8 +1192,10 @@ def delta_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     q at ``q_off + (h // hpg) D``, k at ``k_off + (h // hpg) D`` and v at
     ``v_off + h Dv``. ``state`` [slots, H, Dv, D] f32 (a column's rows side by
     side) carries S between steps (zero when the step's first position is 0).
-    One kernel and one order of operations for prompt portions and single
-    tokens."""
+
+    Steps whose longest feed (``max_q``; 0: not known) has at least four chunks and
+    whose feeds are long on average go chunk by chunk on the f32 matrix cores: the
+    same f32 sums in another order. ``chunked`` forces either form."""
     if not act.is_cuda:
         return ref.delta_scan(act, H, D, Dv, q_off, k_off, v_off, hpg, state, state_slots, cu_q,
                               positions, tok, g_off)
@@ -1202,6 +1207,17 @@ def delta_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     assert min(q_off, k_off, v_off) >= 0 and max(q_off, k_off) + G * D <= W and v_off + H * Dv <= W
     B = _seq_args(state_slots, cu_q, positions, T)
     o = torch.empty(T, H * Dv, dtype=torch.float32, device=act.device)
+    if chunked is None:
+        chunked = max_q >= 4 * DELTA_CHUNK and T >= 2 * DELTA_CHUNK * B
+    if chunked and T:
+        k = kernels()
+        ws = torch.empty(k.loqa_delta_chunks_ws(H, D, Dv, B, T), dtype=torch.float32,
+                         device=act.device)
+        check(k.loqa_delta_chunks(ptr(act), W, H, D, Dv, q_off, k_off, v_off,
+                                  -1 if g_off is None else g_off, hpg, ptr(state), ptr(state_slots),
+                                  ptr(cu_q), ptr(positions), ptr(tok), ptr(ws), ptr(o), B, T,
+                                  stream_ptr(act)), "delta_chunks")
+        return o
     if T:
         check(kernels().loqa_delta_scan(ptr(act), W, H, D, Dv, q_off, k_off, v_off,
                                         -1 if g_off is None else g_off, hpg, ptr(state),

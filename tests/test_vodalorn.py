@@ -489,10 +489,11 @@ def test_chunked_recurrence(H, hpg, D, Dv, decay, starts):
 @pytest.mark.gpu
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_long_prompt_takes_the_chunked_form(dtype):
-    """A model whose prompts are long enough for the chunked recurrence."""
-    layers = [(O.parallel(O.window(size=30), O.retention(heads=2, dim=16, vdim=24, rot_dims=16,
+    """A model whose prompts are long enough for the chunked recurrences."""
+    layers = [(O.delta(heads=4, kv_heads=2, dim=20, vdim=12), None),
+              (O.parallel(O.window(size=30), O.retention(heads=2, dim=16, vdim=24, rot_dims=16,
                                                          decay=[0.97, 0.998])), O.dense_ff())]
-    cfg = O.make_config(layers, loop=(0, 1, 2))
+    cfg = O.make_config(layers, loop=(0, 2, 2))
     sd = O.make_weights(cfg, 15)
     toks = tokens(330, cfg["vocab"], 22)
     want = O.forward(cfg, sd, toks)
@@ -613,6 +614,66 @@ def test_delta_inputs_with_channel_decays_bf16(device, G, D, H, Dv, K):
         assert (act.cpu().double() - want[at:at + n]).abs().max() < 2e-5
         assert (tok[:, :, 1].cpu().double() - beta[at:at + n]).abs().max() < 1e-5
         at += n
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("chan", [True, False])
+@pytest.mark.parametrize("H,hpg,D,Dv", [(3, 1, 8, 10), (4, 2, 128, 64), (2, 2, 36, 33), (1, 1, 5, 3),
+                                        (2, 1, 200, 40), (1, 1, 256, 16), (2, 1, 64, 128)])
+@pytest.mark.parametrize("starts", [(0, 0, 0, 0, 0), (77, 1, 0, 64, 300)])
+def test_chunked_delta_rule(chan, H, hpg, D, Dv, starts):
+    """The chunked form on feeds that end on, before and after a chunk's edge (one
+    of them empty, one a single token), from a fresh and from a carried state,
+    against the oracle; decays of 0, of almost 0 and of 1 among them, write
+    strengths up to 1, one key repeated many times."""
+    lens = (70, 1, 0, 32, 17)
+    B, T, G = len(lens), sum(lens), H // hpg
+    g = torch.Generator().manual_seed(D + chan)
+    q, k = (torch.randn(T, G, D, generator=g) for _ in range(2))
+    k[20:31] = k[20]
+    q, k = q / q.norm(dim=-1, keepdim=True), k / k.norm(dim=-1, keepdim=True)
+    v = torch.randn(T, H, Dv, generator=g)
+    dec = torch.rand(T, H, D, generator=g) ** 0.1
+    dec[:, :, 0], dec[::7, :, 1] = 1.0, 0.0
+    dec[::3, :, 2] = 1e-30
+    beta = torch.rand(T, H, generator=g)
+    beta[20:31] = 1.0
+    if not chan:
+        dec = dec[:, :, 3:4].expand(T, H, D).contiguous()
+        dec[40], dec[45] = 0.0, 1e-30
+    act = torch.cat([q.reshape(T, -1), k.reshape(T, -1), torch.zeros(T, 3), v.reshape(T, -1)] +
+                    ([dec.reshape(T, -1)] if chan else []), 1).cuda()
+    vo = 2 * G * D + 3
+    go = vo + H * Dv if chan else None
+    tok = torch.stack([torch.full((T, H), 7.0) if chan else dec[:, :, 0], beta], -1).cuda()
+    cu, pos = _meta(list(lens), list(starts), "cuda")
+    slots = torch.tensor([4, 0, 5, 2, 1], dtype=torch.int32, device="cuda")
+    state0 = torch.randn(7, H, Dv, D, generator=g) * 0.5
+    outs = []
+    for chunked in (True, False):
+        st = state0.cuda()
+        outs.append((seqmix.delta_scan(act, H, D, Dv, 0, G * D, vo, hpg, st, slots, cu, pos, tok,
+                                       g_off=go, chunked=chunked), st))
+    for x, y in zip(*outs):
+        close(x, y.double().cpu(), 3e-5)
+    o0 = 0
+    rep = lambda x: x.repeat_interleave(hpg, 1)
+    for b, n in enumerate(lens):
+        if not n:
+            continue
+        sl = slice(o0, o0 + n)
+        o0 += n
+        S = torch.zeros(H, D, Dv, dtype=F64) if starts[b] == 0 else \
+            state0[int(slots[b])].transpose(1, 2).double()
+        want = torch.zeros(n, H, Dv, dtype=F64)
+        for t in range(n):
+            kt, qt = rep(k)[sl][t].double(), rep(q)[sl][t].double()
+            S = S * dec[sl][t].double()[:, :, None]
+            u = beta[sl][t].double()[:, None] * (v[sl][t].double() - torch.einsum("hde,hd->he", S, kt))
+            S = S + kt[:, :, None] * u[:, None, :]
+            want[t] = torch.einsum("hde,hd->he", S, qt)
+        close(outs[0][0][sl].view(n, H, Dv), want, 3e-5)
+        close(outs[0][1][int(slots[b])].transpose(1, 2), S, 3e-5)
 
 
 @pytest.mark.parametrize("device", DEVICES)
