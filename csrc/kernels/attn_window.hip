@@ -45,10 +45,11 @@
 // contexts the windows are also dealt out to several workgroups per row, whose
 // partial triples a small combine launch merges.
 //
-// window_attn_mfma_kernel (bf16, D and Dv up to 256 in multiples of 8,
+// window_attn_mfma_kernel (bf16, D up to 256 and Dv up to 512 in multiples of 8,
 // padded with zeros in LDS to the next built size; prompt portions): a
-// workgroup per (64, 128 or 256 query rows of one sequence, query head); each
-// wave owns 32 rows. The block-table entries of the key range go to LDS once.
+// workgroup per (64, 128 or 256 query rows of one sequence, query head, up to 128
+// of its value columns: wider values are shared out, every part forming the scores
+// again); each wave owns 32 rows. The block-table entries of the key range go to LDS once.
 // K and V tiles of 64 keys are gathered from the pages into LDS for all waves
 // (the next tile's 16-byte chunks already in flight in registers);
 // S^T = K Q^T and O^T += V^T P^T run on v_mfma_f32_32x32x16_bf16 with the query
@@ -66,6 +67,7 @@ struct WinAttnParams {
   const float* sink;                 // [H] or null: exp(sink[h]) joins head h's softmax denominator
   const float* slopes;               // [H] or null: slopes[h] * (i - j) comes off head h's score
   long o_ld;                         // row stride of o (head h at column h * Dv)
+  int vparts;                        // matrix-core form: workgroups that share a head's value columns
 };
 
 // K / V pages (and the block table) are read through pointers in the global
@@ -587,8 +589,8 @@ __device__ __forceinline__ float tanh_fast(float z) {
   return 1.f - 2.f * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.885390081777927f * z));
 }
 
-// DK, DV: the sizes in LDS and registers. PAD: the model's sizes p.D <= DK and
-// p.Dv <= DV are smaller (multiples of 8); the rest is zero.
+// DK, DV: the sizes in LDS and registers. PAD: the model's key size p.D <= DK or the
+// workgroup's value columns (<= DV) are fewer (multiples of 8); the rest is zero.
 template <int DK, int DV, int WM_WAVES, bool PAD>
 __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttnParams p) {
   __shared__ __attribute__((aligned(16))) WinMfmaSmem<DK, DV> sm;
@@ -596,9 +598,10 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
   constexpr int WM_THREADS = 64 * WM_WAVES;
   constexpr int NS = DK / 16, NDT = DV / 32;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = lane >> 5;
-  const int head = blockIdx.y, b = blockIdx.z;
+  const int head = (int)blockIdx.y / p.vparts, b = blockIdx.z;
+  const int v0 = ((int)blockIdx.y % p.vparts) * DV;    // this workgroup's value columns
   const int g = head / (p.H / p.G);
-  const int D = PAD ? p.D : DK, Dv = PAD ? p.Dv : DV;
+  const int D = PAD ? p.D : DK, Dv = PAD ? min(DV, p.Dv - v0) : DV;
   const int q0 = p.cu_q[b], qlen = p.cu_q[b + 1] - q0;
   // long row blocks (the most keys) start first
   const int nblk = (int)gridDim.x;
@@ -639,9 +642,9 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     for (int j = 0; j < 16; ++j) acc[i][j] = 0.f;
   float m_run = -1e30f, l_run = 0.f;
   constexpr int CHK = DK / 8, CHV = DV / 8;
-  const size_t kst = (size_t)p.G * D, vst = (size_t)p.G * Dv;
+  const size_t kst = (size_t)p.G * D, vst = (size_t)p.G * p.Dv;
   const WA_GLOBAL bf16_t* kbase = (const WA_GLOBAL bf16_t*)p.kc + (size_t)g * D;
-  const WA_GLOBAL bf16_t* vbase = (const WA_GLOBAL bf16_t*)p.vc + (size_t)g * Dv;
+  const WA_GLOBAL bf16_t* vbase = (const WA_GLOBAL bf16_t*)p.vc + (size_t)g * p.Dv + v0;
   const WA_GLOBAL int* bt = (const WA_GLOBAL int*)p.bt + (size_t)b * p.max_blocks;
   // the pages of this workgroup's key range, looked up once
   const int npg = (kend + p.blk - 1) / p.blk;
@@ -804,8 +807,9 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     const float a = __builtin_amdgcn_exp2f(m_run - mx2);
     inv = a / (l_run * a + __builtin_amdgcn_exp2f(sl - mx2));
   }
-  bf16_t* orow = (bf16_t*)p.o + (size_t)(q0 + qi) * p.o_ld + (size_t)head * Dv;
-  const bf16_t* grow = p.gate ? (const bf16_t*)p.gate + (size_t)(q0 + qi) * p.gate_ld + (size_t)head * Dv
+  bf16_t* orow = (bf16_t*)p.o + (size_t)(q0 + qi) * p.o_ld + (size_t)head * p.Dv + v0;
+  const bf16_t* grow = p.gate ? (const bf16_t*)p.gate + (size_t)(q0 + qi) * p.gate_ld +
+                                    (size_t)head * p.Dv + v0
                               : nullptr;
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
@@ -830,16 +834,18 @@ __global__ __launch_bounds__(64 * WM_WAVES) void window_attn_mfma_kernel(WinAttn
     }
 }
 
-int window_attention_mfma(const WinAttnParams& p, int max_q, hipStream_t st) {
+int window_attention_mfma(const WinAttnParams& p0, int max_q, hipStream_t st) {
   if (max_q <= 0) return 0;
+  WinAttnParams p = p0;
+  p.vparts = (p.Dv + 127) / 128;
   // the widest row block the longest feed fills: the tiles' staging (gather
   // through the page table, LDS stores, barriers) is paid once per block and
   // tile, and measured times fall with the block width even when the grid
   // shrinks below the number of compute units
   const int waves = max_q > 128 ? 8 : (max_q > 64 ? 4 : 2);
-  const dim3 grid((max_q + waves * 32 - 1) / (waves * 32), p.H, p.B);
+  const dim3 grid((max_q + waves * 32 - 1) / (waves * 32), p.H * p.vparts, p.B);
 #define GO(A, C)                                                                              \
-  if (p.D == A && p.Dv == C) {                                                                \
+  if (p.D == A && (p.Dv == C || (C == 128 && p.Dv % C == 0))) {                                                              \
     if (waves == 8)                                                                           \
       hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 8, false>), grid, dim3(512), 0, st, p); \
     else if (waves == 4)                                                                      \
@@ -850,25 +856,10 @@ int window_attention_mfma(const WinAttnParams& p, int max_q, hipStream_t st) {
   }
   GO(64, 64) GO(128, 64) GO(64, 128) GO(128, 128)
 #undef GO
-  // values of more than 128 entries: the accumulators alone take half the
-  // registers of a wave that has its SIMD for itself (4 waves per workgroup)
-#define GO(A, C, PADDED)                                                                      \
-  do {                                                                                        \
-    hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 4, PADDED>),                            \
-                       dim3((max_q + 127) / 128, p.H, p.B), dim3(256), 0, st, p);             \
-    return (int)hipGetLastError();                                                            \
-  } while (0)
-  if (p.Dv > 128) {
-    if (p.D == 128 && p.Dv == 256) GO(128, 256, false);
-    else if (p.D <= 128 && p.Dv <= 256) GO(128, 256, true);
-    else if (p.D <= 256 && p.Dv <= 256) GO(256, 256, true);
-    return (int)hipErrorInvalidValue;
-  }
-#undef GO
   // other sizes: the next built size, in two block widths
-  const dim3 grid_p = waves == 8 ? grid : dim3((max_q + 63) / 64, p.H, p.B);
+  const dim3 grid_p = waves == 8 ? grid : dim3((max_q + 63) / 64, p.H * p.vparts, p.B);
 #define GO(A, C)                                                                              \
-  if (p.D <= A && p.Dv <= C) {                                                                \
+  if (p.D <= A && (p.Dv <= C || C == 128)) {                                                              \
     if (waves == 8)                                                                           \
       hipLaunchKernelGGL((window_attn_mfma_kernel<A, C, 8, true>), grid_p, dim3(512), 0, st, p); \
     else                                                                                      \
@@ -945,11 +936,11 @@ extern "C" int loqa_window_attention(const void* q, int dt, const void* kc, cons
   p.scale = scale; p.cap = cap; p.window = window; p.keep_first = keep_first;
   p.B = B; p.T = T; p.H = H; p.G = G; p.D = D; p.Dv = Dv; p.o = o;
   p.ns = 1; p.part = nullptr; p.sink = (const float*)sink;
-  p.slopes = (const float*)slopes; p.o_ld = o_ld;
+  p.slopes = (const float*)slopes; p.o_ld = o_ld; p.vparts = 1;
   // the matrix-core form reads the gate and writes the output in 8-byte runs
   const bool runs_ok = (!gate || (gate_ld % 4 == 0 && ((size_t)gate & 7) == 0)) && o_ld % 4 == 0 &&
                        ((size_t)o & 7) == 0;
-  if (mfma && dt == 0 && D % 8 == 0 && D <= 256 && Dv % 8 == 0 && Dv <= 256 && runs_ok)
+  if (mfma && dt == 0 && D % 8 == 0 && D <= 256 && Dv % 8 == 0 && Dv <= 512 && runs_ok)
     return window_attention_mfma(p, max_q, st);
   const int rep = H / G;
   // value layout: whole rows in 16-byte runs when Dv / (elements per run) is a

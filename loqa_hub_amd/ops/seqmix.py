@@ -381,8 +381,7 @@ def state_scan(act: torch.Tensor, H: int, D: int, Dv: int, q_off: int, k_off: in
     or per token ``tok[t, h, 0]`` and c = 1 or ``tok[t, h, 1]``. ``act`` f32
     [T, W]: head h reads q at ``q_off + (h // hpg) D``, k at ``k_off + (h // hpg)
     D`` and v at ``v_off + h Dv``. ``state`` [slots, H, D, Dv] f32 carries S
-    between steps (zero when the step's first position is 0). One kernel and
-    one order of operations for prompt portions and single tokens.
+    between steps (zero when the step's first position is 0).
     ``col_block`` (8, 16 or 32; 0: chosen from the batch) sets the value columns
     per workgroup: a caller that runs other work beside the scan asks for the
     denser grid. The result does not depend on it.
@@ -854,9 +853,10 @@ def qk_prep_append(u: torch.Tensor, H: int, G: int, D: int, Dv: int, v_off: int,
 
 
 def window_mfma_sizes(D: int, Dv: int) -> bool:
-    """Head sizes the matrix-core form covers (built for 64 / 128 / 256 both ways;
-    multiples of 8 in between are padded with zeros in LDS)."""
-    return D % 8 == 0 and 0 < D <= 256 and Dv % 8 == 0 and 0 < Dv <= 256
+    """Head sizes the matrix-core form covers (keys built for 64 / 128 / 256, values
+    for 64 / 128 and shared out over workgroups above; multiples of 8 in between are
+    padded with zeros in LDS)."""
+    return D % 8 == 0 and 0 < D <= 256 and Dv % 8 == 0 and 0 < Dv <= 512
 
 
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
