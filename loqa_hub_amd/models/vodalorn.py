@@ -114,7 +114,10 @@ class VodalornWeights:
                 if f.kind == "dense":
                     L["w_up"], L["w_down"] = W(q + "up", f.ff, d), W(q + "down", d, f.ff)
                 else:
-                    L["router"] = F(q + "router", f.experts, d)
+                    # f32 products of 16-bit values are exact: a router stored in
+                    # 16 bits needs no f32 copy for f32 logits
+                    L["router"] = (W if sd[q + "router"].dtype == torch.bfloat16 else F)(
+                        q + "router", f.experts, d)
                     L["e_gate_up"] = torch.stack([
                         torch.cat([W(f"{q}e{e}.gate", f.ff, d), W(f"{q}e{e}.up", f.ff, d)])
                         for e in range(f.experts)]).contiguous()
@@ -479,7 +482,8 @@ class VodalornModel:
 
     @staticmethod
     def _moe(f, L, h) -> torch.Tensor:
-        z = ops.linear(h.float(), L["router"])
+        rw = L["router"]
+        z = seqmix.linear_f32(h if rw.dtype == h.dtype else h.float(), rw)
         idx, wt = seqmix.moe_route(z, None, f.groups, f.keep, f.top, group_rank=f.group_rank,
                                    renorm=f.renorm, weight_scale=f.weight_scale)
         return seqmix.moe_experts(h, idx, wt, L["e_gate_up"], L["e_down"], limit=f.limit)
