@@ -38,7 +38,8 @@
 // staged TC at a time in LDS (rows zero-padded to 16 MAXD), the next group's
 // values already in flight in registers. The recurrence runs token by token
 // in f32; a prompt portion, a single token or any cut of a prompt is the same
-// sequence of operations, for any EC.
+// sequence of operations, for any EC. (Long feeds take the chunked form of
+// delta_chunks.hip instead.)
 #include "seqmix.h"
 #include <type_traits>
 

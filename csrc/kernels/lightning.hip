@@ -30,7 +30,8 @@
 // and the 16 row-partials of o_t are written to LDS and summed in a fixed
 // order after each group. A prompt portion, a single decode token, or any cut
 // of a prompt gives the same bits (for a given EC: the column split does not
-// change any sum).
+// change any sum). (Long feeds with a constant decay take the chunked form of
+// linear_chunks.hip instead.)
 #include "seqmix.h"
 #include <type_traits>
 

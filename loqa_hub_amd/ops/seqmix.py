@@ -13,7 +13,8 @@ As everywhere in ``ops``: GPU tensors run the HIP kernels
 (``csrc/kernels/norm_dyt.hip``, ``attn_latent.hip``, ``lightning.hip``,
 ``moe.hip``, ``seq_rows.hip``, ``attn_sigmoid.hip``, ``norm_scalar.hip``,
 ``norm_rms1p.hip``, ``attn_window.hip``, ``mamba2.hip``, ``matrix_memory.hip``,
-``delta_rule.hip``, ``norm_layer.hip``), CPU tensors the f32
+``delta_rule.hip``, ``norm_layer.hip``, ``linear_chunks.hip``,
+``delta_chunks.hip``), CPU tensors the f32
 PyTorch references (the CPU test tier and the numerics oracle of the GPU
 tests). Activations are bfloat16 or float32
 (``_DT``); the residual stream, scores, softmax, recurrent state, router and

@@ -431,7 +431,8 @@ CUTS = [[37], [1], [2, 1, 3, 17, 1, 13]]
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("cuts", CUTS, ids=lambda c: str(len(c)))
 @pytest.mark.parametrize("m", [O.retention(), O.retention(1, 5, 3, 2, decay=[1.0]),
-                               O.retention(2, 64, 128, 64), O.retention(2, 72, 31, 0, decay=[0.0, 0.99]),
+                               O.retention(2, 64, 128, 64),
+                               O.retention(2, 72, 31, 0, decay=[0.0, 0.99]),
                                O.retention(4, 16, 8, 16)], ids=lambda m: f"{m['dim']}x{m['vdim']}")
 def test_retention_mixer(device, m, cuts):
     got, want = _retention_case(device, m, cuts)
@@ -723,7 +724,8 @@ def test_router(device, E, groups, keep, top, scale):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("T,d,ff,E,top", [(37, 32, 40, 6, 2), (3, 24, 20, 5, 5), (2, 64, 8, 3, 1), (400, 64, 96, 4, 3)])
+@pytest.mark.parametrize("T,d,ff,E,top", [(37, 32, 40, 6, 2), (3, 24, 20, 5, 5), (2, 64, 8, 3, 1),
+                                           (400, 64, 96, 4, 3)])
 def test_clamped_experts(device, dtype, T, d, ff, E, top):
     """Gate and up products beyond the limit on both sides."""
     g = torch.Generator().manual_seed(T)
