@@ -182,7 +182,10 @@ def _run_chunked(chunk: str, pipelined: bool, monkeypatch):
     from loqa_hub_amd.models.configs import llama_config
     monkeypatch.setenv("LOQA_CHUNK_PREFILL", chunk)
     monkeypatch.setenv("LOQA_INLINE_PREFILL", "0")     # every arrival takes a prompt pass
-    eng = LLMEngine(llama_config("test-tiny"), torch.device("cpu"), seed=0, max_seqs=6,
+    # which tokens share a step depends on when the second batch arrives, and with
+    # that the rounding of the 16-bit products: these weights have no argmax so
+    # close that another batch composition turns it
+    eng = LLMEngine(llama_config("test-tiny"), torch.device("cpu"), seed=1, max_seqs=6,
                     max_seq_len=512, use_graphs=False)
     eng.pipelined = pipelined
     texts = ["turn on the lights and play music", "dim the kitchen lights", "hello there",

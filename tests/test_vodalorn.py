@@ -345,8 +345,8 @@ def test_window_edges(device, back):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("H,G,D,Dv,window", [(4, 2, 128, 256, 48), (6, 2, 64, 160, 200), (2, 1, 256, 256, 70),
-                                             (3, 3, 200, 136, 33), (8, 1, 128, 256, 1000), (2, 1, 64, 512, 90),
-                                             (2, 2, 40, 328, 64)])
+                                             (3, 3, 200, 136, 33), (8, 1, 128, 256, 1000),
+                                             (2, 1, 64, 512, 90), (2, 2, 40, 328, 64)])
 def test_wide_values_on_matrix_cores(H, G, D, Dv, window):
     """The prompt-portion kernel with more than 128 value entries against the
     oracle and against the keys-parallel form."""
